@@ -7,26 +7,11 @@
 
 namespace lsh {
 
-static thread_local std::string g_last_error;
-
-int lsh_fail(int code, const char* msg) {
-  g_last_error = msg ? msg : "";
-  return code;
-}
-
-int lsh_check_hip(hipError_t e, const char* what) {
-  if (e == hipSuccess) return LSH_OK;
-  g_last_error = std::string(what ? what : "hip") + ": " + hipGetErrorName(e) + " " +
-                 hipGetErrorString(e);
-  return LSH_ERR_HIP;
-}
-
-int lsh_check_launch(const char* what) { return lsh_check_hip(hipGetLastError(), what); }
 
 static int no_col32(int flag_a, int flag_b, const char* who) {
   if (flag_a || flag_b) {
-    g_last_error = std::string(who) + ": COL32 layouts are cuBLASLt-specific and not provided";
-    return LSH_ERR_UNSUPPORTED;
+    const std::string msg = std::string(who) + ": COL32 layouts are cuBLASLt-specific and not provided";
+    return lsh_fail(LSH_ERR_UNSUPPORTED, msg.c_str());
   }
   return LSH_OK;
 }
@@ -62,9 +47,6 @@ using namespace lsh;
 #define FM(p) reinterpret_cast<float*>(p)
 
 extern "C" {
-
-const char* lsh_last_error(void) { return g_last_error.c_str(); }
-const char* lsh_version(void) { return "lightseq_hip 0.1 (gfx950)"; }
 
 // ---- quantise / dequantise ------------------------------------------------------
 int lsh_launch_quantize_tensor_f16(const void* input, int8_t* output, int batch_tokens,

@@ -1270,31 +1270,9 @@ static thread_local hipEvent_t g_ev_start = nullptr, g_ev_stop = nullptr;
 static std::atomic<bool> g_tile_kernel_enabled{true};
 // the same for the two decode-step kernels (tests compare them bit for bit)
 static std::atomic<bool> g_skinny16_enabled{true};
-static std::atomic<unsigned long> g_route_epoch{0};
-
-unsigned long route_epoch() { return g_route_epoch.load(std::memory_order_acquire); }
-void route_epoch_bump() { g_route_epoch.fetch_add(1, std::memory_order_acq_rel); }
-
 void gemm_i8_time_next_launch(hipEvent_t start, hipEvent_t stop) {
   g_ev_start = start;
   g_ev_stop = stop;
-}
-
-// Compute units of the current device (256 on MI355X), read once per device: the choices below
-// reason in rounds of the chip -- one, two or three resident workgroups per compute unit.
-int cu_count() {
-  static std::mutex mu;
-  static int cached[64] = {};
-  int dev = 0;
-  if (hipGetDevice(&dev) != hipSuccess || dev < 0 || dev >= 64) return 256;
-  std::lock_guard<std::mutex> lock(mu);
-  if (cached[dev] == 0) {
-    int n = 0;
-    if (hipDeviceGetAttribute(&n, hipDeviceAttributeMultiprocessorCount, dev) != hipSuccess || n <= 0)
-      n = 256;
-    cached[dev] = n;
-  }
-  return cached[dev];
 }
 
 static bool stream_ok(int M, int N, int K) {

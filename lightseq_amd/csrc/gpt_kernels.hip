@@ -551,19 +551,6 @@ int gpt_greedy_step(const int8_t* logits, int* ids, int* last_ids, int vocab_siz
 // counter = (draw, 0, row, 0), word 0) mapped to (0, 1] as curand_uniform maps 32 bits, with
 // the state {seed, row, draws} per sequence in device memory, advanced by the kernel.
 // ---------------------------------------------------------------------------------
-__global__ void sample_state_setup_kernel(SampleState* st, int n, unsigned long long seed) {
-  const int i = blockIdx.x * blockDim.x + threadIdx.x;
-  if (i < n) st[i] = SampleState{seed, (unsigned)i, 0u};
-}
-
-int sample_state_setup(void* state, int n, unsigned long long seed, hipStream_t s) {
-  if (!state || n <= 0 || (reinterpret_cast<uintptr_t>(state) & 15u) != 0)
-    return lsh_fail(LSH_ERR_INVALID, "rng_setup: needs a 16-byte aligned state array");
-  sample_state_setup_kernel<<<(n + 255) / 256, 256, 0, s>>>(static_cast<SampleState*>(state), n,
-                                                            seed);
-  return lsh_check_launch("sample_state_setup_kernel");
-}
-
 // The 16 consecutive ids a thread reads per piece belong to 16 classes that do not change from
 // piece to piece (16 * 1024 is a multiple of 1024), so a thread reduces in registers and
 // touches LDS 16 times at the end.  f(e, v, c): slot e of the thread, id v, code c.

@@ -6,12 +6,13 @@
 #include <memory>
 
 #include "ls_model.h"
+#include "model_controls.h"
 #include "quant_bert_encoder.h"
 
 namespace lightseq {
 namespace hip {
 
-class QuantBert : public LSModel {
+class QuantBert : public LSModel, public EncoderControls {
  public:
   QuantBert(const std::string weight_path, const int max_batch_size);
   ~QuantBert();
@@ -19,6 +20,15 @@ class QuantBert : public LSModel {
   void Infer() override;
   void benchmark_mode(bool) override {}
   void* get_stream() override { return stream_.get(); }
+
+  void set_profiling(bool on) override {
+    encoder_->set_profiling(on);
+    encoder_->reset_profile();
+  }
+  std::string profile_json() override { return encoder_->profile_json(); }
+  bool set_encoder_tap(int layer, const std::string& name, void* dst) override {
+    return encoder_->set_tap(layer, name, dst);
+  }
 
   QuantBertEncoder* encoder() { return encoder_.get(); }
   const QuantBertWeight& weight() const { return tw_; }

@@ -401,5 +401,35 @@ void QuantBertEncoder::ffn_add_norm() {
   }
 }
 
+std::string QuantBertEncoder::profile_json() const {
+  std::string out = "[";
+  for (const auto& p : _profile) {
+    if (out.size() > 1) out += ",";
+    out += "{\"site\":\"" + p.site + "\",\"kernel\":\"" + p.kernel + "\",\"m\":" +
+           std::to_string(p.m) + ",\"n\":" + std::to_string(p.n) + ",\"k\":" +
+           std::to_string(p.k) + ",\"launches\":" + std::to_string(p.launches) +
+           ",\"total_ms\":" + std::to_string(p.total_ms) + "}";
+  }
+  return out + "]";
+}
+
+bool QuantBertEncoder::set_tap(int layer, const std::string& name, void* dst) {
+  Taps& t = taps;
+  t.tap_layer = layer;
+  int8_t* p = static_cast<int8_t*>(dst);
+  if (name == "ln1_q") t.ln1_q = p;
+  else if (name == "qkv_q") t.qkv_q = p;
+  else if (name == "ctx_q") t.ctx_q = p;
+  else if (name == "out_q") t.out_q = p;
+  else if (name == "ln2_q") t.ln2_q = p;
+  else if (name == "ffn1_q") t.ffn1_q = p;
+  else if (name == "act_q") t.act_q = p;
+  else if (name == "ffn2_acc") t.ffn2_acc = static_cast<int32_t*>(dst);
+  else if (name == "res_attn") t.res_attn = static_cast<__half*>(dst);
+  else if (name == "res_ffn") t.res_ffn = static_cast<__half*>(dst);
+  else return false;
+  return true;
+}
+
 }  // namespace hip
 }  // namespace lightseq

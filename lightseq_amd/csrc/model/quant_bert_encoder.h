@@ -50,6 +50,8 @@ class QuantBertEncoder {
     double total_ms = 0.0;
   };
   void set_profiling(bool on);
+  std::string profile_json() const;
+  bool set_tap(int layer, const std::string& name, void* dst);  // false: no such tap
   void set_fusion(bool on) { _fuse = on; }
   void collect_profile();
   void reset_profile();

@@ -51,9 +51,7 @@ class QuantDecoder {
   void graph_mode(bool on) { _use_graphs = on; }
   // copies of the intermediates of one layer at one step (names: see quant_decoder.cpp)
   StepTaps step_taps;
-  int graphs_captured() const { return _graphs.captured(); }
-  long graphs_replayed() const { return _graphs.replayed(); }
-  int graph_nodes() const { return _graphs.last_graph_nodes(); }
+  const StepGraphs& graphs() const { return _graphs; }
 
   const int* _p_d_padding_mask;
   const __half* _p_d_encoder_output;

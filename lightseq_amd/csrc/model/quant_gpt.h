@@ -7,12 +7,13 @@
 #include <memory>
 
 #include "ls_model.h"
+#include "model_controls.h"
 #include "quant_gpt_encoder.h"
 
 namespace lightseq {
 namespace hip {
 
-class QuantGpt : public LSModel {
+class QuantGpt : public LSModel, public GenerationControls {
  public:
   QuantGpt(const std::string weight_path, const int max_batch_size);
   ~QuantGpt();
@@ -20,6 +21,17 @@ class QuantGpt : public LSModel {
   void Infer() override;
   void benchmark_mode(bool is_benchmark) override { encoder_->benchmark_mode(is_benchmark); }
   void* get_stream() override { return stream_.get(); }
+
+  StepTaps& step_taps() override { return encoder_->step_taps; }
+  void set_seed(unsigned long long seed) override { encoder_->set_seed(seed); }
+  void graph_mode(bool on) override { encoder_->graph_mode(on); }
+  const StepGraphs& graphs() const override { return encoder_->graphs(); }
+  const PhaseEvents& phases() const override { return encoder_->phases(); }
+  int steps_run() const override { return encoder_->steps_run(); }
+  bool set_step_record(int8_t* logits, int*, int max_steps) override {
+    encoder_->set_step_record(logits, max_steps);
+    return true;
+  }
 
   QuantGptEncoder* encoder() { return encoder_.get(); }
   const QuantGptWeight& weight() const { return tw_; }

@@ -51,9 +51,7 @@ class QuantGptEncoder {
   void graph_mode(bool on) { _use_graphs = on; }
   // copies of the intermediates of one layer at one cached step (names: see step_pass)
   StepTaps step_taps;
-  int graphs_captured() const { return _graphs.captured(); }
-  long graphs_replayed() const { return _graphs.replayed(); }
-  int graph_nodes() const { return _graphs.last_graph_nodes(); }
+  const StepGraphs& graphs() const { return _graphs; }
 
   const int* _p_d_token_id;
   float* _p_d_ppl;

@@ -8,13 +8,14 @@
 #include <memory>
 
 #include "ls_model.h"
+#include "model_controls.h"
 #include "quant_bert_encoder.h"
 #include "quant_decoder.h"
 
 namespace lightseq {
 namespace hip {
 
-class QuantTransformer : public LSModel {
+class QuantTransformer : public LSModel, public GenerationControls, public EncoderControls {
  public:
   QuantTransformer(const std::string weight_path, const int max_batch_size);
   ~QuantTransformer();
@@ -22,6 +23,27 @@ class QuantTransformer : public LSModel {
   void Infer() override;
   void benchmark_mode(bool is_benchmark) override;
   void* get_stream() override { return stream_.get(); }
+
+  StepTaps& step_taps() override { return decoder_->step_taps; }
+  void set_seed(unsigned long long seed) override { decoder_->set_seed(seed); }
+  void graph_mode(bool on) override { decoder_->graph_mode(on); }
+  const StepGraphs& graphs() const override { return decoder_->graphs(); }
+  const PhaseEvents& phases() const override { return decoder_->phases(); }
+  int steps_run() const override { return decoder_->steps_run(); }
+  bool set_step_record(int8_t* logits, int* alive_seq, int max_steps) override {
+    decoder_->set_step_record(logits, alive_seq, max_steps);
+    return true;
+  }
+  void set_profiling(bool on) override {
+    encoder_->set_profiling(on);
+    encoder_->reset_profile();
+  }
+  std::string profile_json() override { return encoder_->profile_json(); }
+  bool set_encoder_tap(int layer, const std::string& name, void* dst) override {
+    if (name != "enc_out") return encoder_->set_tap(layer, name, dst);
+    set_encoder_output_tap(static_cast<__half*>(dst));
+    return true;
+  }
 
   QuantBertEncoder* encoder() { return encoder_.get(); }
   QuantDecoder* decoder() { return decoder_.get(); }
