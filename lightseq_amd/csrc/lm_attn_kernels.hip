@@ -1,0 +1,625 @@
+// Attention of the floating-point decoders over slot caches [slot][kv_head][position][pad]: per-head
+// RMS norm and interleaved rotation, causal attention with a sliding window, kept first tokens and
+// a valueless sink in the soft-max, and an element-wise output gate; a prompt kernel on the matrix
+// cores and a one-token kernel that streams the cache.
+//
+// Keys and values are stored with rows padded to a size the prompt kernel is instantiated for
+// (attn_pad), the padding written as zeros with the row, so no load needs a column guard.
+#include <algorithm>
+
+#include "lm_launch.h"
+
+namespace lsh {
+
+int attn_pad(int dim) {
+  return dim <= 0 ? 0 : dim <= 64 ? 64 : dim <= 96 ? 96 : dim <= 128 ? 128 : dim <= 256 ? 256 : 0;
+}
+
+namespace {
+
+// ------------------------------------------------------------------------------------------------
+// One wavefront per (row, head); lane i holds the pairs i, i + 64 (dimensions 2i, 2i + 1).
+template <typename T>
+__global__ void __launch_bounds__(256)
+attn_prepare_kernel(const T* __restrict__ proj, long ld, int q_col, int k_col, int v_col,
+                    const float* __restrict__ q_norm, const float* __restrict__ k_norm, float eps,
+                    const float2* __restrict__ cos_sin, int rot_pairs, T* __restrict__ q_out,
+                    T* __restrict__ k_cache, T* __restrict__ v_cache,
+                    const int* __restrict__ row_slot, const int* __restrict__ row_pos, long units,
+                    int heads_per_row, AttnShape sh) {
+  const long unit = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (unit >= units) return;
+  const int lane = threadIdx.x & 63;
+  const long row = unit / heads_per_row;
+  int head = (int)(unit - row * heads_per_row);
+  const T* src = proj + row * ld;
+  const int pos = row_pos[row];
+  int kind = 0;  // 0 q, 1 k, 2 v
+  T* dst;
+  if (head < sh.heads) {
+    src += q_col + head * sh.dim;
+    dst = q_out + (row * sh.heads + head) * sh.dim_pad;
+  } else {
+    head -= sh.heads;
+    kind = head < sh.kv_heads ? 1 : 2;
+    if (kind == 2) head -= sh.kv_heads;
+    src += kind == 1 ? k_col + head * sh.dim : v_col + head * sh.vdim;
+    const long at = ((long)row_slot[row] * sh.kv_heads + head) * sh.max_step + pos;
+    dst = kind == 1 ? k_cache + at * sh.dim_pad : v_cache + at * sh.vdim_pad;
+  }
+  const int n = kind == 2 ? sh.vdim : sh.dim, pad = kind == 2 ? sh.vdim_pad : sh.dim_pad;
+  float u[2][2];
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    const int d = 2 * (i * 64 + lane);
+    u[i][0] = d < n ? to_f(src[d]) : 0.f;
+    u[i][1] = d + 1 < n ? to_f(src[d + 1]) : 0.f;
+  }
+  if (kind != 2) {
+    const float ss = wave_sum_dpp(u[0][0] * u[0][0] + u[0][1] * u[0][1] + u[1][0] * u[1][0] +
+                                  u[1][1] * u[1][1]);
+    const float r = 1.0f / sqrtf(ss / (float)n + eps);
+    const float* w = kind == 0 ? q_norm : k_norm;
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      const int p = i * 64 + lane, d = 2 * p;
+      if (w) {
+        if (d < n) u[i][0] = u[i][0] * r * w[d];
+        if (d + 1 < n) u[i][1] = u[i][1] * r * w[d + 1];
+      }
+      if (p < rot_pairs) {
+        const float2 cs = cos_sin[(long)pos * rot_pairs + p];
+        const float a = u[i][0], b = u[i][1];
+        u[i][0] = a * cs.x - b * cs.y;
+        u[i][1] = b * cs.x + a * cs.y;
+      }
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    const int d = 2 * (i * 64 + lane);
+    if (d < pad) stv<2, T>(dst + d, u[i]);  // zeros beyond the head size
+  }
+}
+
+// ------------------------------------------------------------------------------------------------
+// Prompt kernel.  A workgroup takes 128 queries of one (sequence, head), 32 per wavefront, and walks
+// the key tiles of 64 that any of them sees: first the kept tokens, then the window.  Scores are
+// computed transposed (keys x queries), so a lane owns one query: running maximum, sum and the
+// rescaling of its context need no exchange but one with the other half of the wavefront, and the
+// probabilities are the second operand of the context product as they lie in registers.  The sink
+// is the start value of the running soft-max: maximum 0, sum 1, context 0.
+constexpr int kQT = 128, kKT = 64;
+
+__device__ __forceinline__ float exp2_f(float x) { return __builtin_amdgcn_exp2f(x); }
+
+template <typename T, int NK, int NV>  // head sizes in 32s
+__global__ void __launch_bounds__(256)
+attn_prefill_kernel(const T* __restrict__ q, const T* __restrict__ k_cache,
+                    const T* __restrict__ v_cache, const T* __restrict__ proj, long ld, int g_col,
+                    T* __restrict__ out, const SeqSpan* __restrict__ seqs, AttnShape sh,
+                    AttnMask mask) {
+  constexpr int DP = NK * 32, VP = NV * 32, V = FT<T>::kVec;
+  constexpr int KSTR = DP + V;           // elements per key row in LDS
+  constexpr int VSTR = kKT + 16 / sizeof(T);  // keys per value column in LDS
+  constexpr int NKS = DP * sizeof(T) / 32;    // 32-byte slices of a key row
+  extern __shared__ __attribute__((aligned(16))) char smem_raw[];
+  T* Ks = reinterpret_cast<T*>(smem_raw);
+  T* Vt = Ks + kKT * KSTR;
+  const SeqSpan sq = seqs[blockIdx.z];
+  // the longest key ranges first
+  const int qt = (sq.n + kQT - 1) / kQT - 1 - (int)blockIdx.x;
+  if (qt < 0) return;
+  const int head = blockIdx.y, kvh = head / (sh.heads / sh.kv_heads);
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l32 = lane & 31, g = lane >> 5;
+  const int i0 = qt * kQT;                      // first query of the tile, in the span
+  const int i_last = min(i0 + kQT, sq.n) - 1;
+  const int my_i = min(i0 + wave * 32 + l32, sq.n - 1);
+  const int pos = sq.pos0 + my_i;
+  const int wq_lo = sq.pos0 + min(i0 + wave * 32, sq.n - 1);
+  const int wq_hi = sq.pos0 + min(i0 + wave * 32 + 31, sq.n - 1);
+  const bool wave_live = i0 + wave * 32 < sq.n;
+  const int kv_len = sq.pos0 + sq.n;
+  const long cache0 = ((long)sq.slot * sh.kv_heads + kvh) * sh.max_step;
+  const T* kc = k_cache + cache0 * DP;
+  const T* vc = v_cache + cache0 * VP;
+
+  frag_t qf[NKS];
+  {
+    const T* qr = q + ((long)(sq.row0 + my_i) * sh.heads + head) * DP;
+#pragma unroll
+    for (int s = 0; s < NKS; ++s) qf[s] = *reinterpret_cast<const frag_t*>(qr + (2 * s + g) * V);
+  }
+  const float sc2 = mask.scale * 1.44269504088896340736f;
+  float m = mask.sink ? 0.f : -INFINITY, l = mask.sink ? 1.f : 0.f;  // m in units of log2
+  f32x16v acc[NV];
+#pragma unroll
+  for (int d = 0; d < NV; ++d) acc[d] = (f32x16v)0.f;
+
+  const int first_pos = sq.pos0 + i0, last_pos = sq.pos0 + i_last;
+  const int t_end = last_pos / kKT;  // last tile
+  const int t_win = mask.window > 0 ? max(0, first_pos - mask.window + 1) / kKT : 0;
+  const int t_keep = mask.keep_first > 0 ? (min(mask.keep_first, kv_len) - 1) / kKT : -1;
+  for (int t = 0; t <= t_end; ++t) {
+    if (t > t_keep && t < t_win) t = t_win;
+    const int key0 = t * kKT;
+    __syncthreads();
+    // keys: 16-byte chunks, rows beyond the sequence are clamped (their scores are masked)
+    constexpr int CH = DP / V;
+    for (int c = tid; c < kKT * CH; c += 256) {
+      const int r = c / CH, x = c - r * CH;
+      *reinterpret_cast<frag_t*>(&Ks[r * KSTR + x * V]) =
+          *reinterpret_cast<const frag_t*>(kc + (long)min(key0 + r, kv_len - 1) * DP + x * V);
+    }
+    // values transposed: a thread takes 4 keys of one 4-column group and stores 4 keys per column
+    for (int c = tid; c < (kKT / 4) * (VP / 4); c += 256) {
+      const int r4 = c / (VP / 4), x = c - r4 * (VP / 4);
+      float v[4][4];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int key = key0 + r4 * 4 + j;
+        if (key < kv_len) {
+          ldv<4, T>(vc + (long)key * VP + x * 4, v[j]);
+        } else {
+#pragma unroll
+          for (int e = 0; e < 4; ++e) v[j][e] = 0.f;
+        }
+      }
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const float col[4] = {v[0][e], v[1][e], v[2][e], v[3][e]};
+        stv<4, T>(&Vt[(x * 4 + e) * VSTR + r4 * 4], col);
+      }
+    }
+    __syncthreads();
+    if (!wave_live) continue;
+    // does any query of this wavefront see any key of the tile?
+    const bool causal_any = key0 <= wq_hi;
+    const bool win_any = mask.window <= 0 || wq_lo - (key0 + kKT - 1) < mask.window;
+    if (!causal_any || !(win_any || key0 < mask.keep_first)) continue;
+    const bool all = key0 + kKT - 1 <= wq_lo &&
+                     (mask.window <= 0 || wq_hi - key0 < mask.window ||
+                      key0 + kKT <= mask.keep_first);
+    f32x16v sc[2];
+#pragma unroll
+    for (int b = 0; b < 2; ++b) {
+      sc[b] = (f32x16v)0.f;
+      const T* kr = &Ks[(b * 32 + l32) * KSTR + g * V];
+#pragma unroll
+      for (int s = 0; s < NKS; ++s)
+        sc[b] = mma32(T{}, *reinterpret_cast<const frag_t*>(kr + 2 * s * V), qf[s], sc[b]);
+    }
+    float mx = m;
+#pragma unroll
+    for (int b = 0; b < 2; ++b)
+#pragma unroll
+      for (int i = 0; i < 16; ++i) {
+        float v = sc[b][i] * sc2;
+        if (!all) {
+          const int key = key0 + b * 32 + 8 * (i >> 2) + 4 * g + (i & 3);
+          const bool see = key <= pos && (mask.window <= 0 || pos - key < mask.window ||
+                                          key < mask.keep_first);
+          v = see ? v : -INFINITY;
+        }
+        sc[b][i] = v;
+        mx = fmaxf(mx, v);
+      }
+    mx = fmaxf(mx, __shfl_xor(mx, 32));
+    const float f = m == -INFINITY ? 0.f : exp2_f(m - mx);
+    m = mx;
+    // (no sink) a query that has seen nothing yet: all its probabilities are zero
+    const float ref = mx == -INFINITY ? 0.f : mx;
+    float sum = 0.f;
+#pragma unroll
+    for (int b = 0; b < 2; ++b)
+#pragma unroll
+      for (int i = 0; i < 16; ++i) {
+        sc[b][i] = exp2_f(sc[b][i] - ref);
+        sum += sc[b][i];
+      }
+    sum += __shfl_xor(sum, 32);
+    l = l * f + sum;
+#pragma unroll
+    for (int d = 0; d < NV; ++d)
+#pragma unroll
+      for (int i = 0; i < 16; ++i) acc[d][i] *= f;
+    // context: slots of the product are the keys in the order the scores lie in registers
+#pragma unroll
+    for (int b = 0; b < 2; ++b) {
+      if constexpr (sizeof(T) == 2) {
+#pragma unroll
+        for (int h = 0; h < 2; ++h) {
+          bf16x8 pb;
+#pragma unroll
+          for (int j = 0; j < 8; ++j) pb[j] = (__bf16)sc[b][8 * h + j];
+#pragma unroll
+          for (int d = 0; d < NV; ++d) {
+            const T* vr = &Vt[(d * 32 + l32) * VSTR + b * 32 + 16 * h + 4 * g];
+            const uint2 lo = *reinterpret_cast<const uint2*>(vr);
+            const uint2 hi = *reinterpret_cast<const uint2*>(vr + 8);
+            const frag_t va = {lo.x, lo.y, hi.x, hi.y};
+            acc[d] = mma32(T{}, va, __builtin_bit_cast(frag_t, pb), acc[d]);
+          }
+        }
+      } else {
+#pragma unroll
+        for (int h = 0; h < 4; ++h) {
+          const f32x4 pb = {sc[b][4 * h], sc[b][4 * h + 1], sc[b][4 * h + 2], sc[b][4 * h + 3]};
+#pragma unroll
+          for (int d = 0; d < NV; ++d) {
+            const frag_t va = *reinterpret_cast<const frag_t*>(
+                &Vt[(d * 32 + l32) * VSTR + b * 32 + 8 * h + 4 * g]);
+            acc[d] = mma32(T{}, va, __builtin_bit_cast(frag_t, pb), acc[d]);
+          }
+        }
+      }
+    }
+  }
+  if (i0 + wave * 32 + l32 >= sq.n) return;
+  const float inv = l > 0.f ? 1.f / l : 0.f;
+  const long row = sq.row0 + my_i;
+  const T* gate = g_col >= 0 ? proj + row * ld + g_col + head * sh.vdim : nullptr;
+  T* op = out + row * ((long)sh.heads * sh.vdim) + head * sh.vdim;
+  const bool vec = sh.vdim % 4 == 0 && (g_col < 0 || (g_col % 4 == 0 && ld % 4 == 0));
+#pragma unroll
+  for (int d = 0; d < NV; ++d)
+#pragma unroll
+    for (int w = 0; w < 4; ++w) {
+      const int c = d * 32 + 8 * w + 4 * g;
+      if (c >= sh.vdim) continue;
+      float o[4];
+#pragma unroll
+      for (int e = 0; e < 4; ++e) o[e] = acc[d][4 * w + e] * inv;
+      if (vec) {
+        if (gate) {
+          float z[4];
+          ldv<4, T>(gate + c, z);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) o[e] *= sigmoid_f(z[e]);
+        }
+        stv<4, T>(op + c, o);
+      } else {
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          if (c + e < sh.vdim)
+            op[c + e] = from_f<T>(gate ? o[e] * sigmoid_f(to_f(gate[c + e])) : o[e]);
+      }
+    }
+}
+
+template <typename T, int NK, int NV>
+int launch_prefill(const T* q, const T* kc, const T* vc, const T* proj, long ld, int g_col, T* out,
+                   const SeqSpan* seqs, int n_seqs, int max_n, const AttnShape& sh,
+                   const AttnMask& mask, hipStream_t s) {
+  constexpr int V = FT<T>::kVec;
+  constexpr size_t smem = sizeof(T) * ((size_t)kKT * (NK * 32 + V) +
+                                       (size_t)NV * 32 * (kKT + 16 / sizeof(T)));
+  auto kern = attn_prefill_kernel<T, NK, NV>;
+  if (smem > 48 * 1024) {
+    if (int rc = lsh_check_hip(hipFuncSetAttribute(reinterpret_cast<const void*>(kern),
+                                                   hipFuncAttributeMaxDynamicSharedMemorySize,
+                                                   (int)smem),
+                               "hipFuncSetAttribute(attn_prefill)"))
+      return rc;
+  }
+  const dim3 grid((max_n + kQT - 1) / kQT, sh.heads, n_seqs);
+  kern<<<grid, 256, smem, s>>>(q, kc, vc, proj, ld, g_col, out, seqs, sh, mask);
+  return lsh_check_launch("attn_prefill_kernel");
+}
+
+// ------------------------------------------------------------------------------------------------
+// One-token kernel.  A workgroup takes up to R query heads of one (row, kv head) and one part of the
+// visible keys, in chunks of 256: 16 lanes per key form the scores, the chunk's soft-max runs over
+// LDS, then the same 16-lane groups accumulate the values.  The visible keys are numbered
+// 0 .. n_vis - 1, the kept ones first.
+constexpr int kChunk = 256;
+
+template <typename T, int EK, int EV, int R>  // elements per lane of a key / value row
+__global__ void __launch_bounds__(256)
+attn_decode_kernel(const T* __restrict__ q, const T* __restrict__ k_cache,
+                   const T* __restrict__ v_cache, const T* __restrict__ proj, long ld, int g_col,
+                   T* __restrict__ out, const int* __restrict__ row_slot,
+                   const int* __restrict__ row_pos, int nsplit, int head_groups,
+                   float* __restrict__ workspace, AttnShape sh, AttnMask mask) {
+  constexpr int DP = EK * 16, VP = EV * 16;
+  __shared__ float sc[R][kChunk];
+  __shared__ float fac[R], mrow[R], lrow[R];
+  __shared__ float part[4][R][VP];
+  const int row = blockIdx.x, kvh = blockIdx.y / head_groups, hg = blockIdx.y % head_groups;
+  const int split = blockIdx.z;
+  const int rep = sh.heads / sh.kv_heads;
+  const int h0 = kvh * rep + hg * R, nh = min(R, rep - hg * R);
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, grp = tid >> 4, j = tid & 15;
+  const int pos = row_pos[row];
+  const long cache0 = ((long)row_slot[row] * sh.kv_heads + kvh) * sh.max_step;
+  const T* kc = k_cache + cache0 * DP + j * EK;
+  const T* vc = v_cache + cache0 * VP + j * EV;
+  const int lo = mask.window > 0 ? max(0, pos - mask.window + 1) : 0;  // first key of the window
+  const int kept = min(mask.keep_first, lo);                           // kept keys before it
+  const int n_vis = kept + pos + 1 - lo;
+  const int per = ((n_vis + nsplit - 1) / nsplit + 15) & ~15;
+  const int v_lo = min(split * per, n_vis), v_hi = min(v_lo + per, n_vis);
+
+  float qv[R][EK], acc[R][EV];
+#pragma unroll
+  for (int r = 0; r < R; ++r) {
+    const T* qr = q + ((long)row * sh.heads + h0 + min(r, nh - 1)) * DP + j * EK;
+#pragma unroll
+    for (int e = 0; e < EK; e += 2) {
+      float t[2];
+      ldv<2, T>(qr + e, t);
+      qv[r][e] = t[0] * mask.scale * 1.44269504088896340736f;
+      qv[r][e + 1] = t[1] * mask.scale * 1.44269504088896340736f;
+    }
+#pragma unroll
+    for (int e = 0; e < EV; ++e) acc[r][e] = 0.f;
+  }
+  if (tid < R) {
+    const bool sink = mask.sink && split == 0;
+    mrow[tid] = sink ? 0.f : -INFINITY;
+    lrow[tid] = sink ? 1.f : 0.f;
+  }
+  auto key_of = [&](int v) { return v < kept ? v : lo + v - kept; };
+  for (int c0 = v_lo; c0 < v_hi; c0 += kChunk) {
+    const int n = min(kChunk, v_hi - c0);
+    __syncthreads();
+    for (int i = grp; i < n; i += 64) {  // four keys per turn: their loads are in flight together
+      float kv[4][EK];
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        const T* kr = kc + (long)key_of(c0 + min(i + 16 * u, n - 1)) * DP;
+#pragma unroll
+        for (int e = 0; e < EK; e += 2) {
+          float t[2];
+          ldv<2, T>(kr + e, t);
+          kv[u][e] = t[0];
+          kv[u][e + 1] = t[1];
+        }
+      }
+#pragma unroll
+      for (int u = 0; u < 4; ++u)
+#pragma unroll
+        for (int r = 0; r < R; ++r) {
+          float d = 0.f;
+#pragma unroll
+          for (int e = 0; e < EK; ++e) d = fmaf(qv[r][e], kv[u][e], d);
+          d += dpp_f<kDppXor1>(d);
+          d += dpp_f<kDppXor2>(d);
+          d += dpp_f<kDppHalfMirror>(d);
+          d += dpp_f<kDppMirror>(d);
+          if (j == 0 && i + 16 * u < n) sc[r][i + 16 * u] = d;
+        }
+    }
+    __syncthreads();
+    for (int r = wave; r < R; r += 4) {
+      float mx = -INFINITY;
+      for (int i = lane; i < n; i += 64) mx = fmaxf(mx, sc[r][i]);
+      mx = fmaxf(wave_max_dpp(mx), mrow[r]);
+      float sum = 0.f;
+      for (int i = lane; i < n; i += 64) {
+        const float e = exp2_f(sc[r][i] - mx);
+        sc[r][i] = e;
+        sum += e;
+      }
+      sum = wave_sum_dpp(sum);
+      if (lane == 0) {
+        const float f = mrow[r] == -INFINITY ? 0.f : exp2_f(mrow[r] - mx);
+        fac[r] = f;
+        lrow[r] = lrow[r] * f + sum;
+        mrow[r] = mx;
+      }
+    }
+    __syncthreads();
+#pragma unroll
+    for (int r = 0; r < R; ++r) {
+      const float f = fac[r];
+#pragma unroll
+      for (int e = 0; e < EV; ++e) acc[r][e] *= f;
+    }
+    for (int i = grp; i < n; i += 64) {
+      float vv[4][EV];
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        const T* vr = vc + (long)key_of(c0 + min(i + 16 * u, n - 1)) * VP;
+#pragma unroll
+        for (int e = 0; e < EV; e += 2) {
+          float t[2];
+          ldv<2, T>(vr + e, t);
+          vv[u][e] = t[0];
+          vv[u][e + 1] = t[1];
+        }
+      }
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        const bool in = i + 16 * u < n;
+#pragma unroll
+        for (int r = 0; r < R; ++r) {
+          const float p = in ? sc[r][i + 16 * u] : 0.f;
+#pragma unroll
+          for (int e = 0; e < EV; ++e) acc[r][e] = fmaf(p, vv[u][e], acc[r][e]);
+        }
+      }
+    }
+  }
+  // the 16 groups' contexts: over the wavefront's four by lane exchange, then over LDS
+#pragma unroll
+  for (int r = 0; r < R; ++r)
+#pragma unroll
+    for (int e = 0; e < EV; ++e) {
+      float a = acc[r][e];
+      a += __shfl_xor(a, 16);
+      a += __shfl_xor(a, 32);
+      if (lane < 16) part[wave][r][j * EV + e] = a;
+    }
+  __syncthreads();
+  for (int x = tid; x < nh * VP; x += 256) {
+    const int r = x / VP, c = x - r * VP;
+    const float a = (part[0][r][c] + part[1][r][c]) + (part[2][r][c] + part[3][r][c]);
+    const int head = h0 + r;
+    if (nsplit > 1) {
+      // [row][head][split][VP + 2]: context, maximum, sum
+      float* w = workspace + (((long)row * sh.heads + head) * nsplit + split) * (VP + 2);
+      w[c] = a;
+      if (c == 0) {
+        w[VP] = mrow[r];
+        w[VP + 1] = lrow[r];
+      }
+    } else if (c < sh.vdim) {
+      float o = a / lrow[r];
+      if (g_col >= 0) o *= sigmoid_f(to_f(proj[(long)row * ld + g_col + head * sh.vdim + c]));
+      out[(long)row * sh.heads * sh.vdim + head * sh.vdim + c] = from_f<T>(o);
+    }
+  }
+}
+
+template <typename T>
+__global__ void __launch_bounds__(256)
+attn_decode_combine_kernel(const float* __restrict__ workspace, const T* __restrict__ proj, long ld,
+                           int g_col, T* __restrict__ out, int nsplit, int vp, AttnShape sh) {
+  const int row = blockIdx.x, head = blockIdx.y;
+  const float* w = workspace + ((long)row * sh.heads + head) * nsplit * (vp + 2);
+  float m = -INFINITY;
+  for (int p = 0; p < nsplit; ++p) m = fmaxf(m, w[(long)p * (vp + 2) + vp]);
+  for (int c = threadIdx.x; c < sh.vdim; c += blockDim.x) {
+    float a = 0.f, l = 0.f;
+    for (int p = 0; p < nsplit; ++p) {
+      const float* wp = w + (long)p * (vp + 2);
+      const float f = wp[vp] == -INFINITY ? 0.f : exp2_f(wp[vp] - m);
+      a += f * wp[c];
+      l += f * wp[vp + 1];
+    }
+    float o = a / l;
+    if (g_col >= 0) o *= sigmoid_f(to_f(proj[(long)row * ld + g_col + head * sh.vdim + c]));
+    out[(long)row * sh.heads * sh.vdim + head * sh.vdim + c] = from_f<T>(o);
+  }
+}
+
+constexpr int kMaxSplit = 32;
+
+int check_shape(const AttnShape& sh, const char* who) {
+  if (sh.heads <= 0 || sh.kv_heads <= 0 || sh.heads % sh.kv_heads != 0 || sh.max_step <= 0)
+    return lsh_fail(LSH_ERR_INVALID, who);
+  if (attn_pad(sh.dim) == 0 || attn_pad(sh.vdim) == 0 || sh.dim_pad != attn_pad(sh.dim) ||
+      sh.vdim_pad != attn_pad(sh.vdim))
+    return lsh_fail(LSH_ERR_UNSUPPORTED, "attention: head sizes above 256");
+  return LSH_OK;
+}
+
+}  // namespace
+
+template <typename T>
+int attn_prepare(const T* proj, long ld, int q_col, int k_col, int v_col, const float* q_norm,
+                 const float* k_norm, float eps, const float2* cos_sin, int rot_pairs, T* q_out,
+                 T* k_cache, T* v_cache, const int* row_slot, const int* row_pos, int rows,
+                 const AttnShape& sh, hipStream_t s) {
+  if (int rc = check_shape(sh, "attn_prepare: bad shape")) return rc;
+  if (!proj || !q_out || !row_slot || !row_pos || rows <= 0 || rot_pairs < 0 ||
+      2 * rot_pairs > sh.dim || (rot_pairs > 0 && !cos_sin) ||
+      (k_col >= 0 && (!k_cache || !v_cache || v_col < 0)))
+    return lsh_fail(LSH_ERR_INVALID, "attn_prepare: bad arguments");
+  const int per_row = sh.heads + (k_col >= 0 ? 2 * sh.kv_heads : 0);
+  const long units = (long)rows * per_row;
+  attn_prepare_kernel<T><<<(unsigned)((units + 3) / 4), 256, 0, s>>>(
+      proj, ld, q_col, k_col, v_col, q_norm, k_norm, eps, cos_sin, rot_pairs, q_out, k_cache,
+      v_cache, row_slot, row_pos, units, per_row, sh);
+  return lsh_check_launch("attn_prepare_kernel");
+}
+
+#define PICK_V(NK)                                                                              \
+  switch (sh.vdim_pad / 32) {                                                                   \
+    case 2: return launch_prefill<T, NK, 2>(q, k_cache, v_cache, proj, ld, g_col, out, seqs,    \
+                                            n_seqs, max_n, sh, mask, s);                        \
+    case 3: return launch_prefill<T, NK, 3>(q, k_cache, v_cache, proj, ld, g_col, out, seqs,    \
+                                            n_seqs, max_n, sh, mask, s);                        \
+    case 4: return launch_prefill<T, NK, 4>(q, k_cache, v_cache, proj, ld, g_col, out, seqs,    \
+                                            n_seqs, max_n, sh, mask, s);                        \
+    default: return launch_prefill<T, NK, 8>(q, k_cache, v_cache, proj, ld, g_col, out, seqs,   \
+                                             n_seqs, max_n, sh, mask, s);                       \
+  }
+
+template <typename T>
+int attn_prefill(const T* q, const T* k_cache, const T* v_cache, const T* proj, long ld, int g_col,
+                 T* out, const SeqSpan* seqs, int n_seqs, int max_n, const AttnShape& sh,
+                 const AttnMask& mask, hipStream_t s) {
+  if (int rc = check_shape(sh, "attn_prefill: bad shape")) return rc;
+  if (!q || !k_cache || !v_cache || !out || !seqs || n_seqs <= 0 || max_n <= 0 ||
+      (g_col >= 0 && !proj) || n_seqs > 65535 || sh.heads > 65535)
+    return lsh_fail(LSH_ERR_INVALID, "attn_prefill: bad arguments");
+  switch (sh.dim_pad / 32) {
+    case 2: PICK_V(2)
+    case 3: PICK_V(3)
+    case 4: PICK_V(4)
+    default: PICK_V(8)
+  }
+}
+
+size_t attn_decode_workspace(int rows, const AttnShape& sh) {
+  return (size_t)rows * sh.heads * kMaxSplit * (sh.vdim_pad + 2);
+}
+
+#define DEC(EK, EV, R)                                                                           \
+  attn_decode_kernel<T, EK, EV, R><<<grid, 256, 0, s>>>(q, k_cache, v_cache, proj, ld, g_col,    \
+                                                        out, row_slot, row_pos, nsplit, groups,  \
+                                                        workspace, sh, mask)
+#define DEC_R(EK, EV)                                                                            \
+  do {                                                                                           \
+    if (R == 1) DEC(EK, EV, 1);                                                                  \
+    else if (R == 2) DEC(EK, EV, 2);                                                             \
+    else DEC(EK, EV, 4);                                                                         \
+  } while (0)
+#define DEC_V(EK)                                                                                \
+  switch (sh.vdim_pad / 16) {                                                                    \
+    case 4: DEC_R(EK, 4); break;                                                                 \
+    case 6: DEC_R(EK, 6); break;                                                                 \
+    case 8: DEC_R(EK, 8); break;                                                                 \
+    default: DEC_R(EK, 16); break;                                                               \
+  }
+
+template <typename T>
+int attn_decode(const T* q, const T* k_cache, const T* v_cache, const T* proj, long ld, int g_col,
+                T* out, const int* row_slot, const int* row_pos, int rows, int max_len,
+                float* workspace, const AttnShape& sh, const AttnMask& mask, hipStream_t s) {
+  if (int rc = check_shape(sh, "attn_decode: bad shape")) return rc;
+  if (!q || !k_cache || !v_cache || !out || !row_slot || !row_pos || rows <= 0 || max_len <= 0 ||
+      !workspace || (g_col >= 0 && !proj))
+    return lsh_fail(LSH_ERR_INVALID, "attn_decode: bad arguments");
+  const int rep = sh.heads / sh.kv_heads;
+  const int R = rep == 1 ? 1 : rep == 2 ? 2 : 4;
+  const int groups = (rep + R - 1) / R;
+  const long most = mask.window > 0 ? std::min((long)max_len, (long)mask.window + mask.keep_first)
+                                    : (long)max_len;
+  // enough workgroups to fill the chip, parts of at least 128 keys
+  const int want = (int)((2L * cu_count() + (long)rows * sh.kv_heads * groups - 1) /
+                         ((long)rows * sh.kv_heads * groups));
+  const int nsplit = (int)std::max(1L, std::min({(long)kMaxSplit, (long)want, most / 128}));
+  if ((long)sh.kv_heads * groups > 65535) return lsh_fail(LSH_ERR_UNSUPPORTED, "attn_decode: heads");
+  const dim3 grid(rows, sh.kv_heads * groups, nsplit);
+  switch (sh.dim_pad / 16) {
+    case 4: DEC_V(4) break;
+    case 6: DEC_V(6) break;
+    case 8: DEC_V(8) break;
+    default: DEC_V(16) break;
+  }
+  if (int rc = lsh_check_launch("attn_decode_kernel")) return rc;
+  if (nsplit > 1) {
+    attn_decode_combine_kernel<T><<<dim3(rows, sh.heads), sh.vdim <= 64 ? 64 : 128, 0, s>>>(
+        workspace, proj, ld, g_col, out, nsplit, sh.vdim_pad, sh);
+    return lsh_check_launch("attn_decode_combine_kernel");
+  }
+  return LSH_OK;
+}
+
+#define INST(T)                                                                                   \
+  template int attn_prepare<T>(const T*, long, int, int, int, const float*, const float*, float,  \
+                               const float2*, int, T*, T*, T*, const int*, const int*, int,       \
+                               const AttnShape&, hipStream_t);                                    \
+  template int attn_prefill<T>(const T*, const T*, const T*, const T*, long, int, T*,             \
+                               const SeqSpan*, int, int, const AttnShape&, const AttnMask&,       \
+                               hipStream_t);                                                      \
+  template int attn_decode<T>(const T*, const T*, const T*, const T*, long, int, T*, const int*,  \
+                              const int*, int, int, float*, const AttnShape&, const AttnMask&,    \
+                              hipStream_t);
+INST(float)
+INST(bf16_t)
+
+}  // namespace lsh
