@@ -28,7 +28,8 @@ typedef struct ls_model ls_model;
 /* values of lightseq::cuda::DataType, model_base.h:12-26 */
 enum {
   LS_DTYPE_NOT_SUPPORTED = 0, LS_DTYPE_FLOAT32 = 1, LS_DTYPE_INT32 = 2, LS_DTYPE_INT64 = 3,
-  LS_DTYPE_FLOAT16 = 4, LS_DTYPE_INT8 = 5
+  LS_DTYPE_FLOAT16 = 4, LS_DTYPE_INT8 = 5,
+  LS_DTYPE_BFLOAT16 = 13 /* not in the reference */
 };
 #define LS_MAX_DIMS 8
 
@@ -129,6 +130,37 @@ int ls_model_get_graph_nodes(ls_model* model, int* nodes);
  * (kernels/transformerKernels.cc.cu:2270-2274, model/quant_gpt_encoder.cc.cu:66-71) and defines
  * no stream of numbers.  No counterpart in the reference. */
 int ls_model_set_seed(ls_model* model, unsigned long long seed);
+
+/* ---- models in a folder (no counterpart in the reference) -------------------------------
+ * A folder holds config.json and model.safetensors; config.json's "architecture" names the model
+ * class ("Sudevik").  What the folder does not say is in the options; ls_model_default_options
+ * fills in defaults (bfloat16, greedy, 8 sequences of 2048 positions).
+ *
+ * ls_model_infer() of such a model generates: input 0 "token_ids" int32 [batch, seq_len], short
+ * prompts padded on the right with padding_id; output 0 "result" int32 [batch, len]: prompt and
+ * generated ids, short rows padded the same way. */
+typedef struct ls_model_options {
+  int max_batch_size;
+  int max_step;            /* positions a sequence can have */
+  int dtype;               /* LS_DTYPE_BFLOAT16 or LS_DTYPE_FLOAT32 */
+  int topk;                /* 1 greedy, > 1 top-k, 0 top-p */
+  float topp;
+  int eos_id;              /* -1: none */
+  int padding_id;
+  int extra_decode_length; /* tokens generated after the longest prompt */
+} ls_model_options;
+void ls_model_default_options(ls_model_options* options);
+int ls_model_create_from_dir(const char* model_dir, const ls_model_options* options,
+                             ls_model** model);
+int ls_model_get_vocab_size(ls_model* model, int* size);
+/* Step-wise decoding of given tokens through the same step function and caches.  A sequence takes
+ * one of max_batch_size places from open to close.  ls_model_step appends counts[i] tokens to
+ * sequence slots[i]; all entries are one batch; `tokens` holds them entry after entry.  The logits
+ * of the rows named in want_rows (numbers into `tokens`) go to host memory [n_want][vocab]. */
+int ls_model_open_sequence(ls_model* model, int* slot);
+int ls_model_close_sequence(ls_model* model, int slot);
+int ls_model_step(ls_model* model, int entries, const int* slots, const int* counts,
+                  const int* tokens, int n_want, const int* want_rows, float* logits);
 
 #ifdef __cplusplus
 }

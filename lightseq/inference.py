@@ -8,9 +8,9 @@
 run unchanged.  The float models of that module (Transformer, Gpt, Bert, Moe, Vit, T5 ...)
 are not part of this build and raise on access with a message that says so.
 """
-from lightseq_amd.inference import QuantBert, QuantGpt, QuantTransformer  # noqa: F401
+from lightseq_amd.inference import DecoderModel, QuantBert, QuantGpt, QuantTransformer, Sudevik  # noqa: F401
 
-__all__ = ["QuantBert", "QuantGpt", "QuantTransformer"]
+__all__ = ["DecoderModel", "QuantBert", "QuantGpt", "QuantTransformer", "Sudevik"]
 
 _NOT_BUILT = ("Transformer", "Gpt", "Bert", "Moe", "Vit", "T5", "MT5", "XGLM", "QuantVit")
 

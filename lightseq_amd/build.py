@@ -2,9 +2,12 @@
 
 ``python -m lightseq_amd.build`` compiles each translation unit of ``csrc/`` to an
 object file (in parallel) and links them into ``lightseq_amd/lib/``.  The GPU is not
-needed: hipcc cross-compiles.
+needed: hipcc cross-compiles.  ``build_decoder_library`` builds the part that the
+floating-point decoder models need, ``liblightseq_decoder.so``: the same model C ABI
+without the int8 kernels and models.
 """
 import concurrent.futures
+import fcntl
 import os
 import shutil
 import subprocess
@@ -15,6 +18,15 @@ CSRC = os.path.join(_HERE, "csrc")
 OBJ_DIR = os.path.join(CSRC, "_obj")
 LIB_DIR = os.path.join(_HERE, "lib")
 LIB_PATH = os.path.join(LIB_DIR, "liblightseq_hip.so")
+DECODER_LIB_PATH = os.path.join(LIB_DIR, "liblightseq_decoder.so")
+
+# sources of liblightseq_decoder.so
+DECODER_SOURCES = [
+    "core.hip", "gemm_float.hip", "lm_norm_kernels.hip", "lm_attn_kernels.hip", "delta_kernels.hip",
+    "moe_kernels.hip", "lm_sample_kernels.hip", "lm_capi.hip", "model/model_capi.cpp",
+    "model/model_dir.cpp", "model/sudevik.cpp", "model/sudevik_config.cpp",
+    "model/sudevik_decoder.cpp", "model/sudevik_weight.cpp",
+]
 
 ARCH = "gfx950"
 # -packed-fp32-ops off: hipcc must not form v_pk_{add,mul,fma}_f32 from float code.
@@ -56,9 +68,30 @@ def _compile_one(src):
 
 def build_library(verbose=False, jobs=None):
     """Compile everything and link the shared library; returns its path."""
+    return _build(sources(), LIB_PATH, verbose, jobs)
+
+
+def build_decoder_library(verbose=False, jobs=None):
+    """The library of the floating-point decoder models only; returns its path."""
+    return _build([os.path.join(CSRC, s) for s in DECODER_SOURCES], DECODER_LIB_PATH, verbose, jobs)
+
+
+def ensure_decoder_library():
+    """Path of a built library that has the decoder models, building the smaller one if there is
+    none.  Safe when several processes call it at once."""
+    if os.path.exists(LIB_PATH):
+        return LIB_PATH
+    os.makedirs(LIB_DIR, exist_ok=True)
+    with open(os.path.join(LIB_DIR, ".build_lock"), "w") as lock:
+        fcntl.flock(lock, fcntl.LOCK_EX)
+        if os.path.exists(DECODER_LIB_PATH):
+            return DECODER_LIB_PATH
+        return build_decoder_library()
+
+
+def _build(srcs, lib_path, verbose, jobs):
     os.makedirs(OBJ_DIR, exist_ok=True)
     os.makedirs(LIB_DIR, exist_ok=True)
-    srcs = sources()
     jobs = jobs or min(8, len(srcs))
     objs = []
     with concurrent.futures.ThreadPoolExecutor(max_workers=jobs) as ex:
@@ -66,11 +99,12 @@ def build_library(verbose=False, jobs=None):
             objs.append(obj)
             if verbose and log.strip():
                 print(log)
-    cmd = [_hipcc(), "-shared", "-fPIC", "--offload-arch=" + ARCH, "-o", LIB_PATH] + objs
+    cmd = [_hipcc(), "-shared", "-fPIC", "--offload-arch=" + ARCH, "-o", lib_path + ".part"] + objs
     p = subprocess.run(cmd, stdout=subprocess.PIPE, stderr=subprocess.STDOUT, text=True)
     if p.returncode != 0:
         raise RuntimeError("link failed:\n" + p.stdout)
-    return LIB_PATH
+    os.replace(lib_path + ".part", lib_path)
+    return lib_path
 
 
 if __name__ == "__main__":

@@ -15,7 +15,8 @@ namespace hip {
 
 enum DataType {
   kNotSupported = 0, kFloat32 = 1, kInt32 = 2, kInt64 = 3, kFloat16 = 4, kInt8 = 5, kInt16 = 6,
-  kByte = 7, kUInt8 = 8, kUInt16 = 9, kUInt32 = 10, kUInt64 = 11, kFloat64 = 12
+  kByte = 7, kUInt8 = 8, kUInt16 = 9, kUInt32 = 10, kUInt64 = 11, kFloat64 = 12,
+  kBFloat16 = 13  // not in the reference
 };
 
 // One input or output of a model: what the accessor functions of LSModel answer from.  `slot`
@@ -96,6 +97,19 @@ class LSModel {
 
 typedef LSModel* (*LSModelConstructor)(const std::string, const int);
 
+// What a model folder (config.json + weights) does not say about serving it.
+struct ModelOptions {
+  int max_batch_size = 8;
+  int max_step = 2048;          // positions a sequence can have
+  DataType dtype = kBFloat16;   // or kFloat32
+  int topk = 1;                 // 1: greedy; > 1: top-k; 0: top-p
+  float topp = 0.75f;
+  int eos_id = -1;              // -1: none
+  int padding_id = -1;          // right padding of short prompts, and of short results
+  int extra_decode_length = 64; // tokens generated after the longest prompt
+};
+typedef LSModel* (*LSModelDirConstructor)(const std::string, const ModelOptions&);
+
 class LSModelFactory {
  public:
   static LSModelFactory& GetInstance() {
@@ -111,16 +125,25 @@ class LSModelFactory {
     if (iter == object_map_.end()) throw std::runtime_error("Model not supported");
     return iter->second(weight_path, max_batch_size);
   }
+  // Models in folders are registered under the "architecture" of their config.json.
+  void ArchitectureRegister(std::string architecture, LSModelDirConstructor obj) {
+    if (obj) dir_map_.insert({architecture, obj});
+  }
+  LSModel* CreateFromDirectory(const std::string model_dir, const ModelOptions& options);
 
  private:
   LSModelFactory() {}
   std::map<std::string, LSModelConstructor> object_map_;
+  std::map<std::string, LSModelDirConstructor> dir_map_;
 };
 
 class Reflector {
  public:
   Reflector(std::string name, LSModelConstructor obj) {
     LSModelFactory::GetInstance().ModelRegister(name, obj);
+  }
+  Reflector(std::string architecture, LSModelDirConstructor obj) {
+    LSModelFactory::GetInstance().ArchitectureRegister(architecture, obj);
   }
 };
 
@@ -130,6 +153,21 @@ class Reflector {
     return new className(weight_path, max_batch_size);                                      \
   }                                                                                         \
   Reflector reflector_##className(#className, create_object_##className);
+
+// The class under its name (weight_path: the folder, default options) and as the architecture of
+// that name.
+#define LSMODEL_REGISTER_ARCHITECTURE(className)                                            \
+  LSModel* create_object_##className(const std::string path, const int max_batch_size) {    \
+    ModelOptions options;                                                                   \
+    options.max_batch_size = max_batch_size;                                                \
+    return new className(path, options);                                                    \
+  }                                                                                         \
+  LSModel* create_architecture_##className(const std::string path,                          \
+                                           const ModelOptions& options) {                   \
+    return new className(path, options);                                                    \
+  }                                                                                         \
+  Reflector reflector_##className(#className, create_object_##className);                   \
+  Reflector reflector_architecture_##className(#className, create_architecture_##className);
 
 }  // namespace hip
 }  // namespace lightseq

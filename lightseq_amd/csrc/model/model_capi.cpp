@@ -6,16 +6,14 @@
 #include "../../../include/lightseq_model.h"
 #include "../ls_launch.h"
 #include "ls_model.h"
-#include "quant_bert.h"
-#include "quant_gpt.h"
-#include "quant_transformer.h"
+#include "model_controls.h"
 
+using lightseq::hip::EncoderControls;
+using lightseq::hip::GenerationControls;
 using lightseq::hip::LSModel;
 using lightseq::hip::LSModelFactory;
-using lightseq::hip::QuantBert;
-using lightseq::hip::QuantBertEncoder;
-using lightseq::hip::QuantGpt;
-using lightseq::hip::QuantTransformer;
+using lightseq::hip::ModelOptions;
+using lightseq::hip::StepControls;
 
 struct ls_model {
   std::unique_ptr<LSModel> impl;
@@ -42,6 +40,12 @@ int copy_shape(const std::vector<int>& v, int* shape, int* ndim) {
   *ndim = (int)v.size();
   for (size_t i = 0; i < v.size(); ++i) shape[i] = v[i];
   return LSH_OK;
+}
+
+// an optional side of a model, or nullptr
+template <typename Side>
+Side* side_of(ls_model* model) {
+  return dynamic_cast<Side*>(model->impl.get());
 }
 
 #define NEED_MODEL(m) \
@@ -172,40 +176,22 @@ int ls_model_get_stream(ls_model* model, lsh_stream_t* stream) {
   return LSH_OK;
 }
 
-// the encoder stack of either model class, or nullptr
-static QuantBertEncoder* encoder_of(ls_model* model) {
-  if (QuantBert* qb = dynamic_cast<QuantBert*>(model->impl.get())) return qb->encoder();
-  if (QuantTransformer* qt = dynamic_cast<QuantTransformer*>(model->impl.get()))
-    return qt->encoder();
-  return nullptr;
-}
+#define NEED_SIDE(var, Side, message)            \
+  Side* var = side_of<Side>(model);              \
+  if (!var) return lsh::lsh_fail(LSH_ERR_UNSUPPORTED, message)
+#define NO_GENERATION "this model has no generation steps"
 
 int ls_model_set_profiling(ls_model* model, int on) {
   NEED_MODEL(model);
-  QuantBertEncoder* enc = encoder_of(model);
-  if (!enc) return lsh::lsh_fail(LSH_ERR_UNSUPPORTED, "this model has no profiled encoder stack");
-  return guarded([&] {
-    enc->set_profiling(on != 0);
-    enc->reset_profile();
-  });
+  NEED_SIDE(enc, EncoderControls, "this model has no profiled encoder stack");
+  return guarded([&] { enc->set_profiling(on != 0); });
 }
 
 int ls_model_get_profile(ls_model* model, char* buf, int capacity) {
   NEED_MODEL(model);
-  QuantBertEncoder* enc = encoder_of(model);
-  if (!enc) return lsh::lsh_fail(LSH_ERR_UNSUPPORTED, "this model has no profiled encoder stack");
+  NEED_SIDE(enc, EncoderControls, "this model has no profiled encoder stack");
   if (!buf || capacity <= 0) return lsh::lsh_fail(LSH_ERR_INVALID, "null buffer");
-  std::string out = "[";
-  bool first = true;
-  for (const auto& p : enc->profile()) {
-    if (!first) out += ",";
-    first = false;
-    out += "{\"site\":\"" + p.site + "\",\"kernel\":\"" + p.kernel + "\",\"m\":" +
-           std::to_string(p.m) + ",\"n\":" + std::to_string(p.n) + ",\"k\":" +
-           std::to_string(p.k) + ",\"launches\":" + std::to_string(p.launches) +
-           ",\"total_ms\":" + std::to_string(p.total_ms) + "}";
-  }
-  out += "]";
+  const std::string out = enc->profile_json();
   if ((int)out.size() + 1 > capacity) return lsh::lsh_fail(LSH_ERR_INVALID, "buffer too small");
   memcpy(buf, out.c_str(), out.size() + 1);
   return LSH_OK;
@@ -214,140 +200,72 @@ int ls_model_get_profile(ls_model* model, char* buf, int capacity) {
 int ls_model_set_tap(ls_model* model, int layer, const char* name, void* dst) {
   NEED_MODEL(model);
   if (!name) return lsh::lsh_fail(LSH_ERR_INVALID, "null pointer");
-  if (!strcmp(name, "enc_out")) {
-    QuantTransformer* qt = dynamic_cast<QuantTransformer*>(model->impl.get());
-    if (!qt) return lsh::lsh_fail(LSH_ERR_UNSUPPORTED, "enc_out is a QuantTransformer tap");
-    qt->set_encoder_output_tap(static_cast<__half*>(dst));
+  // "dec.<name>": an intermediate of a generation step (layer `layer`, at the step given to
+  // ls_model_set_tap_step)
+  if (!strncmp(name, "dec.", 4)) {
+    NEED_SIDE(gen, GenerationControls, NO_GENERATION);
+    gen->step_taps().set(layer, name + 4, dst);
     return LSH_OK;
   }
-  // "dec.<name>": an intermediate of a generation step of QuantTransformer's decoder or of
-  // QuantGpt (layer `layer`, at the step given to ls_model_set_tap_step)
-  if (!strncmp(name, "dec.", 4)) {
-    if (QuantGpt* qg = dynamic_cast<QuantGpt*>(model->impl.get())) {
-      qg->encoder()->step_taps.set(layer, name + 4, dst);
-      return LSH_OK;
-    }
-    if (QuantTransformer* qt = dynamic_cast<QuantTransformer*>(model->impl.get())) {
-      qt->decoder()->step_taps.set(layer, name + 4, dst);
-      return LSH_OK;
-    }
-    return lsh::lsh_fail(LSH_ERR_UNSUPPORTED, "step taps belong to QuantTransformer and QuantGpt");
-  }
-  QuantBertEncoder* enc = encoder_of(model);
-  if (!enc) return lsh::lsh_fail(LSH_ERR_UNSUPPORTED, "this model has no tapped encoder stack");
-  auto& t = enc->taps;
-  t.tap_layer = layer;
-  int8_t* p = static_cast<int8_t*>(dst);
-  if (!strcmp(name, "ln1_q")) t.ln1_q = p;
-  else if (!strcmp(name, "qkv_q")) t.qkv_q = p;
-  else if (!strcmp(name, "ctx_q")) t.ctx_q = p;
-  else if (!strcmp(name, "out_q")) t.out_q = p;
-  else if (!strcmp(name, "ln2_q")) t.ln2_q = p;
-  else if (!strcmp(name, "ffn1_q")) t.ffn1_q = p;
-  else if (!strcmp(name, "act_q")) t.act_q = p;
-  else if (!strcmp(name, "ffn2_acc")) t.ffn2_acc = static_cast<int32_t*>(dst);
-  else if (!strcmp(name, "res_attn")) t.res_attn = static_cast<__half*>(dst);
-  else if (!strcmp(name, "res_ffn")) t.res_ffn = static_cast<__half*>(dst);
-  else return lsh::lsh_fail(LSH_ERR_INVALID, "unknown tap name");
+  NEED_SIDE(enc, EncoderControls, "this model has no tapped encoder stack");
+  if (!enc->set_encoder_tap(layer, name, dst))
+    return lsh::lsh_fail(LSH_ERR_INVALID, "unknown tap name");
   return LSH_OK;
 }
 
 int ls_model_set_tap_step(ls_model* model, int step) {
   NEED_MODEL(model);
-  if (QuantGpt* qg = dynamic_cast<QuantGpt*>(model->impl.get())) {
-    qg->encoder()->step_taps.set_step(step);
-    return LSH_OK;
-  }
-  if (QuantTransformer* qt = dynamic_cast<QuantTransformer*>(model->impl.get())) {
-    qt->decoder()->step_taps.set_step(step);
-    return LSH_OK;
-  }
-  return lsh::lsh_fail(LSH_ERR_UNSUPPORTED, "step taps belong to QuantTransformer and QuantGpt");
+  NEED_SIDE(gen, GenerationControls, NO_GENERATION);
+  gen->step_taps().set_step(step);
+  return LSH_OK;
 }
 
 int ls_model_set_step_record(ls_model* model, int8_t* logits, int* alive_seq, int max_steps) {
   NEED_MODEL(model);
   if (max_steps < 0) return lsh::lsh_fail(LSH_ERR_INVALID, "negative max_steps");
-  if (QuantGpt* qg = dynamic_cast<QuantGpt*>(model->impl.get())) {
-    qg->encoder()->set_step_record(logits, max_steps);
-    return LSH_OK;
-  }
-  QuantTransformer* qt = dynamic_cast<QuantTransformer*>(model->impl.get());
-  if (!qt)
+  NEED_SIDE(gen, GenerationControls, NO_GENERATION);
+  if (!gen->set_step_record(logits, alive_seq, max_steps))
     return lsh::lsh_fail(LSH_ERR_UNSUPPORTED,
                          "step records are a debug aid of QuantTransformer and QuantGpt");
-  qt->decoder()->set_step_record(logits, alive_seq, max_steps);
   return LSH_OK;
 }
 
 int ls_model_set_graph_mode(ls_model* model, int on) {
   NEED_MODEL(model);
-  if (QuantGpt* qg = dynamic_cast<QuantGpt*>(model->impl.get())) {
-    qg->encoder()->graph_mode(on != 0);
-    return LSH_OK;
-  }
-  if (QuantTransformer* qt = dynamic_cast<QuantTransformer*>(model->impl.get())) {
-    qt->decoder()->graph_mode(on != 0);
-    return LSH_OK;
-  }
-  return lsh::lsh_fail(LSH_ERR_UNSUPPORTED,
-                       "graph mode applies to the generation steps of QuantTransformer and QuantGpt");
+  NEED_SIDE(gen, GenerationControls, NO_GENERATION);
+  gen->graph_mode(on != 0);
+  return LSH_OK;
 }
 
 int ls_model_set_seed(ls_model* model, unsigned long long seed) {
   NEED_MODEL(model);
-  if (QuantGpt* qg = dynamic_cast<QuantGpt*>(model->impl.get()))
-    return guarded([&] { qg->encoder()->set_seed(seed); });
-  if (QuantTransformer* qt = dynamic_cast<QuantTransformer*>(model->impl.get()))
-    return guarded([&] { qt->decoder()->set_seed(seed); });
-  return lsh::lsh_fail(LSH_ERR_UNSUPPORTED,
-                       "a seed applies to the random sampling of QuantGpt and QuantTransformer");
+  NEED_SIDE(gen, GenerationControls, NO_GENERATION);
+  return guarded([&] { gen->set_seed(seed); });
 }
 
 int ls_model_get_graph_stats(ls_model* model, int* captured, long long* replayed) {
   NEED_MODEL(model);
   if (!captured || !replayed) return lsh::lsh_fail(LSH_ERR_INVALID, "null pointer");
-  if (QuantGpt* qg = dynamic_cast<QuantGpt*>(model->impl.get())) {
-    *captured = qg->encoder()->graphs_captured();
-    *replayed = qg->encoder()->graphs_replayed();
-    return LSH_OK;
-  }
-  if (QuantTransformer* qt = dynamic_cast<QuantTransformer*>(model->impl.get())) {
-    *captured = qt->decoder()->graphs_captured();
-    *replayed = qt->decoder()->graphs_replayed();
-    return LSH_OK;
-  }
-  return lsh::lsh_fail(LSH_ERR_UNSUPPORTED,
-                       "graph mode applies to the generation steps of QuantTransformer and QuantGpt");
+  NEED_SIDE(gen, GenerationControls, NO_GENERATION);
+  *captured = gen->graphs().captured();
+  *replayed = gen->graphs().replayed();
+  return LSH_OK;
 }
 
 int ls_model_get_graph_nodes(ls_model* model, int* nodes) {
   NEED_MODEL(model);
   if (!nodes) return lsh::lsh_fail(LSH_ERR_INVALID, "null pointer");
-  if (QuantGpt* qg = dynamic_cast<QuantGpt*>(model->impl.get())) {
-    *nodes = qg->encoder()->graph_nodes();
-    return LSH_OK;
-  }
-  if (QuantTransformer* qt = dynamic_cast<QuantTransformer*>(model->impl.get())) {
-    *nodes = qt->decoder()->graph_nodes();
-    return LSH_OK;
-  }
-  return lsh::lsh_fail(LSH_ERR_UNSUPPORTED,
-                       "graph mode applies to the generation steps of QuantTransformer and QuantGpt");
+  NEED_SIDE(gen, GenerationControls, NO_GENERATION);
+  *nodes = gen->graphs().last_graph_nodes();
+  return LSH_OK;
 }
 
 int ls_model_get_phase_times(ls_model* model, float* prepare_ms, float* steps_ms, int* steps) {
   NEED_MODEL(model);
   if (!prepare_ms || !steps_ms || !steps) return lsh::lsh_fail(LSH_ERR_INVALID, "null pointer");
-  const lightseq::hip::PhaseEvents* ph = nullptr;
-  if (QuantGpt* qg = dynamic_cast<QuantGpt*>(model->impl.get())) ph = &qg->encoder()->phases();
-  if (QuantTransformer* qt = dynamic_cast<QuantTransformer*>(model->impl.get()))
-    ph = &qt->decoder()->phases();
-  if (!ph)
-    return lsh::lsh_fail(LSH_ERR_UNSUPPORTED,
-                         "phase times exist for the generation models QuantTransformer and QuantGpt");
+  NEED_SIDE(gen, GenerationControls, NO_GENERATION);
   bool have = false;
-  const int rc = guarded([&] { have = ph->times(prepare_ms, steps_ms, steps); });
+  const int rc = guarded([&] { have = gen->phases().times(prepare_ms, steps_ms, steps); });
   if (rc != LSH_OK) return rc;
   if (!have) return lsh::lsh_fail(LSH_ERR_INVALID, "no generation run has completed yet");
   return LSH_OK;
@@ -356,16 +274,83 @@ int ls_model_get_phase_times(ls_model* model, float* prepare_ms, float* steps_ms
 int ls_model_get_steps_run(ls_model* model, int* steps) {
   NEED_MODEL(model);
   if (!steps) return lsh::lsh_fail(LSH_ERR_INVALID, "null pointer");
-  if (QuantGpt* qg = dynamic_cast<QuantGpt*>(model->impl.get())) {
-    *steps = qg->encoder()->steps_run();
-    return LSH_OK;
-  }
-  QuantTransformer* qt = dynamic_cast<QuantTransformer*>(model->impl.get());
-  if (!qt)
-    return lsh::lsh_fail(LSH_ERR_UNSUPPORTED,
-                         "step records are a debug aid of QuantTransformer and QuantGpt");
-  *steps = qt->decoder()->steps_run();
+  NEED_SIDE(gen, GenerationControls, NO_GENERATION);
+  *steps = gen->steps_run();
   return LSH_OK;
+}
+
+// ---- models in a folder, step-wise decoding ------------------------------------------------
+void ls_model_default_options(ls_model_options* o) {
+  if (!o) return;
+  const ModelOptions d;
+  o->max_batch_size = d.max_batch_size;
+  o->max_step = d.max_step;
+  o->dtype = (int)d.dtype;
+  o->topk = d.topk;
+  o->topp = d.topp;
+  o->eos_id = d.eos_id;
+  o->padding_id = d.padding_id;
+  o->extra_decode_length = d.extra_decode_length;
+}
+
+int ls_model_create_from_dir(const char* model_dir, const ls_model_options* o, ls_model** model) {
+  if (!model_dir || !model)
+    return lsh::lsh_fail(LSH_ERR_INVALID, "ls_model_create_from_dir: null argument");
+  *model = nullptr;
+  return guarded([&] {
+    ModelOptions opt;
+    if (o) {
+      opt.max_batch_size = o->max_batch_size;
+      opt.max_step = o->max_step;
+      opt.dtype = (lightseq::hip::DataType)o->dtype;
+      opt.topk = o->topk;
+      opt.topp = o->topp;
+      opt.eos_id = o->eos_id;
+      opt.padding_id = o->padding_id;
+      opt.extra_decode_length = o->extra_decode_length;
+    }
+    LSModel* p = LSModelFactory::GetInstance().CreateFromDirectory(model_dir, opt);
+    *model = new ls_model{std::unique_ptr<LSModel>(p), {}};
+  });
+}
+
+#define NO_STEPS "this model does not decode step by step"
+
+int ls_model_get_vocab_size(ls_model* model, int* size) {
+  NEED_MODEL(model);
+  if (!size) return lsh::lsh_fail(LSH_ERR_INVALID, "null pointer");
+  NEED_SIDE(st, StepControls, NO_STEPS);
+  *size = st->vocab_size();
+  return LSH_OK;
+}
+
+int ls_model_open_sequence(ls_model* model, int* slot) {
+  NEED_MODEL(model);
+  if (!slot) return lsh::lsh_fail(LSH_ERR_INVALID, "null pointer");
+  NEED_SIDE(st, StepControls, NO_STEPS);
+  return guarded([&] { *slot = st->open_sequence(); });
+}
+
+int ls_model_close_sequence(ls_model* model, int slot) {
+  NEED_MODEL(model);
+  NEED_SIDE(st, StepControls, NO_STEPS);
+  return guarded([&] { st->close_sequence(slot); });
+}
+
+int ls_model_step(ls_model* model, int entries, const int* slots, const int* counts,
+                  const int* tokens, int n_want, const int* want_rows, float* logits) {
+  NEED_MODEL(model);
+  NEED_SIDE(st, StepControls, NO_STEPS);
+  if (entries <= 0 || !slots || !counts || !tokens || n_want < 0 ||
+      (n_want > 0 && (!want_rows || !logits)))
+    return lsh::lsh_fail(LSH_ERR_INVALID, "ls_model_step: bad arguments");
+  return guarded([&] {
+    long rows = 0;
+    for (int i = 0; i < entries; ++i) rows += counts[i] > 0 ? counts[i] : 0;
+    st->step(std::vector<int>(slots, slots + entries), std::vector<int>(counts, counts + entries),
+             std::vector<int>(tokens, tokens + rows),
+             std::vector<int>(want_rows, want_rows + n_want), logits);
+  });
 }
 
 }  // extern "C"

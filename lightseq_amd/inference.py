@@ -22,6 +22,14 @@ _LS_MAX_DIMS = 8
 _NP_OF_DTYPE = {1: np.float32, 2: np.int32, 4: np.float16}
 _TORCH_OF_DTYPE = {1: torch.float32, 2: torch.int32, 4: torch.float16}
 
+class _ModelOptions(ctypes.Structure):  # ls_model_options
+    _fields_ = [("max_batch_size", _I), ("max_step", _I), ("dtype", _I), ("topk", _I),
+                ("topp", ctypes.c_float), ("eos_id", _I), ("padding_id", _I),
+                ("extra_decode_length", _I)]
+
+
+_FOLDER_DTYPES = {"float32": 1, "bfloat16": 13}
+
 _bound = False
 
 
@@ -62,11 +70,18 @@ def _bind():
         "ls_model_set_seed": [_P, ctypes.c_uint64],
         "ls_model_get_graph_stats": [_P, ip, ctypes.POINTER(ctypes.c_longlong)],
         "ls_model_get_graph_nodes": [_P, ip],
+        "ls_model_create_from_dir": [ctypes.c_char_p, ctypes.POINTER(_ModelOptions), pp],
+        "ls_model_get_vocab_size": [_P, ip],
+        "ls_model_open_sequence": [_P, ip],
+        "ls_model_close_sequence": [_P, _I],
+        "ls_model_step": [_P, _I, _P, _P, _P, _I, _P, _P],
     }
     for name, argtypes in sigs.items():
         fn = getattr(L, name)
         fn.restype = _I
         fn.argtypes = argtypes
+    L.ls_model_default_options.restype = None
+    L.ls_model_default_options.argtypes = [ctypes.POINTER(_ModelOptions)]
     _bound = True
     return L
 
@@ -77,6 +92,9 @@ class LSModel:
     def __init__(self, class_name, weight_path, max_batch_size):
         self._lib = _bind()
         self._h = _P()
+        self._create(class_name, weight_path, max_batch_size)
+
+    def _create(self, class_name, weight_path, max_batch_size):
         self._call("ls_model_create", class_name.encode(), str(weight_path).encode(),
                    int(max_batch_size), ctypes.byref(self._h))
 
@@ -185,7 +203,7 @@ class LSModel:
         return a.value, b.value, n.value
 
     def graph_mode(self, flag):
-        """QuantTransformer / QuantGpt: replay generation steps as HIP graphs."""
+        """Generation models: replay generation steps as HIP graphs."""
         self._call("ls_model_set_graph_mode", self._h, int(bool(flag)))
 
     def set_seed(self, seed):
@@ -312,3 +330,87 @@ class QuantGpt(_HostIOModel):
 
     def steps_run(self):
         return self._int("ls_model_get_steps_run")
+
+
+class DecoderModel(LSModel):
+    """A decoder-only language model in a folder (``config.json``, ``model.safetensors``); the
+    folder's ``"architecture"`` chooses the class behind it.
+
+    ``infer`` takes and returns int32 ``[batch, len]`` arrays, short rows padded on the right with
+    ``padding_id``; :meth:`generate` is the same with lists.  :meth:`step` feeds given tokens to
+    sequences that the caller opened."""
+
+    def __init__(self, model_dir, dtype="bfloat16", **options):
+        self._options = dict(options, dtype=_FOLDER_DTYPES[dtype])
+        super().__init__(None, model_dir, None)
+        self.padding_id = self._o.padding_id
+        self.vocab_size = self._int("ls_model_get_vocab_size")
+        self._device_io = None
+
+    def _create(self, _class_name, model_dir, _max_batch_size):
+        self._o = _ModelOptions()
+        self._lib.ls_model_default_options(ctypes.byref(self._o))
+        for k, v in self._options.items():
+            if k not in dict(_ModelOptions._fields_):
+                raise TypeError("unknown option %r" % k)
+            setattr(self._o, k, v)
+        self._call("ls_model_create_from_dir", str(model_dir).encode(), ctypes.byref(self._o),
+                   ctypes.byref(self._h))
+
+    def infer(self, token_ids):
+        a = np.ascontiguousarray(token_ids, dtype=np.int32)
+        if a.ndim != 2:
+            raise ValueError("token_ids must be a 2-D int32 array [batch, seq_len]")
+        if a.shape[0] > self._o.max_batch_size or a.shape[1] > self._o.max_step:
+            raise lib.LSHError(lib.LSH_ERR_INVALID, "input larger than the model's maximum shape",
+                               "infer")
+        n = self._o.max_batch_size * self._o.max_step
+        if self._device_io is None:
+            self._device_io = [torch.zeros(n, dtype=torch.int32, device="cuda:0") for _ in range(2)]
+            self.set_input_ptr(0, self._device_io[0].data_ptr())
+            self.set_output_ptr(0, self._device_io[1].data_ptr())
+        self._device_io[0][:a.size].copy_(torch.from_numpy(a.reshape(-1)))
+        torch.cuda.synchronize()
+        self.set_input_shape(0, a.shape)
+        self.infer_device()
+        shape = self.get_output_shape(0)
+        return self._device_io[1][:int(np.prod(shape))].reshape(shape).cpu().numpy()
+
+    def generate(self, prompts):
+        """Lists of ids -> lists of ids (prompt and continuation)."""
+        a = np.full((len(prompts), max(len(p) for p in prompts)), self.padding_id, np.int32)
+        for i, p in enumerate(prompts):
+            a[i, :len(p)] = p
+        out = []
+        for row in self.infer(a).tolist():
+            while row and row[-1] == self.padding_id:
+                row.pop()
+            out.append(row)
+        return out
+
+    # -- given tokens, step by step -------------------------------------------
+    def open_sequence(self):
+        return self._int("ls_model_open_sequence")
+
+    def close_sequence(self, slot):
+        self._call("ls_model_close_sequence", self._h, int(slot))
+
+    def step(self, entries, want=()):
+        """``entries``: [(slot, tokens)], one batch.  ``want``: rows, numbered through the entries'
+        tokens, whose logits come back as float32 ``[len(want), vocab]``."""
+        slots = np.array([e[0] for e in entries], np.int32)
+        counts = np.array([len(e[1]) for e in entries], np.int32)
+        tokens = np.concatenate([np.asarray(e[1], np.int32).reshape(-1) for e in entries])
+        rows = np.array(list(want), np.int32)
+        logits = np.empty((len(rows), self.vocab_size), np.float32)
+        p = lambda a: _P(a.ctypes.data if a.size else None)  # noqa: E731
+        self._call("ls_model_step", self._h, len(slots), p(slots), p(counts),
+                   p(np.ascontiguousarray(tokens)), len(rows), p(rows), p(logits))
+        return logits
+
+    def steps_run(self):
+        return self._int("ls_model_get_steps_run")
+
+
+class Sudevik(DecoderModel):
+    """Gated-delta and sliding-window-attention layers with mixtures of experts."""

@@ -165,23 +165,58 @@ _SIGNATURES = {
     "ls_destroy_layer": (False, "c" + "i"),
 }
 
+# floating-point decoder kernels (include/lightseq_lm.h): name -> (has _bf16/_f32 variants, codes)
+_LM_SIGNATURES = {
+    "lsh_lm_attn_pad": (False, "i"),
+    "lsh_lm_attn_decode_workspace": (False, "ip"),
+    "lsh_lm_delta_chunked_workspace": (False, "iip"),
+    "lsh_lm_delta_chunked_supported": (False, "p"),
+    "lsh_lm_moe_route": (False, "ppppp" + "iii" + "s"),
+    "lsh_lm_sample": (False, "p" + "iii" + "f" + "i" + "pp" + "i" + "pppp" + "s"),
+    "lsh_lm_gemm": (True, "plpplpliiiis"),
+    "lsh_lm_gemm_f32_out": (True, "plppiiis"),
+    "lsh_lm_gemm_planes": (True, "plppiiiips"),
+    "lsh_lm_moe_up": (True, "pppppiiiiis"),
+    "lsh_lm_moe_down": (True, "pppppiiiiis"),
+    "lsh_lm_norm": (True, "ppiillppppppiifppippis"),
+    "lsh_lm_attn_prepare": (True, "pliiippfpipppppips"),
+    "lsh_lm_attn_prefill": (True, "pppplippiipps"),
+    "lsh_lm_attn_decode": (True, "pppplipppiippps"),
+    "lsh_lm_delta_prepare": (True, "plpppppppppppiips"),
+    "lsh_lm_delta_scan": (True, "ppppppppips"),
+    "lsh_lm_delta_chunked": (True, "pppppppppiiips"),
+    "lsh_lm_delta_gated_norm": (True, "pplipfpips"),
+    "lsh_lm_delta_step": (True, "plipppppfpppppips"),
+}
+_LM_RETURNS_COUNT = ("lsh_lm_attn_decode_workspace", "lsh_lm_delta_chunked_workspace")
+
 _lib = None
 
 
-def load():
-    """Load the shared library (once).  Raises if it has not been built."""
+def load(path=None):
+    """Load the shared library (once).  Raises if it has not been built.  ``path``: a library with
+    the decoder models only (``build.ensure_decoder_library``), to be named at the first call."""
     global _lib
     if _lib is not None:
         return _lib
-    if not os.path.exists(LIB_PATH):
+    path = path or LIB_PATH
+    if not os.path.exists(path):
         raise RuntimeError(
             "%s is missing: build it with `python -m lightseq_amd.build` "
-            "(there is no CPU fallback)" % LIB_PATH)
-    lib = ctypes.CDLL(LIB_PATH)
+            "(there is no CPU fallback)" % path)
+    lib = ctypes.CDLL(path)
     lib.lsh_last_error.restype = ctypes.c_char_p
     lib.lsh_last_error.argtypes = []
     lib.lsh_version.restype = ctypes.c_char_p
     lib.lsh_version.argtypes = []
+    for name, (typed, codes) in _LM_SIGNATURES.items():
+        for suffix in (("_bf16", "_f32") if typed else ("",)):
+            fn = getattr(lib, name + suffix)
+            fn.restype = _L if name in _LM_RETURNS_COUNT else _I
+            fn.argtypes = [_CODES[c] for c in codes]
+    if os.path.basename(path) != os.path.basename(LIB_PATH):
+        _lib = lib
+        return lib
     lib.lsh_length_norm.restype = ctypes.c_float
     lib.lsh_length_norm.argtypes = [_I, _F]
     for name, (typed, codes) in _SIGNATURES.items():
