@@ -8,8 +8,9 @@ import re
 import pytest
 
 ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
-HEADERS = [os.path.join(ROOT, "include", h) for h in ("lightseq_hip.h", "lightseq_ops.h", "lightseq_model.h")]
-PROTO_RE = re.compile(r"^\s*(?:const\s+char\s*\*|int|float)\s+((?:lsh|ls)_\w+)\s*\(([^;]*?)\)\s*;",
+HEADERS = [os.path.join(ROOT, "include", h) for h in ("lightseq_hip.h", "lightseq_ops.h", "lightseq_model.h",
+                                                      "lightseq_lm.h")]
+PROTO_RE = re.compile(r"^\s*(?:const\s+char\s*\*|int|float|int64_t|void)\s+((?:lsh|ls)_\w+)\s*\(([^;]*?)\)\s*;",
                       re.M | re.S)
 
 
@@ -67,11 +68,18 @@ def test_ctypes_table_matches_header():
             assert full in protos, full
             want = "".join(_code(a) for a in protos[full].split(","))
             assert want == codes, (full, want, codes)
+    lm = {}
+    for name, (typed, codes) in lib._LM_SIGNATURES.items():
+        for suffix in (("_bf16", "_f32") if typed else ("",)):
+            full = name + suffix
+            lm[full] = "".join(_code(a) for a in protos[full].split(","))
+            assert lm[full] == codes, (full, lm[full], codes)
+    assert set(lm) == {n for n in protos if n.startswith("lsh_lm_")}
     # and nothing in lightseq_hip.h / lightseq_ops.h is left unbound
     bound = {n + s for n, (t, _) in lib._SIGNATURES.items() for s in (("_f16", "_f32") if t else ("",))}
     kernels_header = re.sub(r"/\*.*?\*/", "", open(HEADERS[0]).read() + open(HEADERS[1]).read(),
                             flags=re.S)
-    declared = {n for n, _ in PROTO_RE.findall(kernels_header)} - {"lsh_last_error", "lsh_version",
+    declared = {n for n, _ in PROTO_RE.findall(kernels_header)} - {"lsh_last_error", "lsh_version", "lsh_beam_search_step_workspace",
                                                                          "lsh_length_norm"}
     assert declared == bound, declared ^ bound
 
