@@ -42,6 +42,11 @@ workloads (beam-search translation, greedy GPT generation) through ``QuantTransf
 decode step between HIP events on the model's stream, its launches, a roofline block (one step's
 algorithmic HBM bytes -- weights, cached keys and values, logits -- against 8 TB/s) and the CPU
 oracle on a few steps of the same width.  The default line carries both under ``generation``.
+
+``--workload sudevik`` times the bfloat16 Sudevik decoder (``lightseq_amd.synthetic`` sizes) beside
+``QuantGpt`` of the same width, depth, heads, vocabulary and active feed-forward size: prompt tokens/s
+and decode-step time of each, from HIP events on the model's stream around the prompt pass and the step
+loop of whole ``Infer()`` calls.
 """
 import argparse
 import json
@@ -753,6 +758,121 @@ def bench_generation(workload, steps, warmup, graphs=False, with_cpu=True):
     return out
 
 
+# (batch, prompt, generated tokens) of the Sudevik comparison: a long prompt batch, a decoding batch
+SUDEVIK_SHAPES = [(8, 1024, 32), (32, 256, 64)]
+
+
+def _sudevik_work(cfg, batch, prompt, new):
+    """Multiply-add work of the prompt pass (x 2) and algorithmic HBM bytes of a decode step: every
+    weight that a step of this batch touches once (experts: the expected number of distinct ones), the
+    visible keys and values, recurrent states read and written."""
+    W, V = cfg["width"], cfg["vocab"]
+    macs = nbytes = 0.0
+    for l in cfg["layers"]:
+        m = l["mixer"]
+        H, G, D, VD = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+        if l["type"] == "attention":
+            own = m.get("kv_from") is None
+            proj = W * (H * D + H * VD + (G * (D + VD) if own else 0)) + W * H * VD
+            win = m["mask"]["size"] + m["mask"]["keep_first"]
+            seen = sum(min(i + 1, win) for i in range(prompt)) / prompt
+            macs += H * (D + VD) * seen
+            nbytes += 2 * batch * G * (D + VD) * min(win, prompt + new / 2)
+        else:
+            C = 2 * G * D + H * VD
+            proj = W * (C + H * VD + 2 * H) + W * H * VD
+            macs += 3 * H * D * VD  # read, write, read-out of the state
+            nbytes += batch * (8 * H * D * VD + 2 * C * m["conv"])
+        E, top, ff = l["mlp"]["router"]["experts"], l["mlp"]["router"]["top"], l["mlp"]["expert"]["ff"]
+        macs += proj + W * E + 3 * top * W * ff
+        hit = E * (1 - (1 - top / E) ** batch)
+        nbytes += 2 * (proj + W * E + 3 * hit * W * ff)
+    return 2 * macs * batch * prompt, nbytes + 2 * W * V + 4 * batch * V
+
+
+def _time_decoder(model, batch, prompt, new, upload, steps, warmup):
+    """Mean (prompt ms, ms per decode step, launches of a step) over whole Infer() calls."""
+    import numpy as np
+    model.benchmark_mode(True)
+    upload()
+    model.graph_mode(True)
+    for _ in range(2):
+        model.infer_device()
+    launches = model.graph_nodes()
+    model.graph_mode(False)
+    for _ in range(warmup):
+        model.infer_device()
+    times = []
+    for _ in range(steps):
+        model.infer_device()
+        a, b, n = model.phase_times()
+        times.append((a, b / n))
+    a, b = np.median(np.array(times), axis=0)
+    return {"prompt_ms": float(a), "prompt_tokens_per_s": batch * prompt / (a * 1e-3),
+            "ms_per_decode_step": float(b), "decode_tokens_per_s": batch / (b * 1e-3),
+            "launches_per_step": launches}
+
+
+def bench_sudevik(args):
+    import shutil
+    import numpy as np
+    from lightseq_amd import inference, synthetic
+    out = {"metric": "decoder throughput beside QuantGpt", "dtype": "bf16 (QuantGpt: int8)", "data": "synthetic",
+           "n_gpus": 1, "steps": args.steps, "warmup": args.warmup, "results": []}
+    rng = np.random.default_rng(0)
+    for size in args.sizes.split(","):
+        cfg = synthetic.sudevik_config(size)
+        L, W, V = len(cfg["layers"]), cfg["width"], cfg["vocab"]
+        H = cfg["layers"][0]["mixer"]["heads"]
+        mlp = cfg["layers"][0]["mlp"]
+        inner = 3 * mlp["router"]["top"] * mlp["expert"]["ff"] // 2  # the same active weights
+        folder = tempfile.mkdtemp(prefix="ls_bench_")
+        try:
+            if args.only != "gpt":
+                synthetic.write_sudevik(folder, cfg)
+            for batch, prompt, new in SUDEVIK_SHAPES:
+                res = {"size": size, "layers": L, "width": W, "heads": H, "vocab": V, "active_ffn": inner,
+                       "batch": batch, "prompt": prompt, "new": new}
+                ids = rng.integers(0, V - 1, size=(batch, prompt), dtype=np.int32)
+                if args.only != "gpt":
+                    m = inference.DecoderModel(folder, max_batch_size=batch, max_step=prompt + new,
+                                               extra_decode_length=new)
+
+                    def upload():
+                        m.benchmark_mode(True)
+                        m.infer(ids)
+                    r = _time_decoder(m, batch, prompt, new, upload, args.steps, args.warmup)
+                    m.close()
+                    flop, nbytes = _sudevik_work(cfg, batch, prompt, new)
+                    r["prompt_tflops"] = flop / (r["prompt_ms"] * 1e-3) / 1e12
+                    r["prompt_frac_of_2500_tflops"] = r["prompt_tflops"] / 2500
+                    r["decode_gbs"] = nbytes / (r["ms_per_decode_step"] * 1e-3) / 1e9
+                    r["decode_frac_of_hbm"] = r["decode_gbs"] / HBM_PEAK_GBS
+                    res["sudevik"] = r
+                if args.only != "sudevik":
+                    g = dict(n_layer=L, hidden=W, inner=inner, head_num=H, max_step=prompt + new, vocab=V,
+                             padding_id=V - 1, eos_id=V - 1, topk=1, extra_decode_length=new, sampling_method="topk")
+                    path = os.path.join(folder, "gpt.pb")
+                    synthetic.write_quant_gpt(path, g, seed=0)
+                    m = inference.QuantGpt(path, batch)
+                    os.remove(path)
+                    r = _time_decoder(m, batch, prompt, new, lambda: m._upload(ids), args.steps, args.warmup)
+                    m.close()
+                    per_tok = L * (4 * W * W + 2 * W * inner + 2 * W * (prompt + 1) / 2)
+                    r["prompt_tops"] = 2 * per_tok * batch * prompt / (r["prompt_ms"] * 1e-3) / 1e12
+                    r["prompt_frac_of_5000_tops"] = r["prompt_tops"] / INT8_MFMA_PEAK_TOPS
+                    nbytes = L * (4 * W * W + 2 * W * inner) + V * W + L * batch * 2 * W * (prompt + new / 2) \
+                        + 2 * batch * V
+                    r["decode_gbs"] = nbytes / (r["ms_per_decode_step"] * 1e-3) / 1e9
+                    r["decode_frac_of_hbm"] = r["decode_gbs"] / HBM_PEAK_GBS
+                    res["quant_gpt"] = r
+                out["results"].append(res)
+                print(json.dumps(res), file=sys.stderr, flush=True)
+        finally:
+            shutil.rmtree(folder, ignore_errors=True)
+    return out
+
+
 def _leave():
     """Nothing may outlive the command: no helper thread or OpenMP team keeps the interpreter alive.  Under a
     profiler (rocprofv3 exports ROCP* variables) the process ends the ordinary way instead: the tool writes its
@@ -770,7 +890,7 @@ def main():
     ap.add_argument("--steps", type=int, default=None)
     ap.add_argument("--warmup", type=int, default=None)
     ap.add_argument("--workload", default="bert_base",
-                    choices=["bert_base", "transformer_big", "gpt2_medium"])
+                    choices=["bert_base", "transformer_big", "gpt2_medium", "sudevik"])
     ap.add_argument("--no-cpu-baseline", action="store_true")
     ap.add_argument("--no-fused", action="store_true",
                     help="skip the stand-alone timing of the fused kernels")
@@ -778,6 +898,8 @@ def main():
                     help="default workload: skip the two generation workloads of the `generation` block")
     ap.add_argument("--ffn-segment", action="store_true",
                     help="A/B and phase stamps of the one-launch feed-forward segment (not the headline line)")
+    ap.add_argument("--only", default="", help="sudevik workload: one of sudevik, gpt (for a profiler run)")
+    ap.add_argument("--sizes", default="base,large", help="sudevik workload: configurations to time")
     ap.add_argument("--graphs", action="store_true",
                     help="generation workloads: replay the steps as HIP graphs (ls_model_set_graph_mode)")
     ap.add_argument("--copy-calibration", action="store_true",
@@ -806,6 +928,10 @@ def main():
         torch.cuda.synchronize()
     if args.ffn_segment:
         print(json.dumps(bench_ffn_segment(args)))
+        _leave()
+        return
+    if args.workload == "sudevik":
+        print(json.dumps(bench_sudevik(args)))
         _leave()
         return
     out = bench_bert(args) if bert else bench_generation(args.workload, args.steps, args.warmup,

@@ -59,6 +59,10 @@ int lsh_lm_gemm_planes_f32(const void* A, int64_t lda, const void* W, float* C, 
     int K, int max_planes, int* planes_used, lsh_stream_t stream);
 int lsh_lm_gemm_planes_bf16(const void* A, int64_t lda, const void* W, float* C, int M, int N,
     int K, int max_planes, int* planes_used, lsh_stream_t stream);
+int lsh_lm_moe_router_f32(const void* h, const void* w, const float* bias, float* weight, int* count,
+    int* list, int tokens, int width, int experts, int top, lsh_stream_t stream);
+int lsh_lm_moe_router_bf16(const void* h, const void* w, const float* bias, float* weight, int* count,
+    int* list, int tokens, int width, int experts, int top, lsh_stream_t stream);
 int lsh_lm_moe_up_f32(const void* h, const void* w, void* act, const int* count, const int* list,
     int tokens, int top, int experts, int width, int ff, lsh_stream_t stream);
 int lsh_lm_moe_up_bf16(const void* h, const void* w, void* act, const int* count, const int* list,

@@ -131,6 +131,103 @@ delta_prepare_kernel(const T* __restrict__ proj, long ld, const float* __restric
   }
 }
 
+// The same for head sizes, columns and row lengths in fours: LPH lanes per head, four channels per
+// lane, 64 / LPH heads per wavefront.  The last block row computes the gates.
+template <typename T, int NT, int LPH>
+__global__ void __launch_bounds__(256)
+delta_prepare4_kernel(const T* __restrict__ proj, long ld, const float* __restrict__ ba,
+                      const float* __restrict__ conv_w, const float* __restrict__ a_log,
+                      const float* __restrict__ dt_bias, const T* __restrict__ ring,
+                      float* __restrict__ q, float* __restrict__ k, T* __restrict__ v,
+                      float* __restrict__ log_g, float* __restrict__ beta,
+                      const SeqSpan* __restrict__ seqs, DeltaShape sh) {
+  const SeqSpan sq = seqs[blockIdx.z];
+  const int t0 = blockIdx.x * kConvTile;
+  if (t0 >= sq.n) return;
+  const int t1 = min(t0 + kConvTile, sq.n);
+  const int G = sh.kv_heads, H = sh.heads, D = sh.dim, VD = sh.vdim;
+  if (blockIdx.y == gridDim.y - 1) {
+    for (int x = threadIdx.x; x < (t1 - t0) * H; x += 256) {
+      const int t = x / H, h = x - t * H;
+      const long row = sq.row0 + t0 + t;
+      const float b = ba[row * 2 * H + h], a = ba[row * 2 * H + H + h];
+      beta[row * H + h] = sigmoid_f(b);
+      log_g[row * H + h] = -expf(a_log[h]) * softplus_f(a + dt_bias[h]);
+    }
+    return;
+  }
+  const int unit_raw = (int)(blockIdx.y * 256 + threadIdx.x) / LPH;
+  const int unit = min(unit_raw, 2 * G + H - 1);
+  const bool is_v = unit >= 2 * G;
+  const int n = is_v ? VD : D, d = (threadIdx.x % LPH) * 4;
+  const int ch = (is_v ? 2 * G * D + (unit - 2 * G) * VD : unit * D) + d;  // first of four channels
+  const bool in = unit_raw < 2 * G + H && d < n;
+  const int C = sh.channels();
+  float w[NT][4], x[NT][4];  // window: x[NT - 1] is the current token
+  auto load = [&](int t, float (&o)[4]) {
+    const int p = sq.pos0 + t;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) o[e] = 0.f;
+    if (in && p >= 0) {
+      if (t >= 0) ldv<4, T>(proj + (sq.row0 + t) * ld + ch, o);
+      else ldv<4, T>(ring + ((long)sq.slot * sh.taps + p % sh.taps) * C + ch, o);
+    }
+  };
+#pragma unroll
+  for (int s = 0; s < NT; ++s) {
+    const int lag = NT - 1 - s;  // tokens back
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      w[s][e] = in && lag < sh.taps ? conv_w[(long)(ch + e) * sh.taps + sh.taps - 1 - lag] : 0.f;
+      x[s][e] = 0.f;
+    }
+    if (lag > 0 && lag < sh.taps) load(t0 - lag, x[s]);
+  }
+  float nx[2][4];
+  load(t0, nx[0]);
+  if (t0 + 1 < t1) load(t0 + 1, nx[1]);
+  for (int t = t0; t < t1; ++t) {
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      x[NT - 1][e] = nx[0][e];
+      nx[0][e] = nx[1][e];
+    }
+    if (t + 2 < t1) load(t + 2, nx[1]);
+    float y[4], ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      float c = 0.f;
+#pragma unroll
+      for (int s = 0; s < NT; ++s) c = fmaf(w[s][e], x[s][e], c);
+      y[e] = silu_f(c);
+      ss += y[e] * y[e];
+    }
+    ss += dpp_f<kDppXor1>(ss);
+    ss += dpp_f<kDppXor2>(ss);
+    ss += dpp_f<kDppHalfMirror>(ss);
+    ss += dpp_f<kDppMirror>(ss);
+    if (LPH > 16) ss += __shfl_xor(ss, 16);
+    if (LPH > 32) ss += __shfl_xor(ss, 32);
+    const long row = sq.row0 + t;
+    if (in) {
+      if (is_v) {
+        stv<4, T>(v + row * H * VD + (unit - 2 * G) * VD + d, y);
+      } else {
+        const bool is_q = unit < G;
+        float r = 1.0f / sqrtf(ss + 1e-6f);
+        if (is_q) r *= 1.0f / sqrtf((float)D);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) y[e] *= r;
+        stv<4, float>((is_q ? q + (row * G + unit) * D : k + (row * G + unit - G) * D) + d, y);
+      }
+    }
+#pragma unroll
+    for (int s = 0; s < NT - 1; ++s)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) x[s][e] = x[s + 1][e];
+  }
+}
+
 // inputs of the span's last taps positions into the ring (its older readers have finished: stream order)
 template <typename T>
 __global__ void __launch_bounds__(256)
@@ -383,6 +480,7 @@ delta_chunk_scan_kernel(const float* __restrict__ q, const float* __restrict__ k
                         float* __restrict__ o, const SeqSpan* __restrict__ seqs, int vblocks,
                         DeltaShape sh) {
   constexpr int MAXD = 64 * NDW, SS = MAXD + 4, US = kC + 4, NS = 4 * NDW;
+  constexpr bool PREFETCH = NDW <= 2;  // two chunks' operands fit the registers
   __shared__ __attribute__((aligned(16))) float St[NVB * 16][SS], Ut[NVB * 16][US],
       Ud[NVB * 16][US];
   const int H = sh.heads, D = sh.dim, VD = sh.vdim, G = sh.kv_heads;
@@ -455,11 +553,8 @@ delta_chunk_scan_kernel(const float* __restrict__ q, const float* __restrict__ k
     a.b4 = *reinterpret_cast<const f32x4*>(pb + w * 16 + 4 * qd);
     a.b_last = pb[kC - 1];
   };
-  Ops cur, nxt;
-  fetch(0, cur);
-  __syncthreads();
-  for (int ch = 0; ch < chunks; ++ch) {
-    if (ch + 1 < chunks) fetch(ch + 1, nxt);
+  auto chunk = [&](int ch, const Ops& cur, Ops& nxt) {
+    if (PREFETCH && ch + 1 < chunks) fetch(ch + 1, nxt);
     const int n = min(kC, sq.n - ch * kC);
     f32x4 ws_acc[NVB], o_acc[NVB];
 #pragma unroll
@@ -517,7 +612,21 @@ delta_chunk_scan_kernel(const float* __restrict__ q, const float* __restrict__ k
       }
     }
     __syncthreads();
-    cur = nxt;
+  };
+  Ops ops[PREFETCH ? 2 : 1];
+  if constexpr (PREFETCH) {
+    fetch(0, ops[0]);
+    __syncthreads();
+    for (int ch = 0; ch < chunks; ch += 2) {
+      chunk(ch, ops[0], ops[1]);
+      if (ch + 1 < chunks) chunk(ch + 1, ops[1], ops[0]);
+    }
+  } else {
+    __syncthreads();
+    for (int ch = 0; ch < chunks; ++ch) {
+      fetch(ch, ops[0]);
+      chunk(ch, ops[0], ops[0]);
+    }
   }
 #pragma unroll
   for (int i = 0; i < NDW; ++i)
@@ -561,6 +670,37 @@ delta_gated_norm_kernel(const float* __restrict__ o, const T* __restrict__ proj,
       const int d = 2 * (i * 64 + lane) + e;
       if (d < VD) out[unit * VD + d] = from_f<T>(x[i][e] * r * norm_w[d] * silu_f(to_f(gate[d])));
     }
+}
+
+// LPH lanes per head, four elements per lane
+template <typename T, int LPH>
+__global__ void __launch_bounds__(256)
+delta_gated_norm4_kernel(const float* __restrict__ o, const T* __restrict__ proj, long ld, int g_col,
+                         const float* __restrict__ norm_w, float eps, T* __restrict__ out, int units,
+                         DeltaShape sh) {
+  const int unit_raw = (int)((blockIdx.x * 256 + threadIdx.x) / LPH);
+  const int unit = min(unit_raw, units - 1), VD = sh.vdim, d = (threadIdx.x % LPH) * 4;
+  const int row = unit / sh.heads, h = unit - row * sh.heads;
+  float x[4] = {0.f, 0.f, 0.f, 0.f}, z[4], w[4];
+  const bool in = d < VD;
+  if (in) {
+    ldv<4, float>(o + (long)unit * VD + d, x);
+    ldv<4, T>(proj + row * ld + g_col + h * VD + d, z);
+    ldv<4, float>(norm_w + d, w);
+  }
+  float ss = x[0] * x[0] + x[1] * x[1] + x[2] * x[2] + x[3] * x[3];
+  ss += dpp_f<kDppXor1>(ss);
+  ss += dpp_f<kDppXor2>(ss);
+  ss += dpp_f<kDppHalfMirror>(ss);
+  ss += dpp_f<kDppMirror>(ss);
+  if (LPH > 16) ss += __shfl_xor(ss, 16);
+  if (LPH > 32) ss += __shfl_xor(ss, 32);
+  const float r = 1.0f / sqrtf(ss / (float)VD + eps);
+  if (in && unit_raw < units) {
+#pragma unroll
+    for (int e = 0; e < 4; ++e) x[e] = x[e] * r * w[e] * silu_f(z[e]);
+    stv<4, T>(out + (long)unit * VD + d, x);
+  }
 }
 
 // ------------------------------------------------------------------------------------------------
@@ -700,9 +840,25 @@ int delta_prepare(const T* proj, long ld, const float* ba, const float* conv_w, 
   if (!proj || !ba || !conv_w || !a_log || !dt_bias || !conv_ring || !q || !k || !v || !log_g ||
       !beta || !seqs || n_seqs <= 0 || max_n <= 0 || n_seqs > 65535)
     return lsh_fail(LSH_ERR_INVALID, "delta_prepare: bad arguments");
-  const dim3 grid((max_n + kConvTile - 1) / kConvTile, (2 * sh.kv_heads + sh.heads + 1 + 3) / 4,
-                  n_seqs);
-  if (sh.taps <= 4)
+  const int tiles = (max_n + kConvTile - 1) / kConvTile, units = 2 * sh.kv_heads + sh.heads;
+  const dim3 grid(tiles, (units + 1 + 3) / 4, n_seqs);
+  if (sh.dim % 4 == 0 && sh.vdim % 4 == 0 && ld % 4 == 0) {
+    const int wide = std::max(sh.dim, sh.vdim);
+#define PREP4(NT, LPH)                                                                             \
+  delta_prepare4_kernel<T, NT, LPH><<<dim3(tiles, (units * LPH + 255) / 256 + 1, n_seqs), 256, 0,  \
+                                      s>>>(proj, ld, ba, conv_w, a_log, dt_bias, conv_ring, q, k,  \
+                                           v, log_g, beta, seqs, sh)
+#define PREP4_T(LPH)                  \
+  do {                                \
+    if (sh.taps <= 4) PREP4(4, LPH);  \
+    else PREP4(8, LPH);               \
+  } while (0)
+    if (wide <= 64) PREP4_T(16);
+    else if (wide <= 128) PREP4_T(32);
+    else PREP4_T(64);
+#undef PREP4_T
+#undef PREP4
+  } else if (sh.taps <= 4)
     delta_prepare_kernel<T, 4><<<grid, 256, 0, s>>>(proj, ld, ba, conv_w, a_log, dt_bias, conv_ring,
                                                     q, k, v, log_g, beta, seqs, sh);
   else
@@ -782,6 +938,16 @@ int delta_gated_norm(const float* o, const T* proj, long ld, int g_col, const fl
   if (!o || !proj || !norm_w || !out || rows <= 0)
     return lsh_fail(LSH_ERR_INVALID, "delta_gated_norm: bad arguments");
   const long units = (long)rows * sh.heads;
+  if (sh.vdim % 4 == 0 && ld % 4 == 0 && g_col % 4 == 0 && units < (1L << 24)) {
+#define NORM4(LPH)                                                                        \
+  delta_gated_norm4_kernel<T, LPH><<<(unsigned)((units * LPH + 255) / 256), 256, 0, s>>>( \
+      o, proj, ld, g_col, norm_w, eps, out, (int)units, sh)
+    if (sh.vdim <= 64) NORM4(16);
+    else if (sh.vdim <= 128) NORM4(32);
+    else NORM4(64);
+#undef NORM4
+    return lsh_check_launch("delta_gated_norm4_kernel");
+  }
   delta_gated_norm_kernel<T><<<(unsigned)((units + 3) / 4), 256, 0, s>>>(o, proj, ld, g_col, norm_w,
                                                                         eps, out, units, sh);
   return lsh_check_launch("delta_gated_norm_kernel");

@@ -82,6 +82,69 @@ attn_prepare_kernel(const T* __restrict__ proj, long ld, int q_col, int k_col, i
   }
 }
 
+// The same for head sizes, columns and row lengths in fours: LPH lanes per head, four elements (two
+// pairs) per lane, 64 / LPH heads per wavefront.
+template <typename T, int LPH>
+__global__ void __launch_bounds__(256)
+attn_prepare4_kernel(const T* __restrict__ proj, long ld, int q_col, int k_col, int v_col,
+                     const float* __restrict__ q_norm, const float* __restrict__ k_norm, float eps,
+                     const float2* __restrict__ cos_sin, int rot_pairs, T* __restrict__ q_out,
+                     T* __restrict__ k_cache, T* __restrict__ v_cache,
+                     const int* __restrict__ row_slot, const int* __restrict__ row_pos, int units,
+                     int heads_per_row, AttnShape sh) {
+  const int unit_raw = (int)((blockIdx.x * 256 + threadIdx.x) / LPH);
+  const int unit = min(unit_raw, units - 1);  // every lane takes part in the exchanges
+  const int d = (threadIdx.x % LPH) * 4;
+  const int row = unit / heads_per_row;
+  int head = unit - row * heads_per_row;
+  const int pos = row_pos[row];
+  const T* src = proj + row * ld;
+  int kind = 0;
+  T* dst;
+  if (head < sh.heads) {
+    src += q_col + head * sh.dim;
+    dst = q_out + ((long)row * sh.heads + head) * sh.dim_pad;
+  } else {
+    head -= sh.heads;
+    kind = head < sh.kv_heads ? 1 : 2;
+    if (kind == 2) head -= sh.kv_heads;
+    src += kind == 1 ? k_col + head * sh.dim : v_col + head * sh.vdim;
+    const long at = ((long)row_slot[row] * sh.kv_heads + head) * sh.max_step + pos;
+    dst = kind == 1 ? k_cache + at * sh.dim_pad : v_cache + at * sh.vdim_pad;
+  }
+  const int n = kind == 2 ? sh.vdim : sh.dim, pad = kind == 2 ? sh.vdim_pad : sh.dim_pad;
+  float u[4] = {0.f, 0.f, 0.f, 0.f};
+  if (d < n) ldv<4, T>(src + d, u);
+  float ss = u[0] * u[0] + u[1] * u[1] + u[2] * u[2] + u[3] * u[3];
+  ss += dpp_f<kDppXor1>(ss);
+  ss += dpp_f<kDppXor2>(ss);
+  ss += dpp_f<kDppHalfMirror>(ss);
+  ss += dpp_f<kDppMirror>(ss);
+  if (LPH > 16) ss += __shfl_xor(ss, 16);
+  if (LPH > 32) ss += __shfl_xor(ss, 32);
+  if (kind != 2) {
+    const float r = 1.0f / sqrtf(ss / (float)n + eps);
+    const float* w = kind == 0 ? q_norm : k_norm;
+    if (w && d < n) {
+      float wv[4];
+      ldv<4, float>(w + d, wv);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) u[e] = u[e] * r * wv[e];
+    }
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      const int p = d / 2 + i;
+      if (p < rot_pairs) {
+        const float2 cs = cos_sin[(long)pos * rot_pairs + p];
+        const float a = u[2 * i], b = u[2 * i + 1];
+        u[2 * i] = a * cs.x - b * cs.y;
+        u[2 * i + 1] = b * cs.x + a * cs.y;
+      }
+    }
+  }
+  if (unit_raw < units && d < pad) stv<4, T>(dst + d, u);
+}
+
 // ------------------------------------------------------------------------------------------------
 // Prompt kernel.  A workgroup takes 128 queries of one (sequence, head), 32 per wavefront, and walks
 // the key tiles of 64 that any of them sees: first the kept tokens, then the window.  Scores are
@@ -308,23 +371,54 @@ int launch_prefill(const T* q, const T* kc, const T* vc, const T* proj, long ld,
 }
 
 // ------------------------------------------------------------------------------------------------
-// One-token kernel.  A workgroup takes up to R query heads of one (row, kv head) and one part of the
-// visible keys, in chunks of 256: 16 lanes per key form the scores, the chunk's soft-max runs over
-// LDS, then the same 16-lane groups accumulate the values.  The visible keys are numbered
-// 0 .. n_vis - 1, the kept ones first.
-constexpr int kChunk = 256;
+// One-token kernel.  A workgroup of 8 wavefronts takes up to R query heads of one (row, kv head) and
+// one part of the visible keys (numbered 0 .. n_vis - 1, the kept ones first).  16 lanes share a key;
+// such a group keeps the running soft-max of the keys it has seen in registers, so nothing is
+// exchanged until the end, and it requests the keys and values of its next turn before it computes
+// on the present ones.
+constexpr int kDecThreads = 512, kDecGroups = kDecThreads / 16;
+
+// N consecutive elements in 4-byte words, converted when they are used
+template <typename T, int N>
+struct Packed {
+  static constexpr int W = N * (int)sizeof(T) / 4;
+  uint32_t w[W];
+  __device__ __forceinline__ void load(const T* p) {  // 4-byte aligned
+    if constexpr (W % 4 == 0) {
+#pragma unroll
+      for (int i = 0; i < W; i += 4) {
+        const frag_t t = *reinterpret_cast<const frag_t*>(reinterpret_cast<const uint32_t*>(p) + i);
+#pragma unroll
+        for (int k = 0; k < 4; ++k) w[i + k] = t[k];
+      }
+    } else if constexpr (W % 2 == 0) {
+#pragma unroll
+      for (int i = 0; i < W; i += 2) {
+        const uint2 t = *reinterpret_cast<const uint2*>(reinterpret_cast<const uint32_t*>(p) + i);
+        w[i] = t.x;
+        w[i + 1] = t.y;
+      }
+    } else {
+#pragma unroll
+      for (int i = 0; i < W; ++i) w[i] = reinterpret_cast<const uint32_t*>(p)[i];
+    }
+  }
+  __device__ __forceinline__ float get(int e) const {
+    if constexpr (sizeof(T) == 4) return __builtin_bit_cast(float, w[e]);
+    else return __builtin_bit_cast(float, e & 1 ? w[e >> 1] & 0xffff0000u : w[e >> 1] << 16);
+  }
+};
 
 template <typename T, int EK, int EV, int R>  // elements per lane of a key / value row
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(kDecThreads)
 attn_decode_kernel(const T* __restrict__ q, const T* __restrict__ k_cache,
                    const T* __restrict__ v_cache, const T* __restrict__ proj, long ld, int g_col,
                    T* __restrict__ out, const int* __restrict__ row_slot,
                    const int* __restrict__ row_pos, int nsplit, int head_groups,
                    float* __restrict__ workspace, AttnShape sh, AttnMask mask) {
   constexpr int DP = EK * 16, VP = EV * 16;
-  __shared__ float sc[R][kChunk];
-  __shared__ float fac[R], mrow[R], lrow[R];
-  __shared__ float part[4][R][VP];
+  constexpr int U = (EK + EV) * (int)sizeof(T) > 64 ? 2 : 4;  // keys per group and turn
+  __shared__ float part[8][R][VP], pm[8][R], pl[8][R];
   const int row = blockIdx.x, kvh = blockIdx.y / head_groups, hg = blockIdx.y % head_groups;
   const int split = blockIdx.z;
   const int rep = sh.heads / sh.kv_heads;
@@ -340,132 +434,123 @@ attn_decode_kernel(const T* __restrict__ q, const T* __restrict__ k_cache,
   const int per = ((n_vis + nsplit - 1) / nsplit + 15) & ~15;
   const int v_lo = min(split * per, n_vis), v_hi = min(v_lo + per, n_vis);
 
-  float qv[R][EK], acc[R][EV];
+  Packed<T, EK> kb[2][U];
+  Packed<T, EV> vb[2][U];
+  auto fetch = [&](int c0, Packed<T, EK> (&ko)[U], Packed<T, EV> (&vo)[U]) {
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int v = min(c0 + u * kDecGroups + grp, v_hi - 1);
+      const long key = v < kept ? v : lo + v - kept;
+      ko[u].load(kc + key * DP);
+      vo[u].load(vc + key * VP);
+    }
+  };
+  if (v_lo < v_hi) fetch(v_lo, kb[0], vb[0]);
+
+  float qv[R][EK], acc[R][EV], m[R], l[R];
 #pragma unroll
   for (int r = 0; r < R; ++r) {
-    const T* qr = q + ((long)row * sh.heads + h0 + min(r, nh - 1)) * DP + j * EK;
+    Packed<T, EK> t;
+    t.load(q + ((long)row * sh.heads + h0 + min(r, nh - 1)) * DP + j * EK);
 #pragma unroll
-    for (int e = 0; e < EK; e += 2) {
-      float t[2];
-      ldv<2, T>(qr + e, t);
-      qv[r][e] = t[0] * mask.scale * 1.44269504088896340736f;
-      qv[r][e + 1] = t[1] * mask.scale * 1.44269504088896340736f;
-    }
+    for (int e = 0; e < EK; ++e) qv[r][e] = t.get(e) * (mask.scale * 1.44269504088896340736f);
 #pragma unroll
     for (int e = 0; e < EV; ++e) acc[r][e] = 0.f;
+    m[r] = -INFINITY;
+    l[r] = 0.f;
   }
-  if (tid < R) {
-    const bool sink = mask.sink && split == 0;
-    mrow[tid] = sink ? 0.f : -INFINITY;
-    lrow[tid] = sink ? 1.f : 0.f;
-  }
-  auto key_of = [&](int v) { return v < kept ? v : lo + v - kept; };
-  for (int c0 = v_lo; c0 < v_hi; c0 += kChunk) {
-    const int n = min(kChunk, v_hi - c0);
-    __syncthreads();
-    for (int i = grp; i < n; i += 64) {  // four keys per turn: their loads are in flight together
-      float kv[4][EK];
+  auto turn = [&](int c0, const Packed<T, EK> (&ki)[U], const Packed<T, EV> (&vi)[U]) {
+    float s[U][R];
 #pragma unroll
-      for (int u = 0; u < 4; ++u) {
-        const T* kr = kc + (long)key_of(c0 + min(i + 16 * u, n - 1)) * DP;
+    for (int u = 0; u < U; ++u) {
+      const bool in = c0 + u * kDecGroups + grp < v_hi;
 #pragma unroll
-        for (int e = 0; e < EK; e += 2) {
-          float t[2];
-          ldv<2, T>(kr + e, t);
-          kv[u][e] = t[0];
-          kv[u][e + 1] = t[1];
-        }
-      }
+      for (int r = 0; r < R; ++r) {
+        float d = 0.f;
 #pragma unroll
-      for (int u = 0; u < 4; ++u)
-#pragma unroll
-        for (int r = 0; r < R; ++r) {
-          float d = 0.f;
-#pragma unroll
-          for (int e = 0; e < EK; ++e) d = fmaf(qv[r][e], kv[u][e], d);
-          d += dpp_f<kDppXor1>(d);
-          d += dpp_f<kDppXor2>(d);
-          d += dpp_f<kDppHalfMirror>(d);
-          d += dpp_f<kDppMirror>(d);
-          if (j == 0 && i + 16 * u < n) sc[r][i + 16 * u] = d;
-        }
-    }
-    __syncthreads();
-    for (int r = wave; r < R; r += 4) {
-      float mx = -INFINITY;
-      for (int i = lane; i < n; i += 64) mx = fmaxf(mx, sc[r][i]);
-      mx = fmaxf(wave_max_dpp(mx), mrow[r]);
-      float sum = 0.f;
-      for (int i = lane; i < n; i += 64) {
-        const float e = exp2_f(sc[r][i] - mx);
-        sc[r][i] = e;
-        sum += e;
-      }
-      sum = wave_sum_dpp(sum);
-      if (lane == 0) {
-        const float f = mrow[r] == -INFINITY ? 0.f : exp2_f(mrow[r] - mx);
-        fac[r] = f;
-        lrow[r] = lrow[r] * f + sum;
-        mrow[r] = mx;
+        for (int e = 0; e < EK; ++e) d = fmaf(qv[r][e], ki[u].get(e), d);
+        d += dpp_f<kDppXor1>(d);
+        d += dpp_f<kDppXor2>(d);
+        d += dpp_f<kDppHalfMirror>(d);
+        d += dpp_f<kDppMirror>(d);
+        s[u][r] = in ? d : -INFINITY;
       }
     }
-    __syncthreads();
 #pragma unroll
     for (int r = 0; r < R; ++r) {
-      const float f = fac[r];
+      float mx = m[r];
+#pragma unroll
+      for (int u = 0; u < U; ++u) mx = fmaxf(mx, s[u][r]);
+      const float ref = mx == -INFINITY ? 0.f : mx;  // nothing seen yet: all weights are zero
+      const float f = exp2_f(m[r] - ref);
+      m[r] = mx;
+      l[r] *= f;
 #pragma unroll
       for (int e = 0; e < EV; ++e) acc[r][e] *= f;
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        const float p = exp2_f(s[u][r] - ref);
+        l[r] += p;
+#pragma unroll
+        for (int e = 0; e < EV; ++e) acc[r][e] = fmaf(p, vi[u].get(e), acc[r][e]);
+      }
     }
-    for (int i = grp; i < n; i += 64) {
-      float vv[4][EV];
-#pragma unroll
-      for (int u = 0; u < 4; ++u) {
-        const T* vr = vc + (long)key_of(c0 + min(i + 16 * u, n - 1)) * VP;
-#pragma unroll
-        for (int e = 0; e < EV; e += 2) {
-          float t[2];
-          ldv<2, T>(vr + e, t);
-          vv[u][e] = t[0];
-          vv[u][e + 1] = t[1];
-        }
-      }
-#pragma unroll
-      for (int u = 0; u < 4; ++u) {
-        const bool in = i + 16 * u < n;
-#pragma unroll
-        for (int r = 0; r < R; ++r) {
-          const float p = in ? sc[r][i + 16 * u] : 0.f;
-#pragma unroll
-          for (int e = 0; e < EV; ++e) acc[r][e] = fmaf(p, vv[u][e], acc[r][e]);
-        }
-      }
+  };
+  constexpr int STEP = U * kDecGroups;
+  for (int c0 = v_lo; c0 < v_hi; c0 += 2 * STEP) {
+    if (c0 + STEP < v_hi) fetch(c0 + STEP, kb[1], vb[1]);
+    turn(c0, kb[0], vb[0]);
+    if (c0 + STEP < v_hi) {
+      if (c0 + 2 * STEP < v_hi) fetch(c0 + 2 * STEP, kb[0], vb[0]);
+      turn(c0 + STEP, kb[1], vb[1]);
     }
   }
-  // the 16 groups' contexts: over the wavefront's four by lane exchange, then over LDS
+  // merge the groups: the wavefront's four by lane exchange, the wavefronts over LDS
 #pragma unroll
-  for (int r = 0; r < R; ++r)
+  for (int r = 0; r < R; ++r) {
+    float mx = fmaxf(m[r], __shfl_xor(m[r], 16));
+    mx = fmaxf(mx, __shfl_xor(mx, 32));
+    const float f = m[r] == -INFINITY ? 0.f : exp2_f(m[r] - mx);
+    float t = l[r] * f;
+    t += __shfl_xor(t, 16);
+    t += __shfl_xor(t, 32);
 #pragma unroll
     for (int e = 0; e < EV; ++e) {
-      float a = acc[r][e];
+      float a = acc[r][e] * f;
       a += __shfl_xor(a, 16);
       a += __shfl_xor(a, 32);
       if (lane < 16) part[wave][r][j * EV + e] = a;
     }
+    if (lane == 0) {
+      pm[wave][r] = mx;
+      pl[wave][r] = t;
+    }
+  }
   __syncthreads();
-  for (int x = tid; x < nh * VP; x += 256) {
+  const bool sink = mask.sink && split == 0;
+  for (int x = tid; x < nh * VP; x += kDecThreads) {
     const int r = x / VP, c = x - r * VP;
-    const float a = (part[0][r][c] + part[1][r][c]) + (part[2][r][c] + part[3][r][c]);
+    float mx = sink ? 0.f : -INFINITY;
+#pragma unroll
+    for (int w = 0; w < 8; ++w) mx = fmaxf(mx, pm[w][r]);
+    float a = 0.f, t = sink ? exp2_f(-mx) : 0.f;
+#pragma unroll
+    for (int w = 0; w < 8; ++w) {
+      const float f = pm[w][r] == -INFINITY ? 0.f : exp2_f(pm[w][r] - mx);
+      a = fmaf(f, part[w][r][c], a);
+      t = fmaf(f, pl[w][r], t);
+    }
     const int head = h0 + r;
     if (nsplit > 1) {
       // [row][head][split][VP + 2]: context, maximum, sum
-      float* w = workspace + (((long)row * sh.heads + head) * nsplit + split) * (VP + 2);
-      w[c] = a;
+      float* ws = workspace + (((long)row * sh.heads + head) * nsplit + split) * (VP + 2);
+      ws[c] = a;
       if (c == 0) {
-        w[VP] = mrow[r];
-        w[VP + 1] = lrow[r];
+        ws[VP] = mx;
+        ws[VP + 1] = t;
       }
     } else if (c < sh.vdim) {
-      float o = a / lrow[r];
+      float o = a / t;
       if (g_col >= 0) o *= sigmoid_f(to_f(proj[(long)row * ld + g_col + head * sh.vdim + c]));
       out[(long)row * sh.heads * sh.vdim + head * sh.vdim + c] = from_f<T>(o);
     }
@@ -519,6 +604,20 @@ int attn_prepare(const T* proj, long ld, int q_col, int k_col, int v_col, const 
     return lsh_fail(LSH_ERR_INVALID, "attn_prepare: bad arguments");
   const int per_row = sh.heads + (k_col >= 0 ? 2 * sh.kv_heads : 0);
   const long units = (long)rows * per_row;
+  const bool own = k_col >= 0;
+  if (sh.dim % 4 == 0 && ld % 4 == 0 && q_col % 4 == 0 && units < (1L << 24) &&
+      (!own || (sh.vdim % 4 == 0 && k_col % 4 == 0 && v_col % 4 == 0))) {
+    const int pad = own ? std::max(sh.dim_pad, sh.vdim_pad) : sh.dim_pad;
+#define PREP4(LPH)                                                                              \
+  attn_prepare4_kernel<T, LPH><<<(unsigned)((units * LPH + 255) / 256), 256, 0, s>>>(           \
+      proj, ld, q_col, k_col, v_col, q_norm, k_norm, eps, cos_sin, rot_pairs, q_out, k_cache,   \
+      v_cache, row_slot, row_pos, (int)units, per_row, sh)
+    if (pad <= 64) PREP4(16);
+    else if (pad <= 128) PREP4(32);
+    else PREP4(64);
+#undef PREP4
+    return lsh_check_launch("attn_prepare4_kernel");
+  }
   attn_prepare_kernel<T><<<(unsigned)((units + 3) / 4), 256, 0, s>>>(
       proj, ld, q_col, k_col, v_col, q_norm, k_norm, eps, cos_sin, rot_pairs, q_out, k_cache,
       v_cache, row_slot, row_pos, units, per_row, sh);
@@ -558,7 +657,7 @@ size_t attn_decode_workspace(int rows, const AttnShape& sh) {
 }
 
 #define DEC(EK, EV, R)                                                                           \
-  attn_decode_kernel<T, EK, EV, R><<<grid, 256, 0, s>>>(q, k_cache, v_cache, proj, ld, g_col,    \
+  attn_decode_kernel<T, EK, EV, R><<<grid, kDecThreads, 0, s>>>(q, k_cache, v_cache, proj, ld, g_col,    \
                                                         out, row_slot, row_pos, nsplit, groups,  \
                                                         workspace, sh, mask)
 #define DEC_R(EK, EV)                                                                            \
@@ -588,10 +687,11 @@ int attn_decode(const T* q, const T* k_cache, const T* v_cache, const T* proj, l
   const int groups = (rep + R - 1) / R;
   const long most = mask.window > 0 ? std::min((long)max_len, (long)mask.window + mask.keep_first)
                                     : (long)max_len;
-  // enough workgroups to fill the chip, parts of at least 128 keys
+  // enough workgroups to fill the chip, but parts of at least 1024 keys: a shorter part is done
+  // before the launch that would join the parts has started
   const int want = (int)((2L * cu_count() + (long)rows * sh.kv_heads * groups - 1) /
                          ((long)rows * sh.kv_heads * groups));
-  const int nsplit = (int)std::max(1L, std::min({(long)kMaxSplit, (long)want, most / 128}));
+  const int nsplit = (int)std::max(1L, std::min({(long)kMaxSplit, (long)want, most / 1024}));
   if ((long)sh.kv_heads * groups > 65535) return lsh_fail(LSH_ERR_UNSUPPORTED, "attn_decode: heads");
   const dim3 grid(rows, sh.kv_heads * groups, nsplit);
   switch (sh.dim_pad / 16) {

@@ -67,6 +67,12 @@ int lsh_lm_sample(const float* logits, int rows, int vocab, int topk, float topp
     return gemm_float_planes<T>((const T*)A, lda, (const T*)W, C, M, N, K, max_planes,             \
                                 planes_used, HS(s));                                               \
   }                                                                                                \
+  int lsh_lm_moe_router_##SUF(const void* h, const void* w, const float* bias, float* weight,       \
+                              int* count, int* list, int tokens, int width, int experts, int top,  \
+                              lsh_stream_t s) {                                                    \
+    return moe_router<T>((const T*)h, (const T*)w, bias, weight, count, list, tokens, width,       \
+                         experts, top, HS(s));                                                     \
+  }                                                                                                \
   int lsh_lm_moe_up_##SUF(const void* h, const void* w, void* act, const int* count,               \
                           const int* list, int tokens, int top, int experts, int width, int ff,    \
                           lsh_stream_t s) {                                                        \

@@ -44,6 +44,10 @@ int moe_down(const T* act, const T* w, TO* out, const int* count, const int* lis
 // over them; fills the lists above.  count must be zero before (lm_norm's zero_count does it).
 int moe_route(const float* logits, const float* bias, float* weight, int* count, int* list,
               int tokens, int experts, int top, hipStream_t s);
+// the logits' product (float32 sums of h and w as they are) and the same choice, for few tokens
+template <typename T>
+int moe_router(const T* h, const T* w, const float* bias, float* weight, int* count, int* list,
+               int tokens, int width, int experts, int top, hipStream_t s);
 
 // ---- norms on the residual stream (lm_norm_kernels.hip) ---------------------------------------
 // What is added to the residual row before the norm: parts many summands, part p of row r at

@@ -37,9 +37,27 @@ struct SampleLds {
 // the first candidate in that order which comes after (z, id)
 __device__ Best next_best(const float* lr, int vocab, float z, int id, SampleLds& sh) {
   Best b{-INFINITY, 0x7fffffff};
-  for (int v = threadIdx.x; v < vocab; v += blockDim.x) {
-    const float x = lr[v];
-    if (before(z, id, x, v) && before(x, v, b.z, b.id)) b = Best{x, v};
+  if (vocab % 4 == 0) {  // rows start at 16 bytes
+    const int quads = vocab / 4;
+    for (int v0 = threadIdx.x; v0 < quads; v0 += 4 * blockDim.x) {
+      float4 t[4];
+#pragma unroll
+      for (int u = 0; u < 4; ++u)
+        t[u] = reinterpret_cast<const float4*>(lr)[min(v0 + u * (int)blockDim.x, quads - 1)];
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        const int v = min(v0 + u * (int)blockDim.x, quads - 1) * 4;
+        const float x[4] = {t[u].x, t[u].y, t[u].z, t[u].w};
+#pragma unroll
+        for (int k = 0; k < 4; ++k)
+          if (before(z, id, x[k], v + k) && before(x[k], v + k, b.z, b.id)) b = Best{x[k], v + k};
+      }
+    }
+  } else {
+    for (int v = threadIdx.x; v < vocab; v += blockDim.x) {
+      const float x = lr[v];
+      if (before(z, id, x, v) && before(x, v, b.z, b.id)) b = Best{x, v};
+    }
   }
   b = wave_best(b);
   const int wid = threadIdx.x >> 6, nw = blockDim.x >> 6;

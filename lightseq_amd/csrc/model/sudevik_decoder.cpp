@@ -257,10 +257,15 @@ class Stack : public SudevikStack {
   // _h -> weighted expert outputs
   AddSpec experts(const SudevikLayerConfig& l, const SudevikLayerWeight<T>& w, int R, bool few) {
     const int W = _c.width;
-    LSH_CALL((gemm_float<T, float>(_h.get(), W, w.router.get(), _router.get(), l.experts, nullptr, 0,
-                                   l.experts, R, l.experts, W, _stream)));
-    LSH_CALL(moe_route(_router.get(), w.router_b.get(), _weight.get(), _count.get(), _list.get(), R,
-                       l.experts, l.top, _stream));
+    if (few) {
+      LSH_CALL(moe_router<T>(_h.get(), w.router.get(), w.router_b.get(), _weight.get(), _count.get(),
+                             _list.get(), R, W, l.experts, l.top, _stream));
+    } else {
+      LSH_CALL((gemm_float<T, float>(_h.get(), W, w.router.get(), _router.get(), l.experts, nullptr,
+                                     0, l.experts, R, l.experts, W, _stream)));
+      LSH_CALL(moe_route(_router.get(), w.router_b.get(), _weight.get(), _count.get(), _list.get(),
+                         R, l.experts, l.top, _stream));
+    }
     LSH_CALL(moe_up<T>(_h.get(), w.up.get(), _act.get(), _count.get(), _list.get(), R, l.top,
                        l.experts, W, l.ff, _stream));
     AddSpec add;

@@ -176,6 +176,7 @@ _LM_SIGNATURES = {
     "lsh_lm_gemm": (True, "plpplpliiiis"),
     "lsh_lm_gemm_f32_out": (True, "plppiiis"),
     "lsh_lm_gemm_planes": (True, "plppiiiips"),
+    "lsh_lm_moe_router": (True, "pppppp" + "iiii" + "s"),
     "lsh_lm_moe_up": (True, "pppppiiiiis"),
     "lsh_lm_moe_down": (True, "pppppiiiiis"),
     "lsh_lm_norm": (True, "ppiillppppppiifppippis"),

@@ -329,3 +329,107 @@ def write_quant_gpt(path, cfg, seed=0, ln_noise=0.02, w_std=None):
     with open(path, "wb") as f:
         f.write(proto.encode("QuantGpt", msg))
     return msg
+
+
+# ---- decoder models in folders (config.json + model.safetensors) ---------------------------------
+def sudevik_config(name):
+    """Shapes of the named synthetic Sudevik decoders: two gated-delta layers to one attention layer."""
+    def layers(n, heads, delta, attn, window, mlp):
+        out = []
+        for i in range(n):
+            if i % 3 == 2:
+                m = dict(heads=heads, scale=attn["dim"] ** -0.5, mask=dict(size=window, keep_first=4),
+                         rot=dict(base=1e6, dims=attn["dim"],
+                                  scaling=dict(factor=4.0, original=4096, fast=32.0, slow=1.0)), **attn)
+                if i == n - 1:
+                    m["kv_from"] = i - 3
+                out.append({"type": "attention", "mixer": m, "mlp": mlp})
+            else:
+                out.append({"type": "delta", "mixer": dict(heads=heads, conv=4, **delta), "mlp": mlp})
+        return out
+
+    def moe(experts, top, ff):
+        return {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top}}
+    cfgs = {
+        "base": dict(vocab=32000, width=1024,
+                     layers=layers(12, 16, dict(kv_heads=8, dim=64, vdim=64),
+                                   dict(kv_heads=4, dim=64, vdim=64), 512, moe(16, 2, 1024))),
+        "large": dict(vocab=32000, width=2048,
+                      layers=layers(6, 16, dict(kv_heads=8, dim=128, vdim=128),
+                                    dict(kv_heads=4, dim=128, vdim=128), 1024, moe(16, 2, 2048))),
+    }
+    return dict(cfgs[name], architecture="Sudevik", norm={"eps": 1e-6})
+
+
+def sudevik_shapes(cfg):
+    """name -> shape of every tensor of a Sudevik model."""
+    W, V, t = cfg["width"], cfg["vocab"], {}
+
+    def norm(name):
+        t[name] = t[name + ".b"] = (W,)
+    t["embed"] = t["head"] = (V, W)
+    norm("final.norm")
+    for i, l in enumerate(cfg["layers"]):
+        p, m, q = "l%d." % i, l["mixer"], "l%d.mix." % i
+        H, G, D, VD = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+        for n in ("norm1", "norm1b") + (("norm2", "norm2b") if l.get("mlp") else ()):
+            norm(p + n)
+        if l["type"] == "attention":
+            t[q + "q"], t[q + "q.norm"] = (H * D, W), (D,)
+            if m.get("kv_from") is None:
+                t[q + "k"], t[q + "v"], t[q + "k.norm"] = (G * D, W), (G * VD, W), (D,)
+        else:
+            for n, rows in (("q", G * D), ("k", G * D), ("v", H * VD)):
+                t[q + n], t[q + n + ".conv"] = (rows, W), (rows, m["conv"])
+            t[q + "b"] = t[q + "a"] = (H, W)
+            t[q + "A_log"] = t[q + "dt_bias"] = (H,)
+            t[q + "norm"] = (VD,)
+        t[q + "g"], t[q + "o"] = (H * VD, W), (W, H * VD)
+        if l.get("mlp"):
+            E, ff = l["mlp"]["router"]["experts"], l["mlp"]["expert"]["ff"]
+            t[p + "mlp.router"], t[p + "mlp.router.b"] = (E, W), (E,)
+            for e in range(E):
+                for n, s in (("gate", (ff, W)), ("up", (ff, W)), ("down", (W, ff))):
+                    t["%smlp.e%d.%s" % (p, e, n)] = s
+    return t
+
+
+def write_sudevik(folder, cfg, seed=0):
+    """Random weights ~N(0, 1 / inputs) (norm weights 1, biases 0), bfloat16.  Large matrices are cut
+    from one pool of random numbers, scaled by powers of two in their exponents."""
+    import json
+    import os
+    rng = np.random.default_rng(seed)
+    pool = (rng.standard_normal(1 << 22, dtype=np.float32).view(np.uint32) >> 16).astype(np.uint16)
+    shapes = sudevik_shapes(cfg)
+    os.makedirs(folder, exist_ok=True)
+    with open(os.path.join(folder, "config.json"), "w") as f:
+        json.dump(cfg, f)
+    head, at = {}, 0
+    for name, s in shapes.items():
+        n = 2 * int(np.prod(s))
+        head[name] = {"dtype": "BF16", "shape": list(s), "data_offsets": [at, at + n]}
+        at += n
+    h = json.dumps(head).encode()
+    h += b" " * (-len(h) % 8)
+    with open(os.path.join(folder, "model.safetensors"), "wb") as f:
+        f.write(len(h).to_bytes(8, "little") + h)
+        for name, s in shapes.items():
+            n = int(np.prod(s))
+            if len(s) == 1:
+                one = name.endswith("norm") or name[:-1].endswith("norm1") or ".norm" in name
+                v = 0x3f80 if one and not name.endswith(".b") else 0
+                if name.endswith("A_log"):
+                    v = 0xbf80
+                f.write(np.full(n, v, np.uint16).tobytes())
+                continue
+            drop = 0 if name.endswith(".conv") else int(round(0.5 * np.log2(s[-1])))
+            scaled = pool - np.uint16(drop << 7)
+            start = int(rng.integers(0, len(pool)))
+            left = n
+            while left:
+                part = scaled[start:start + left]
+                f.write(part.tobytes())
+                left -= len(part)
+                start = 0
+    return cfg

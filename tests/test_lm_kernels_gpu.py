@@ -100,8 +100,21 @@ def test_gemm(dt, m, n, k, split):
 
 
 # -- routing and experts --------------------------------------------------------------------------
-@pytest.mark.parametrize("tokens,experts,top", [(1, 1, 1), (37, 5, 3), (64, 64, 8), (9, 200, 17), (300, 513, 2)])
+@pytest.mark.parametrize("tokens,experts,top", [(1, 1, 1), (37, 5, 3), (64, 64, 8), (9, 200, 17), (300, 513, 2),
+                                                (513, 16, 2), (1001, 200, 5), (700, 600, 3)])
 def test_route(tokens, experts, top):
+    check_route(tokens, experts, top, None, 0)
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("tokens,experts,top,width", [(1, 1, 1, 64), (37, 5, 3, 75), (64, 70, 8, 1024), (9, 200, 17, 40),
+                                                      (3, 513, 2, 136)])
+def test_router(dt, tokens, experts, top, width):
+    check_route(tokens, experts, top, dt, width)
+
+
+def check_route(tokens, experts, top, dt, width):
+    """The choice from given logits, or (dt) from the rows and the router's weights."""
     r = rng(tokens)
     z = r.normal(size=(tokens, experts)).astype(np.float32)
     z[:, experts // 2] = z[:, 0]  # equal logits
@@ -109,7 +122,14 @@ def test_route(tokens, experts, top):
     bias[experts // 2] = bias[0]
     w = torch.zeros(tokens, top, device="cuda")
     count, lst = ints(np.zeros(experts)), ints(np.full((experts, tokens), -1))
-    call("lsh_lm_moe_route", dev(z), dev(bias), w, count, lst, tokens, experts, top)
+    if dt is None:
+        call("lsh_lm_moe_route", dev(z), dev(bias), w, count, lst, tokens, experts, top)
+    else:
+        # small integers: every order of addition gives the same logits, equal ones included
+        h, wr = r.integers(-2, 3, (tokens, width)), r.integers(-2, 3, (experts, width))
+        wr[experts // 2] = wr[0]
+        z = (h @ wr.T).astype(np.float32)
+        call("lsh_lm_moe_router_" + dt, dev(h, dt), dev(wr, dt), dev(bias), w, count, lst, tokens, width, experts, top)
     w, count, lst = host(w), count.cpu().numpy(), lst.cpu().numpy()
     seen = {}
     for e in range(experts):
@@ -335,6 +355,7 @@ DECODE = [
     (3, 1, 20, 27, [6, 7, 8, 9, 200], 7, 2), (9, 1, 128, 200, [318, 17], 100, 60),
     (2, 2, 256, 40, [0, 255, 256, 257], 256, 1), (1, 1, 33, 256, [50], 1, 3),
     (5, 1, 64, 96, [1500, 1023, 1024, 3, 2000], 1024, 5), (16, 2, 128, 128, [2047, 100], 0, 0),
+    (2, 1, 64, 64, [5000, 1100, 2303], 0, 0), (1, 1, 96, 128, [4100, 2], 3000, 7),
 ]
 
 
