@@ -262,18 +262,20 @@ gemm_tile_kernel(GemmArgs a, int tiles_m, int tiles_n) {
 }
 
 // ------------------------------------------------------------------------------------------------
-// 16 columns per workgroup, groups of 16 * MB rows.  The weight fragment is the first operand: lane
+// 16 * NS columns per workgroup (kDense; several strips share the activations), groups of 16 * MB
+// rows.  The weight fragment is the first operand: lane
 // (c = lane % 16, q = lane / 16) holds column n0 + c's 16-byte chunk q of a 64-byte K slice.
-template <typename T, typename TO, int MODE, int MB>
+template <typename T, typename TO, int MODE, int MB, int NS = 1>
 __global__ void __launch_bounds__(256)
 gemm_skinny_kernel(GemmArgs a) {
-  constexpr int NB = MODE == kMoeUp ? 2 : 1;
+  static_assert(NS == 1 || MODE == kDense, "strips of one matrix");
+  constexpr int NB = MODE == kMoeUp ? 2 : NS;
   constexpr int V = FT<T>::kVec;
   constexpr int U = 4;  // 64-byte slices per turn: 256 bytes of every row
   __shared__ float red[4][NB][MB][16][17];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int c = lane & 15, q = lane >> 4;
-  const int n0 = blockIdx.x * 16;
+  const int n0 = blockIdx.x * 16 * NS;
   RowSet rs{0, 0, a.M};
   int k_lo = 0, k_hi = a.K;
   if (MODE != kDense) {
@@ -288,7 +290,9 @@ gemm_skinny_kernel(GemmArgs a) {
   if (MODE != kDense) W += (long)rs.expert * NB * a.N * a.K;
   const T* wrow[NB];
 #pragma unroll
-  for (int j = 0; j < NB; ++j) wrow[j] = W + (long)(min(n0 + c, a.N - 1) + j * a.N) * a.K;
+  for (int j = 0; j < NB; ++j)
+    wrow[j] = W + (MODE == kMoeUp ? (long)(min(n0 + c, a.N - 1) + j * a.N)
+                                  : (long)min(n0 + j * 16 + c, a.N - 1)) * a.K;
   const T* A = reinterpret_cast<const T*>(a.A);
   const int first_end = rs.last;
   for (int first = 0; first < first_end; first += 16 * MB) {
@@ -328,23 +332,30 @@ gemm_skinny_kernel(GemmArgs a) {
 #pragma unroll
         for (int v = 0; v < 4; ++v) red[wave][j][i][c][4 * q + v] = acc[j][i][v];
     __syncthreads();
-    const int n = n0 + (tid & 15), r = tid >> 4;
+    const int r = tid >> 4;
 #pragma unroll
     for (int i = 0; i < MB; ++i) {
       const int row = first + i * 16 + r;
-      if (row < rs.last && n < a.N) {
-        float s[NB];
+      if (row >= rs.last) continue;
+      float s[NB];
 #pragma unroll
-        for (int j = 0; j < NB; ++j)
-          s[j] = (red[0][j][i][r][tid & 15] + red[1][j][i][r][tid & 15]) +
-                 (red[2][j][i][r][tid & 15] + red[3][j][i][r][tid & 15]);
-        const long m = dst_row<MODE>(a, rs, row);
-        if constexpr (MODE == kMoeUp)
-          reinterpret_cast<TO*>(a.C)[m * a.ldc + n] = from_f<TO>(silu_f(s[0]) * s[1]);
-        else if (MODE == kDense && a.planes > 1)
-          reinterpret_cast<TO*>(a.C)[((long)blockIdx.y * a.M + m) * a.ldc + n] = from_f<TO>(s[0]);
-        else
-          store_col<TO>(a, m, n, s[0]);
+      for (int j = 0; j < NB; ++j)
+        s[j] = (red[0][j][i][r][tid & 15] + red[1][j][i][r][tid & 15]) +
+               (red[2][j][i][r][tid & 15] + red[3][j][i][r][tid & 15]);
+      const long m = dst_row<MODE>(a, rs, row);
+      if constexpr (MODE == kMoeUp) {
+        const int n = n0 + (tid & 15);
+        if (n < a.N) reinterpret_cast<TO*>(a.C)[m * a.ldc + n] = from_f<TO>(silu_f(s[0]) * s[NB - 1]);
+      } else {
+#pragma unroll
+        for (int j = 0; j < NB; ++j) {
+          const int n = n0 + j * 16 + (tid & 15);
+          if (n >= a.N) continue;
+          if (MODE == kDense && a.planes > 1)
+            reinterpret_cast<TO*>(a.C)[((long)blockIdx.y * a.M + m) * a.ldc + n] = from_f<TO>(s[j]);
+          else
+            store_col<TO>(a, m, n, s[j]);
+        }
       }
     }
     __syncthreads();
@@ -443,6 +454,14 @@ template <typename T, typename TO, int MODE>
 int launch_skinny(const GemmArgs& a, int rows, hipStream_t s) {
   const dim3 grid((a.N + 15) / 16, MODE == kDense ? a.planes : a.experts);
   if (grid.y > 65535) return lsh_fail(LSH_ERR_UNSUPPORTED, "float gemm: too many experts");
+  if constexpr (MODE == kDense) {
+    if (a.planes == 1 && rows > 16 && a.N >= 64 * cu_count()) {
+      const dim3 half((a.N + 31) / 32, 1);
+      if (rows <= 32) gemm_skinny_kernel<T, TO, MODE, 2, 2><<<half, 256, 0, s>>>(a);
+      else gemm_skinny_kernel<T, TO, MODE, 4, 2><<<half, 256, 0, s>>>(a);
+      return lsh_check_launch("gemm_skinny_kernel");
+    }
+  }
   if (rows <= 16) gemm_skinny_kernel<T, TO, MODE, 1><<<grid, 256, 0, s>>>(a);
   else if (rows <= 32 || MODE != kDense) gemm_skinny_kernel<T, TO, MODE, 2><<<grid, 256, 0, s>>>(a);
   else gemm_skinny_kernel<T, TO, MODE, 4><<<grid, 256, 0, s>>>(a);

@@ -157,7 +157,7 @@ constexpr int kQT = 128, kKT = 64;
 __device__ __forceinline__ float exp2_f(float x) { return __builtin_amdgcn_exp2f(x); }
 
 template <typename T, int NK, int NV>  // head sizes in 32s
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(256, sizeof(T) == 2 && NK <= 4 && NV <= 4 ? 2 : 1)
 attn_prefill_kernel(const T* __restrict__ q, const T* __restrict__ k_cache,
                     const T* __restrict__ v_cache, const T* __restrict__ proj, long ld, int g_col,
                     T* __restrict__ out, const SeqSpan* __restrict__ seqs, AttnShape sh,
@@ -203,37 +203,57 @@ attn_prefill_kernel(const T* __restrict__ q, const T* __restrict__ k_cache,
   const int t_end = last_pos / kKT;  // last tile
   const int t_win = mask.window > 0 ? max(0, first_pos - mask.window + 1) / kKT : 0;
   const int t_keep = mask.keep_first > 0 ? (min(mask.keep_first, kv_len) - 1) / kKT : -1;
-  for (int t = 0; t <= t_end; ++t) {
-    if (t > t_keep && t < t_win) t = t_win;
-    const int key0 = t * kKT;
-    __syncthreads();
-    // keys: 16-byte chunks, rows beyond the sequence are clamped (their scores are masked)
-    constexpr int CH = DP / V;
-    for (int c = tid; c < kKT * CH; c += 256) {
-      const int r = c / CH, x = c - r * CH;
-      *reinterpret_cast<frag_t*>(&Ks[r * KSTR + x * V]) =
-          *reinterpret_cast<const frag_t*>(kc + (long)min(key0 + r, kv_len - 1) * DP + x * V);
+  // the next tile's keys (16-byte chunks; rows beyond the sequence are clamped, their scores are
+  // masked) and values (4 keys x 4 columns per unit; rows beyond it are zero) wait in registers
+  // while the present one is used
+  typedef T T4 __attribute__((ext_vector_type(4)));
+  constexpr int CH = DP / V, KU = kKT * CH / 256;
+  constexpr int VU = ((kKT / 4) * (VP / 4) + 255) / 256;
+  frag_t kr[KU];
+  T4 vr[VU][4];
+  auto fetch = [&](int key0) {
+#pragma unroll
+    for (int u = 0; u < KU; ++u) {
+      const int c = u * 256 + tid, r = c / CH, x = c - r * CH;
+      kr[u] = *reinterpret_cast<const frag_t*>(kc + (long)min(key0 + r, kv_len - 1) * DP + x * V);
     }
-    // values transposed: a thread takes 4 keys of one 4-column group and stores 4 keys per column
-    for (int c = tid; c < (kKT / 4) * (VP / 4); c += 256) {
-      const int r4 = c / (VP / 4), x = c - r4 * (VP / 4);
-      float v[4][4];
+#pragma unroll
+    for (int u = 0; u < VU; ++u) {
+      const int c = u * 256 + tid, r4 = c / (VP / 4), x = c - r4 * (VP / 4);
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
         const int key = key0 + r4 * 4 + j;
-        if (key < kv_len) {
-          ldv<4, T>(vc + (long)key * VP + x * 4, v[j]);
-        } else {
-#pragma unroll
-          for (int e = 0; e < 4; ++e) v[j][e] = 0.f;
-        }
-      }
-#pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        const float col[4] = {v[0][e], v[1][e], v[2][e], v[3][e]};
-        stv<4, T>(&Vt[(x * 4 + e) * VSTR + r4 * 4], col);
+        vr[u][j] = key < kv_len && r4 < kKT / 4 ? *reinterpret_cast<const T4*>(vc + (long)key * VP + x * 4)
+                                                : (T4)0.f;
       }
     }
+  };
+  auto next_tile = [&](int t) {
+    ++t;
+    return t > t_keep && t < t_win ? t_win : t;
+  };
+  int t = next_tile(-1);
+  fetch(t * kKT);
+  for (; t <= t_end; t = next_tile(t)) {
+    const int key0 = t * kKT;
+    __syncthreads();
+#pragma unroll
+    for (int u = 0; u < KU; ++u) {
+      const int c = u * 256 + tid, r = c / CH, x = c - r * CH;
+      *reinterpret_cast<frag_t*>(&Ks[r * KSTR + x * V]) = kr[u];
+    }
+#pragma unroll
+    for (int u = 0; u < VU; ++u) {
+      const int c = u * 256 + tid, r4 = c / (VP / 4), x = c - r4 * (VP / 4);
+      if (r4 < kKT / 4) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const T4 col = {vr[u][0][e], vr[u][1][e], vr[u][2][e], vr[u][3][e]};
+          *reinterpret_cast<T4*>(&Vt[(x * 4 + e) * VSTR + r4 * 4]) = col;
+        }
+      }
+    }
+    if (next_tile(t) <= t_end) fetch(next_tile(t) * kKT);
     __syncthreads();
     if (!wave_live) continue;
     // does any query of this wavefront see any key of the tile?
@@ -683,7 +703,10 @@ int attn_decode(const T* q, const T* k_cache, const T* v_cache, const T* proj, l
       !workspace || (g_col >= 0 && !proj))
     return lsh_fail(LSH_ERR_INVALID, "attn_decode: bad arguments");
   const int rep = sh.heads / sh.kv_heads;
-  const int R = rep == 1 ? 1 : rep == 2 ? 2 : 4;
+  // heads per workgroup: several share the loads of a key, but only as many as leave the chip filled
+  // (the kernel's time is the arithmetic of the compute units that work)
+  const long each = (long)rows * sh.kv_heads, fill = 2L * cu_count();
+  const int R = rep == 1 || each * rep <= fill ? 1 : rep == 2 || each * ((rep + 1) / 2) <= fill ? 2 : 4;
   const int groups = (rep + R - 1) / R;
   const long most = mask.window > 0 ? std::min((long)max_len, (long)mask.window + mask.keep_first)
                                     : (long)max_len;

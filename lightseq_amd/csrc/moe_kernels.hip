@@ -13,27 +13,22 @@ __device__ __forceinline__ void choose(const float (&z)[EPL], int experts, int t
                                        float& my_w) {
   const int lane = threadIdx.x & 63;
   float my_z = -INFINITY;
-  my_e = 0;
+  my_e = 0x7fffffff;
   unsigned taken = 0;  // this lane's logits already chosen
   for (int j = 0; j < top; ++j) {
     float m = -INFINITY;
-    int me = 0x7fffffff;
 #pragma unroll
     for (int i = 0; i < EPL; ++i)
-      if (!(taken >> i & 1u) && i * 64 + lane < experts && (z[i] > m || me == 0x7fffffff)) {
-        m = z[i];
-        me = i * 64 + lane;
-      }
+      if (!(taken >> i & 1u)) m = fmaxf(m, z[i]);
+    m = wave_max_dpp(m);
+    int me = 0x7fffffff;  // the lowest index among the largest
 #pragma unroll
-    for (int d = 32; d > 0; d >>= 1) {
-      const float om = __shfl_xor(m, d);
-      const int oe = __shfl_xor(me, d);
-      if (om > m || (om == m && oe < me)) {
-        m = om;
-        me = oe;
-      }
+    for (int i = EPL - 1; i >= 0; --i) {
+      const unsigned long long hit =
+          __ballot(!(taken >> i & 1u) && i * 64 + lane < experts && z[i] == m);
+      if (hit) me = i * 64 + __ffsll(hit) - 1;
     }
-    if ((me & 63) == lane) taken |= 1u << (me >> 6);
+    if ((me & 63) == lane) taken |= 1u << ((me >> 6) & 31);
     if (lane == j) {
       my_z = m;
       my_e = me;
@@ -43,32 +38,38 @@ __device__ __forceinline__ void choose(const float (&z)[EPL], int experts, int t
   my_w = ex / wave_sum(ex);
 }
 
-// A workgroup takes 4 * TPW tokens and counts its choices in LDS first, so that an expert's counter
+// A workgroup takes NW * TPW tokens and counts its choices in LDS first, so that an expert's counter
 // sees one addition per workgroup.  EPL logits per lane: experts <= 64 * EPL.
-template <int EPL, int TPW>
-__global__ void __launch_bounds__(256)
+template <int EPL, int TPW, int NW>
+__global__ void __launch_bounds__(64 * NW)
 moe_route_kernel(const float* __restrict__ logits, const float* __restrict__ bias,
                  float* __restrict__ weight, int* __restrict__ count, int* __restrict__ list,
                  int tokens, int experts, int top) {
   __shared__ int cnt[64 * EPL], base[64 * EPL];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  for (int e = threadIdx.x; e < experts; e += 256) cnt[e] = 0;
+  for (int e = threadIdx.x; e < experts; e += 64 * NW) cnt[e] = 0;
   __syncthreads();
+  const int t0 = (blockIdx.x * NW + wave) * TPW;
+  float z[TPW][EPL];
+#pragma unroll
+  for (int u = 0; u < TPW; ++u)
+#pragma unroll
+    for (int i = 0; i < EPL; ++i) {
+      const int e = i * 64 + lane;
+      z[u][i] = e < experts ? logits[(long)min(t0 + u, tokens - 1) * experts + e] +
+                                  (bias ? bias[e] : 0.f)
+                            : -INFINITY;
+    }
   int my_e[TPW], rank[TPW];
 #pragma unroll
   for (int u = 0; u < TPW; ++u) {
-    const int t = (blockIdx.x * 4 + wave) * TPW + u;
+    const int t = t0 + u;
     my_e[u] = -1;
     rank[u] = 0;
     if (t < tokens) {
-      float z[EPL], w;
-#pragma unroll
-      for (int i = 0; i < EPL; ++i) {
-        const int e = i * 64 + lane;
-        z[i] = e < experts ? logits[(long)t * experts + e] + (bias ? bias[e] : 0.f) : -INFINITY;
-      }
+      float w;
       int e;
-      choose<EPL>(z, experts, top, e, w);
+      choose<EPL>(z[u], experts, top, e, w);
       if (lane < top) {
         weight[(long)t * top + lane] = w;
         if (e < experts) {  // always, for finite logits
@@ -79,13 +80,13 @@ moe_route_kernel(const float* __restrict__ logits, const float* __restrict__ bia
     }
   }
   __syncthreads();
-  for (int e = threadIdx.x; e < experts; e += 256)
+  for (int e = threadIdx.x; e < experts; e += 64 * NW)
     if (cnt[e] > 0) base[e] = atomicAdd(&count[e], cnt[e]);
   __syncthreads();
 #pragma unroll
   for (int u = 0; u < TPW; ++u)
     if (my_e[u] >= 0) {
-      const int t = (blockIdx.x * 4 + wave) * TPW + u;
+      const int t = t0 + u;
       list[(long)my_e[u] * tokens + base[my_e[u]] + rank[u]] = t * top + lane;
     }
 }
@@ -157,19 +158,18 @@ int moe_route(const float* logits, const float* bias, float* weight, int* count,
   if (int rc = check(tokens, experts, top)) return rc;
   if (!logits || !weight || !count || !list)
     return lsh_fail(LSH_ERR_INVALID, "moe_route: bad arguments");
-#define ROUTE(EPL, TPW)                                                                  \
-  moe_route_kernel<EPL, TPW><<<(tokens + 4 * TPW - 1) / (4 * TPW), 256, 0, s>>>(         \
+#define ROUTE(EPL, TPW, NW)                                                                      \
+  moe_route_kernel<EPL, TPW, NW><<<(tokens + NW * TPW - 1) / (NW * TPW), 64 * NW, 0, s>>>(       \
       logits, bias, weight, count, list, tokens, experts, top)
   const bool many = tokens >= 512;
   if (experts <= 64) {
-    if (many) ROUTE(1, 8);
-    else ROUTE(1, 1);
+    if (many) ROUTE(1, 8, 16);
+    else ROUTE(1, 1, 4);
   } else if (experts <= 256) {
-    if (many) ROUTE(4, 8);
-    else ROUTE(4, 1);
+    if (many) ROUTE(4, 4, 16);
+    else ROUTE(4, 1, 4);
   } else {
-    if (many) ROUTE(16, 8);
-    else ROUTE(16, 1);
+    ROUTE(16, 1, 4);
   }
 #undef ROUTE
   return lsh_check_launch("moe_route_kernel");

@@ -75,7 +75,7 @@ def rng(seed=0):
 @pytest.mark.parametrize("m,n,k,split", [
     (1, 40, 64, 40), (5, 33, 48, 20), (16, 256, 512, 250), (40, 64, 1024, 64), (64, 100, 72, 64),
     (65, 128, 64, 128), (130, 200, 128, 190), (257, 96, 192, 96), (300, 50, 27, 44), (3, 70, 75, 70),
-    (2048, 2048, 256, 2048), (2100, 2080, 128, 2072),
+    (20, 16400, 72, 16400), (50, 16500, 64, 16487), (2048, 2048, 256, 2048), (2100, 2080, 128, 2072),
 ])
 def test_gemm(dt, m, n, k, split):
     r = rng(m * n + k)
