@@ -24,7 +24,7 @@ namespace {
 // (or the gates) over a tile of tokens and keeps the convolution's window in registers.
 constexpr int kConvTile = 16;
 
-template <typename T, int NT>  // taps <= NT
+template <typename T, int NT>  // at most NT taps
 __global__ void __launch_bounds__(256)
 delta_prepare_kernel(const T* __restrict__ proj, long ld, const float* __restrict__ ba,
                      const float* __restrict__ conv_w, const float* __restrict__ a_log,
@@ -315,7 +315,7 @@ __device__ __forceinline__ frag_t scale4(frag_t a, const float* s) {
   return __builtin_bit_cast(frag_t, x);
 }
 
-template <typename T>
+template <typename T, int NDW>  // dim, vdim <= 64 * NDW
 __global__ void __launch_bounds__(256)
 delta_chunk_prep_kernel(const float* __restrict__ q, const float* __restrict__ k,
                         const T* __restrict__ v, const float* __restrict__ log_g,
@@ -338,10 +338,32 @@ delta_chunk_prep_kernel(const float* __restrict__ q, const float* __restrict__ k
   const long row0 = sq.row0 + c0;
   float* out = ws + ((sq.row0 / kC + blockIdx.z + blockIdx.x) * (long)H + h) * chunk_floats(sh);
   float *oW = out, *oP = oW + kC * D, *oU = oP + kC * kC, *ob = oU + kC * VD;
-  for (int x = tid; x < kC * (D / 4); x += 256) {
-    const int r = x / (D / 4), d = (x - r * (D / 4)) * 4;
-    *reinterpret_cast<frag_t*>(&X[r * KS + d]) =
-        r < n ? *reinterpret_cast<const frag_t*>(k + ((row0 + r) * G + kvh) * D + d) : fz();
+  // everything this chunk reads is requested at once: keys (to LDS), the query fragments of the
+  // wavefront's rows, and the values, which wait in registers for their turn in LDS
+  typedef T T4 __attribute__((ext_vector_type(4)));
+  frag_t kq[4 * NDW], fq[4 * NDW];
+  T4 vq[4 * NDW];
+  const int qi = w * 16 + c;
+  {
+    const float* qr = q + ((row0 + min(qi, n - 1)) * G + kvh) * D;
+#pragma unroll
+    for (int u = 0; u < 4 * NDW; ++u) {
+      const int x = u * 256 + tid, r = x / (D / 4), d = (x - r * (D / 4)) * 4;
+      kq[u] = r < n ? *reinterpret_cast<const frag_t*>(k + ((row0 + r) * G + kvh) * D + d) : fz();
+    }
+#pragma unroll
+    for (int u = 0; u < 4 * NDW; ++u)
+      fq[u] = u < D / 16 && qi < n ? *reinterpret_cast<const frag_t*>(qr + u * 16 + qd * 4) : fz();
+#pragma unroll
+    for (int u = 0; u < 4 * NDW; ++u) {
+      const int x = u * 256 + tid, r = x / (VD / 4), d = (x - r * (VD / 4)) * 4;
+      vq[u] = r < n ? *reinterpret_cast<const T4*>(v + ((row0 + r) * H + h) * VD + d) : (T4)0.f;
+    }
+  }
+#pragma unroll
+  for (int u = 0; u < 4 * NDW; ++u) {
+    const int x = u * 256 + tid, r = x / (D / 4), d = (x - r * (D / 4)) * 4;
+    if (r < kC) *reinterpret_cast<frag_t*>(&X[r * KS + d]) = kq[u];
   }
   if (w == 0) {
     float b = lane < n ? log_g[(row0 + lane) * H + h] : 0.f;
@@ -363,20 +385,19 @@ delta_chunk_prep_kernel(const float* __restrict__ q, const float* __restrict__ k
     f32x4 kk[4], qk[4];
 #pragma unroll
     for (int j = 0; j < 4; ++j) kk[j] = qk[j] = (f32x4)0.f;
-    const int qi = w * 16 + c;
-    const float* qr = q + ((row0 + min(qi, n - 1)) * G + kvh) * D;
-    for (int s = 0; s < D / 16; ++s) {
-      const int d = s * 16 + qd * 4;
-      const frag_t fk = *reinterpret_cast<const frag_t*>(&X[qi * KS + d]);
-      const frag_t fq = qi < n ? *reinterpret_cast<const frag_t*>(qr + d) : fz();
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
-        if (j <= w) {
-          const frag_t fb = *reinterpret_cast<const frag_t*>(&X[(j * 16 + c) * KS + d]);
-          kk[j] = mma16(0.f, fk, fb, kk[j]);
-          qk[j] = mma16(0.f, fq, fb, qk[j]);
-        }
-    }
+    for (int s = 0; s < 4 * NDW; ++s)
+      if (s < D / 16) {
+        const int d = s * 16 + qd * 4;
+        const frag_t fk = *reinterpret_cast<const frag_t*>(&X[qi * KS + d]);
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          if (j <= w) {
+            const frag_t fb = *reinterpret_cast<const frag_t*>(&X[(j * 16 + c) * KS + d]);
+            kk[j] = mma16(0.f, fk, fb, kk[j]);
+            qk[j] = mma16(0.f, fq[s], fb, qk[j]);
+          }
+      }
 #pragma unroll
     for (int j = 0; j < 4; ++j)
 #pragma unroll
@@ -404,38 +425,34 @@ delta_chunk_prep_kernel(const float* __restrict__ q, const float* __restrict__ k
   }
   __syncthreads();
   // below the diagonal, by distance: T_ij = -T_ii sum_{j <= m < i} L_im T_mj
+#pragma unroll
   for (int dist = 1; dist < 4; ++dist) {
     const int r = tid >> 4, cc = tid & 15;
+    // rows are read in fours
+    auto dot = [&](const float* a, const float* t, int len) {
+      float s = 0.f;
+      for (int m = 0; m < len; m += 4) {
+        const f32x4 x = *reinterpret_cast<const f32x4*>(a + m);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) s = fmaf(x[e], t[(m + e) * LS], s);
+      }
+      return s;
+    };
     float acc[3];
 #pragma unroll
-    for (int b = 0; b < 3; ++b) {
-      acc[b] = 0.f;
-      const int bi = b + dist;
-      if (bi < 4)
-        for (int m = b * 16; m < bi * 16; ++m)
-          acc[b] = fmaf(L[(bi * 16 + r) * LS + m], Tm[m * LS + b * 16 + cc], acc[b]);
-    }
+    for (int b = 0; b < 4 - dist; ++b)
+      acc[b] = dot(&L[((b + dist) * 16 + r) * LS + b * 16], &Tm[b * 16 * LS + b * 16 + cc], 16 * dist);
     // the sums wait in the target blocks, which nothing else reads at this distance
+#pragma unroll
+    for (int b = 0; b < 4 - dist; ++b) Tm[((b + dist) * 16 + r) * LS + b * 16 + cc] = acc[b];
     __syncthreads();
 #pragma unroll
-    for (int b = 0; b < 3; ++b)
-      if (b + dist < 4) Tm[((b + dist) * 16 + r) * LS + b * 16 + cc] = acc[b];
-    __syncthreads();
-    float res[3];
-#pragma unroll
-    for (int b = 0; b < 3; ++b) {
-      res[b] = 0.f;
-      const int bi = b + dist;
-      if (bi < 4)
-#pragma unroll
-        for (int m = 0; m < 16; ++m)
-          res[b] = fmaf(-Tm[(bi * 16 + r) * LS + bi * 16 + m],
-                        Tm[(bi * 16 + m) * LS + b * 16 + cc], res[b]);
-    }
+    for (int b = 0; b < 4 - dist; ++b)
+      acc[b] = -dot(&Tm[((b + dist) * 16 + r) * LS + (b + dist) * 16],
+                    &Tm[(b + dist) * 16 * LS + b * 16 + cc], 16);
     __syncthreads();
 #pragma unroll
-    for (int b = 0; b < 3; ++b)
-      if (b + dist < 4) Tm[((b + dist) * 16 + r) * LS + b * 16 + cc] = res[b];
+    for (int b = 0; b < 4 - dist; ++b) Tm[((b + dist) * 16 + r) * LS + b * 16 + cc] = acc[b];
     __syncthreads();
   }
   // T diag(scale) X for the columns of X, rows of wavefront w
@@ -461,9 +478,13 @@ delta_chunk_prep_kernel(const float* __restrict__ q, const float* __restrict__ k
   };
   product(sc, oW, D);
   __syncthreads();
-  for (int x = tid; x < kC * VD; x += 256) {
-    const int r = x / VD, d = x - r * VD;
-    X[r * KS + d] = r < n ? to_f(v[((row0 + r) * H + h) * VD + d]) : 0.f;
+#pragma unroll
+  for (int u = 0; u < 4 * NDW; ++u) {
+    const int x = u * 256 + tid, r = x / (VD / 4), d = (x - r * (VD / 4)) * 4;
+    if (r < kC) {
+      const f32x4 t = {to_f((T)vq[u][0]), to_f((T)vq[u][1]), to_f((T)vq[u][2]), to_f((T)vq[u][3])};
+      *reinterpret_cast<f32x4*>(&X[r * KS + d]) = t;
+    }
   }
   __syncthreads();
   product(bt, oU, VD);
@@ -474,15 +495,16 @@ delta_chunk_prep_kernel(const float* __restrict__ q, const float* __restrict__ k
 // transposed in LDS as an operand; the chunk's operands go from global memory straight into
 // fragments, each element to the one wavefront that needs it.
 template <int NDW, int NVB>  // dim <= 64 * NDW
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(256, NDW == 1 ? 2 : 1)
 delta_chunk_scan_kernel(const float* __restrict__ q, const float* __restrict__ k,
                         const float* __restrict__ ws, float* __restrict__ state,
                         float* __restrict__ o, const SeqSpan* __restrict__ seqs, int vblocks,
                         DeltaShape sh) {
   constexpr int MAXD = 64 * NDW, SS = MAXD + 4, US = kC + 4, NS = 4 * NDW;
-  constexpr bool PREFETCH = NDW <= 2;  // two chunks' operands fit the registers
-  __shared__ __attribute__((aligned(16))) float St[NVB * 16][SS], Ut[NVB * 16][US],
-      Ud[NVB * 16][US];
+  extern __shared__ __attribute__((aligned(16))) float sm[];
+  float(*St)[SS] = reinterpret_cast<float(*)[SS]>(sm);
+  float(*Ut)[US] = reinterpret_cast<float(*)[US]>(sm + NVB * 16 * SS);
+  float(*Ud)[US] = Ut + NVB * 16;
   const int H = sh.heads, D = sh.dim, VD = sh.vdim, G = sh.kv_heads;
   // the value blocks of a head read the same operands: H * sequences apart in the grid
   const int hs = gridDim.x / vblocks;
@@ -509,29 +531,40 @@ delta_chunk_scan_kernel(const float* __restrict__ q, const float* __restrict__ k
   const int chunks = (sq.n + kC - 1) / kC;
   const long cf = chunk_floats(sh);
   const float* base = ws + ((sq.row0 / kC + si) * (long)H + h) * cf;
-  struct Ops {
-    frag_t fw[NS], fq[NS], fp[4];
-    f32x4 fk[NDW][4];
-    f32x4 u0[NVB];
-    f32x4 b4;      // cumulative log decay of the rows 4 qd ..
-    float b_last;
-  };
-  auto fetch = [&](int ch, Ops& a) {
-    const float* p = base + (long)ch * H * cf;
-    const float *pW = p, *pP = pW + kC * D, *pU = pP + kC * kC, *pb = pU + kC * VD;
-    const int n = min(kC, sq.n - ch * kC);
-    const long row0 = sq.row0 + (long)ch * kC;
-    const int i = w * 16 + c;
-    const float* qr = q + ((row0 + min(i, n - 1)) * G + kvh) * D;
+  // The chunk's operands: those of its first half (products with S) and of its second (products with
+  // U).  Both are requested at its start; holding a chunk's set ahead costs more in register moves
+  // than it hides.
+  frag_t fw[NS], fq[NS], fp[4];
+  f32x4 fk[NDW][4], u0[NVB], b4;  // b4: cumulative log decay of the rows 4 qd ..
+  float b_last;
+  auto fetch1 = [&](int ch) {
+    const float* pW = base + (long)ch * H * cf;
+    const float *pU = pW + kC * (D + kC), *pb = pU + kC * VD;
+    const int n = min(kC, sq.n - ch * kC), i = w * 16 + c;
+    const float* qr = q + ((sq.row0 + (long)ch * kC + min(i, n - 1)) * G + kvh) * D;
 #pragma unroll
     for (int s = 0; s < NS; ++s)
       if (s < ns) {
-        a.fw[s] = *reinterpret_cast<const frag_t*>(pW + (long)i * D + s * 16 + qd * 4);
-        a.fq[s] = *reinterpret_cast<const frag_t*>(qr + s * 16 + qd * 4);
+        fw[s] = *reinterpret_cast<const frag_t*>(pW + (long)i * D + s * 16 + qd * 4);
+        fq[s] = *reinterpret_cast<const frag_t*>(qr + s * 16 + qd * 4);
       }
 #pragma unroll
+    for (int b = 0; b < NVB; ++b)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int vc = v0 + b * 16 + c;
+        u0[b][r] = vc < VD ? pU[(long)(w * 16 + 4 * qd + r) * VD + vc] : 0.f;
+      }
+    b4 = *reinterpret_cast<const f32x4*>(pb + w * 16 + 4 * qd);
+    b_last = pb[kC - 1];
+  };
+  auto fetch2 = [&](int ch) {
+    const float* pP = base + (long)ch * H * cf + kC * D;
+    const int n = min(kC, sq.n - ch * kC);
+    const long row0 = sq.row0 + (long)ch * kC;
+#pragma unroll
     for (int s = 0; s < 4; ++s)
-      a.fp[s] = *reinterpret_cast<const frag_t*>(pP + i * kC + s * 16 + qd * 4);
+      fp[s] = *reinterpret_cast<const frag_t*>(pP + (w * 16 + c) * kC + s * 16 + qd * 4);
 #pragma unroll
     for (int x = 0; x < NDW; ++x) {
       const int db = w + 4 * x;
@@ -540,21 +573,14 @@ delta_chunk_scan_kernel(const float* __restrict__ q, const float* __restrict__ k
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
           const int t = s * 16 + qd * 4 + j;
-          a.fk[x][s][j] = db < ns && t < n ? k[((row0 + t) * G + kvh) * D + db * 16 + c] : 0.f;
+          fk[x][s][j] = db < ns && t < n ? k[((row0 + t) * G + kvh) * D + db * 16 + c] : 0.f;
         }
     }
-#pragma unroll
-    for (int b = 0; b < NVB; ++b)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int vc = v0 + b * 16 + c;
-        a.u0[b][r] = vc < VD ? pU[(long)(w * 16 + 4 * qd + r) * VD + vc] : 0.f;
-      }
-    a.b4 = *reinterpret_cast<const f32x4*>(pb + w * 16 + 4 * qd);
-    a.b_last = pb[kC - 1];
   };
-  auto chunk = [&](int ch, const Ops& cur, Ops& nxt) {
-    if (PREFETCH && ch + 1 < chunks) fetch(ch + 1, nxt);
+  __syncthreads();
+  for (int ch = 0; ch < chunks; ++ch) {
+    fetch1(ch);
+    fetch2(ch);
     const int n = min(kC, sq.n - ch * kC);
     f32x4 ws_acc[NVB], o_acc[NVB];
 #pragma unroll
@@ -565,38 +591,33 @@ delta_chunk_scan_kernel(const float* __restrict__ q, const float* __restrict__ k
 #pragma unroll
         for (int b = 0; b < NVB; ++b) {
           const frag_t fs = *reinterpret_cast<const frag_t*>(&St[b * 16 + c][s * 16 + qd * 4]);
-          ws_acc[b] = mma16(0.f, cur.fw[s], fs, ws_acc[b]);
-          o_acc[b] = mma16(0.f, cur.fq[s], fs, o_acc[b]);
+          ws_acc[b] = mma16(0.f, fw[s], fs, ws_acc[b]);
+          o_acc[b] = mma16(0.f, fq[s], fs, o_acc[b]);
         }
       }
+    f32x4 e_row, e_left;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      e_row[r] = expf(b4[r]);
+      e_left[r] = expf(b_last - b4[r]);
+    }
+    const float decay = expf(b_last);
 #pragma unroll
     for (int b = 0; b < NVB; ++b) {
-      f32x4 u, ud;
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        u[r] = cur.u0[b][r] - ws_acc[b][r];
-        ud[r] = u[r] * expf(cur.b_last - cur.b4[r]);
-        o_acc[b][r] *= expf(cur.b4[r]);
-      }
+      const f32x4 u = u0[b] - ws_acc[b];
+      o_acc[b] *= e_row;
       *reinterpret_cast<f32x4*>(&Ut[b * 16 + c][w * 16 + 4 * qd]) = u;
-      *reinterpret_cast<f32x4*>(&Ud[b * 16 + c][w * 16 + 4 * qd]) = ud;
+      *reinterpret_cast<f32x4*>(&Ud[b * 16 + c][w * 16 + 4 * qd]) = u * e_left;
     }
     __syncthreads();
-    const float decay = expf(cur.b_last);
 #pragma unroll
     for (int b = 0; b < NVB; ++b) {
 #pragma unroll
       for (int s = 0; s < 4; ++s)
         if (s <= w)
-          o_acc[b] = mma16(0.f, cur.fp[s],
+          o_acc[b] = mma16(0.f, fp[s],
                            *reinterpret_cast<const frag_t*>(&Ut[b * 16 + c][s * 16 + qd * 4]),
                            o_acc[b]);
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int t = w * 16 + 4 * qd + r, vc = v0 + b * 16 + c;
-        if (t < n && vc < VD)
-          o[((sq.row0 + (long)ch * kC + t) * H + h) * VD + vc] = o_acc[b][r];
-      }
 #pragma unroll
       for (int x = 0; x < NDW; ++x) {
         const int db = w + 4 * x;
@@ -604,29 +625,22 @@ delta_chunk_scan_kernel(const float* __restrict__ q, const float* __restrict__ k
           S[x][b] *= decay;
 #pragma unroll
           for (int s = 0; s < 4; ++s)
-            S[x][b] = mma16(0.f, __builtin_bit_cast(frag_t, cur.fk[x][s]),
+            S[x][b] = mma16(0.f, __builtin_bit_cast(frag_t, fk[x][s]),
                             *reinterpret_cast<const frag_t*>(&Ud[b * 16 + c][s * 16 + qd * 4]),
                             S[x][b]);
           *reinterpret_cast<f32x4*>(&St[b * 16 + c][db * 16 + 4 * qd]) = S[x][b];
         }
       }
     }
+#pragma unroll
+    for (int b = 0; b < NVB; ++b)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int t = w * 16 + 4 * qd + r, vc = v0 + b * 16 + c;
+        if (t < n && vc < VD)
+          o[((sq.row0 + (long)ch * kC + t) * H + h) * VD + vc] = o_acc[b][r];
+      }
     __syncthreads();
-  };
-  Ops ops[PREFETCH ? 2 : 1];
-  if constexpr (PREFETCH) {
-    fetch(0, ops[0]);
-    __syncthreads();
-    for (int ch = 0; ch < chunks; ch += 2) {
-      chunk(ch, ops[0], ops[1]);
-      if (ch + 1 < chunks) chunk(ch + 1, ops[1], ops[0]);
-    }
-  } else {
-    __syncthreads();
-    for (int ch = 0; ch < chunks; ++ch) {
-      fetch(ch, ops[0]);
-      chunk(ch, ops[0], ops[0]);
-    }
   }
 #pragma unroll
   for (int i = 0; i < NDW; ++i)
@@ -824,8 +838,8 @@ int check_shape(const DeltaShape& sh) {
   if (sh.heads <= 0 || sh.kv_heads <= 0 || sh.heads % sh.kv_heads != 0 || sh.dim <= 0 ||
       sh.vdim <= 0 || sh.taps <= 0)
     return lsh_fail(LSH_ERR_INVALID, "delta: bad shape");
-  if (sh.dim > 256 || sh.vdim > 256 || sh.taps > 8)
-    return lsh_fail(LSH_ERR_UNSUPPORTED, "delta: head sizes up to 256, at most 8 taps");
+  if (sh.dim > 256 || sh.vdim > 256 || sh.taps > 16)
+    return lsh_fail(LSH_ERR_UNSUPPORTED, "delta: head sizes up to 256, at most 16 taps");
   return LSH_OK;
 }
 
@@ -842,7 +856,7 @@ int delta_prepare(const T* proj, long ld, const float* ba, const float* conv_w, 
     return lsh_fail(LSH_ERR_INVALID, "delta_prepare: bad arguments");
   const int tiles = (max_n + kConvTile - 1) / kConvTile, units = 2 * sh.kv_heads + sh.heads;
   const dim3 grid(tiles, (units + 1 + 3) / 4, n_seqs);
-  if (sh.dim % 4 == 0 && sh.vdim % 4 == 0 && ld % 4 == 0) {
+  if (sh.dim % 4 == 0 && sh.vdim % 4 == 0 && ld % 4 == 0 && sh.taps <= 8) {
     const int wide = std::max(sh.dim, sh.vdim);
 #define PREP4(NT, LPH)                                                                             \
   delta_prepare4_kernel<T, NT, LPH><<<dim3(tiles, (units * LPH + 255) / 256 + 1, n_seqs), 256, 0,  \
@@ -858,12 +872,13 @@ int delta_prepare(const T* proj, long ld, const float* ba, const float* conv_w, 
     else PREP4_T(64);
 #undef PREP4_T
 #undef PREP4
-  } else if (sh.taps <= 4)
+  } else if (sh.taps <= 4) {
     delta_prepare_kernel<T, 4><<<grid, 256, 0, s>>>(proj, ld, ba, conv_w, a_log, dt_bias, conv_ring,
                                                     q, k, v, log_g, beta, seqs, sh);
-  else
-    delta_prepare_kernel<T, 8><<<grid, 256, 0, s>>>(proj, ld, ba, conv_w, a_log, dt_bias, conv_ring,
+  } else {
+    delta_prepare_kernel<T, 16><<<grid, 256, 0, s>>>(proj, ld, ba, conv_w, a_log, dt_bias, conv_ring,
                                                     q, k, v, log_g, beta, seqs, sh);
+  }
   if (int rc = lsh_check_launch("delta_prepare_kernel")) return rc;
   delta_ring_kernel<T><<<dim3((sh.channels() + 255) / 256, n_seqs), 256, 0, s>>>(proj, ld, conv_ring,
                                                                                 seqs, sh);
@@ -901,7 +916,10 @@ int delta_chunked(const float* q, const float* k, const T* v, const float* log_g
     return lsh_fail(LSH_ERR_INVALID, "delta_chunked: bad arguments");
   if (!delta_chunked_supported(sh))
     return lsh_fail(LSH_ERR_UNSUPPORTED, "delta_chunked: head sizes must be multiples of 16");
-  auto prep = delta_chunk_prep_kernel<T>;
+  const int widest = std::max(sh.dim, sh.vdim);
+  auto prep = widest <= 64    ? delta_chunk_prep_kernel<T, 1>
+              : widest <= 128 ? delta_chunk_prep_kernel<T, 2>
+                              : delta_chunk_prep_kernel<T, 4>;
   const size_t smem = sizeof(float) * ((size_t)kC * (std::max(sh.dim, sh.vdim) + 4) +
                                        2 * (size_t)kC * (kC + 4) + 3 * kC);
   if (int rc = lsh_check_hip(hipFuncSetAttribute(reinterpret_cast<const void*>(prep),
@@ -912,20 +930,33 @@ int delta_chunked(const float* q, const float* k, const T* v, const float* log_g
   prep<<<dim3((max_n + kC - 1) / kC, sh.heads, n_seqs), 256, smem, s>>>(q, k, v, log_g, beta,
                                                                         workspace, seqs, sh);
   if (int rc = lsh_check_launch("delta_chunk_prep_kernel")) return rc;
-  const bool wide = (long)sh.heads * n_seqs * (sh.vdim / 16) >= 2L * cu_count();
-  const int nvb = wide ? 2 : 1;
+  // value columns per workgroup: as many as leave every compute unit one (they share the operands)
+  int nvb = sh.dim > 128 ? 2 : 4;
+  while (nvb > 1 && (long)sh.heads * n_seqs * ((sh.vdim + 16 * nvb - 1) / (16 * nvb)) < cu_count())
+    nvb /= 2;
   const int vblocks = (sh.vdim + 16 * nvb - 1) / (16 * nvb);
   const unsigned grid = (unsigned)vblocks * sh.heads * n_seqs;
-#define SCAN(NDW, NVB)                                                                          \
-  delta_chunk_scan_kernel<NDW, NVB><<<grid, 256, 0, s>>>(q, k, workspace, state, o, seqs, vblocks, sh)
-#define SCAN_V(NDW)            \
-  do {                         \
-    if (wide) SCAN(NDW, 2);    \
-    else SCAN(NDW, 1);         \
+#define SCAN(NDW, NVB)                                                                            \
+  do {                                                                                            \
+    auto scan = delta_chunk_scan_kernel<NDW, NVB>;                                                \
+    const int lds = (int)sizeof(float) * NVB * 16 * (64 * NDW + 4 + 2 * (kC + 4));                \
+    if (int rc = lsh_check_hip(hipFuncSetAttribute(reinterpret_cast<const void*>(scan),           \
+                                                   hipFuncAttributeMaxDynamicSharedMemorySize,    \
+                                                   lds),                                          \
+                               "hipFuncSetAttribute(delta_chunk_scan)"))                          \
+      return rc;                                                                                  \
+    scan<<<grid, 256, lds, s>>>(q, k, workspace, state, o, seqs, vblocks, sh);                    \
+  } while (0)
+#define SCAN_V(NDW)              \
+  do {                           \
+    if (nvb == 4) SCAN(NDW, 4);  \
+    else if (nvb == 2) SCAN(NDW, 2); \
+    else SCAN(NDW, 1);           \
   } while (0)
   if (sh.dim <= 64) SCAN_V(1);
   else if (sh.dim <= 128) SCAN_V(2);
-  else SCAN_V(4);
+  else if (nvb == 2) SCAN(4, 2);
+  else SCAN(4, 1);
 #undef SCAN_V
 #undef SCAN
   return lsh_check_launch("delta_chunk_scan_kernel");

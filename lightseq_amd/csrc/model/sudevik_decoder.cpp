@@ -153,7 +153,8 @@ class Stack : public SudevikStack {
     for (const SudevikLayerConfig& l : _c.layers) {
       if (l.dim > 256 || l.vdim > 256)
         throw std::runtime_error("config: head sizes above 256 are not supported");
-      if (l.taps > 8) throw std::runtime_error("config: convolutions of more than 8 taps are not supported");
+      if (l.taps > 16)
+        throw std::runtime_error("config: convolutions of more than 16 taps are not supported");
       if (l.experts > 1024 || l.top > 64)
         throw std::runtime_error("config: at most 64 choices of at most 1024 experts are supported");
     }

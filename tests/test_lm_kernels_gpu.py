@@ -464,7 +464,7 @@ class Delta:
 DELTA = [
     # H, G, D, VD, taps
     (4, 2, 32, 48, 4), (6, 2, 21, 19, 2), (2, 1, 144, 160, 1), (1, 1, 12, 70, 5), (3, 3, 128, 128, 8), (2, 2, 256, 256, 3),
-    (2, 1, 64, 30, 4), (2, 1, 80, 16, 3),
+    (2, 1, 64, 30, 4), (2, 1, 80, 16, 3), (2, 1, 32, 32, 11),
 ]
 
 
