@@ -58,6 +58,13 @@ class Json {
       throw std::runtime_error("json: an integer was expected");
     return (long)number_;
   }
+  // the member `key`, a size or a count
+  int positive(const char* key) const {
+    const long v = at(key).integer();
+    if (v <= 0 || v > (1L << 30))
+      throw std::runtime_error(std::string("config: '") + key + "' must be a positive integer");
+    return (int)v;
+  }
   const std::string& string() const {
     need(kString, "a string");
     return string_;

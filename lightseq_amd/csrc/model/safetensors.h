@@ -57,18 +57,22 @@ class SafeTensors {
   }
 
   bool has(const std::string& name) const { return tensors_.count(name) != 0; }
-  // the tensor, with the shape it must have
-  const Tensor& get(const std::string& name, const std::vector<long>& shape) const {
+  const Tensor& get(const std::string& name) const {
     auto it = tensors_.find(name);
     if (it == tensors_.end()) throw std::runtime_error("tensor '" + name + "' is missing");
-    if (it->second.shape != shape) {
+    return it->second;
+  }
+  // the tensor, with the shape it must have
+  const Tensor& get(const std::string& name, const std::vector<long>& shape) const {
+    const Tensor& t = get(name);
+    if (t.shape != shape) {
       std::string m = "tensor '" + name + "' has the shape [";
-      for (long d : it->second.shape) m += std::to_string(d) + " ";
+      for (long d : t.shape) m += std::to_string(d) + " ";
       m += "], expected [";
       for (long d : shape) m += std::to_string(d) + " ";
       throw std::runtime_error(m + "]");
     }
-    return it->second;
+    return t;
   }
 
  private:

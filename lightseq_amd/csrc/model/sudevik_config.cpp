@@ -25,38 +25,27 @@ std::vector<double> RotaryConfig::frequencies(double* magnitude) const {
   return f;
 }
 
-namespace {
-
-int positive(const Json& o, const char* key) {
-  const long v = o.at(key).integer();
-  if (v <= 0 || v > (1L << 30))
-    throw std::runtime_error(std::string("config: '") + key + "' must be a positive integer");
-  return (int)v;
-}
-
-}  // namespace
-
 SudevikConfig SudevikConfig::parse(const Json& c) {
   SudevikConfig out;
-  out.vocab = positive(c, "vocab");
-  out.width = positive(c, "width");
+  out.vocab = c.positive("vocab");
+  out.width = c.positive("width");
   out.eps = c.at("norm").at("eps").number();
   for (const Json& e : c.at("layers").items()) {
     SudevikLayerConfig l;
     const int index = (int)out.layers.size();
     const std::string type = e.at("type").string();
     const Json& m = e.at("mixer");
-    l.heads = positive(m, "heads");
-    l.kv_heads = positive(m, "kv_heads");
-    l.dim = positive(m, "dim");
-    l.vdim = positive(m, "vdim");
+    l.heads = m.positive("heads");
+    l.kv_heads = m.positive("kv_heads");
+    l.dim = m.positive("dim");
+    l.vdim = m.positive("vdim");
     if (l.heads % l.kv_heads) throw std::runtime_error("config: heads must be a multiple of kv_heads");
     if (type == "attention") {
       l.attention = true;
       l.scale = m.at("scale").number();
       const Json& rot = m["rot"];
       if (!rot.is_null()) {
-        l.rot.dims = positive(rot, "dims");
+        l.rot.dims = rot.positive("dims");
         l.rot.base = rot.at("base").number();
         if (l.rot.dims % 2 || l.rot.dims > l.dim)
           throw std::runtime_error("config: rot.dims must be even and at most dim");
@@ -71,7 +60,7 @@ SudevikConfig SudevikConfig::parse(const Json& c) {
       }
       const Json& mask = m["mask"];
       if (!mask.is_null()) {
-        l.window = positive(mask, "size");
+        l.window = mask.positive("size");
         if (!mask["keep_first"].is_null()) l.keep_first = (int)mask["keep_first"].integer();
       }
       if (!m["kv_from"].is_null()) {
@@ -84,7 +73,7 @@ SudevikConfig SudevikConfig::parse(const Json& c) {
           throw std::runtime_error("config: kv_from names a layer of other head sizes");
       }
     } else if (type == "delta") {
-      l.taps = positive(m, "conv");
+      l.taps = m.positive("conv");
     } else {
       throw std::runtime_error("config: unknown layer type '" + type + "'");
     }
@@ -92,9 +81,9 @@ SudevikConfig SudevikConfig::parse(const Json& c) {
     if (!f.is_null()) {
       if (f.at("kind").string() != "moe")
         throw std::runtime_error("config: unknown mlp kind '" + f.at("kind").string() + "'");
-      l.ff = positive(f.at("expert"), "ff");
-      l.experts = positive(f.at("router"), "experts");
-      l.top = positive(f.at("router"), "top");
+      l.ff = f.at("expert").positive("ff");
+      l.experts = f.at("router").positive("experts");
+      l.top = f.at("router").positive("top");
       if (l.top > l.experts) throw std::runtime_error("config: more choices than experts");
     }
     out.layers.push_back(l);

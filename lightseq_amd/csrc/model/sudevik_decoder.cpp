@@ -3,6 +3,9 @@
 #include <algorithm>
 #include <cmath>
 
+#include "sequence_cache.h"
+#include "sudevik_weight.h"
+
 namespace lightseq {
 namespace hip {
 
@@ -15,7 +18,7 @@ constexpr int kMaxPlanes = 8;
 constexpr int kScanRows = 8;  // spans this short run the recurrence token by token
 
 template <typename T>
-class Stack : public SudevikStack {
+class Stack : public DecoderStack {
  public:
   Stack(const SudevikConfig& c, const SafeTensors& file, int slots, int max_step, hipStream_t s)
       : _c(c), _max_step(max_step), _slots(slots), _stream(s) {
@@ -287,7 +290,7 @@ class Stack : public SudevikStack {
     return add;
   }
 
-  const SudevikConfig& _c;
+  const SudevikConfig _c;
   const int _max_step, _slots;
   hipStream_t _stream;
   SudevikWeight<T> _w;
@@ -303,7 +306,7 @@ class Stack : public SudevikStack {
 
 }  // namespace
 
-std::unique_ptr<SudevikStack> SudevikStack::create(const SudevikConfig& config,
+std::unique_ptr<DecoderStack> create_sudevik_stack(const SudevikConfig& config,
                                                    const SafeTensors& file, bool float32, int slots,
                                                    int max_step, hipStream_t stream) {
   if (float32) return std::make_unique<Stack<float>>(config, file, slots, max_step, stream);
