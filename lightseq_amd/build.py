@@ -23,9 +23,11 @@ DECODER_LIB_PATH = os.path.join(LIB_DIR, "liblightseq_decoder.so")
 # sources of liblightseq_decoder.so
 DECODER_SOURCES = [
     "core.hip", "gemm_float.hip", "lm_norm_kernels.hip", "lm_attn_kernels.hip", "delta_kernels.hip",
-    "moe_kernels.hip", "lm_sample_kernels.hip", "lm_capi.hip", "model/model_capi.cpp",
-    "model/model_dir.cpp", "model/sudevik.cpp", "model/sudevik_config.cpp",
-    "model/sudevik_decoder.cpp", "model/sudevik_weight.cpp",
+    "gla_kernels.hip", "moe_kernels.hip", "lm_sample_kernels.hip", "lm_capi.hip",
+    "model/model_capi.cpp", "model/model_dir.cpp", "model/decoder_lm.cpp", "model/sudevik.cpp",
+    "model/sudevik_config.cpp", "model/sudevik_decoder.cpp", "model/sudevik_weight.cpp",
+    "model/gebuzen.cpp", "model/gebuzen_config.cpp", "model/gebuzen_decoder.cpp",
+    "model/gebuzen_weight.cpp",
 ]
 
 ARCH = "gfx950"

@@ -20,7 +20,9 @@ namespace lsh {
 
 namespace {
 
-enum GemmMode { kDense = 0, kMoeUp = 1, kMoeDown = 2 };
+enum GemmMode { kDense = 0, kMoeUp = 1, kMoeDown = 2, kGated = 3 };
+constexpr bool is_dense(int mode) { return mode == kDense || mode == kGated; }  // all rows, in order
+constexpr bool is_up(int mode) { return mode == kMoeUp || mode == kGated; }     // gate and up rows
 
 struct GemmArgs {
   const void *A, *W;
@@ -28,10 +30,12 @@ struct GemmArgs {
   float* C2;
   long lda, ldc, ld2;
   int n_split;
-  int M, N, K;  // kMoeUp: N = ff, weights [experts][2][N][K]; kMoeDown: [experts][N][K]
+  int M, N, K;  // kGated: weights [2][N][K]; kMoeUp: N = ff, weights [experts][2][N][K]; kMoeDown: [experts][N][K]
   const int *count, *list;
   int list_stride, experts, top;
   int planes, k_per_plane;  // gemm_skinny_kernel, kDense
+  GemmEpilogue epi;         // kDense
+  int act;                  // kMoeUp, kGated
 };
 
 // rows of one tile: where they are read and written
@@ -39,16 +43,27 @@ struct RowSet {
   int expert, first, last;  // rows [first, last) of the expert's list, or of the matrix
 };
 
+__device__ __forceinline__ float gated(const GemmArgs& a, float gate, float up) {
+  return (a.act == kGateRelu ? fmaxf(gate, 0.f) : silu_f(gate)) * up;
+}
+// the result of column n from its sum
+template <int MODE>
+__device__ __forceinline__ float finish(const GemmArgs& a, int n, float sum) {
+  if (MODE != kDense) return sum;
+  const float v = sum * a.epi.scale;
+  return a.epi.bias ? v + a.epi.bias[n] : v;
+}
+
 template <int MODE>
 __device__ __forceinline__ long src_row(const GemmArgs& a, const RowSet& rs, int r) {
   r = min(r, rs.last - 1);
-  if (MODE == kDense) return r;
+  if (is_dense(MODE)) return r;
   const int id = a.list[(long)rs.expert * a.list_stride + r];
   return MODE == kMoeUp ? id / a.top : id;
 }
 template <int MODE>
 __device__ __forceinline__ long dst_row(const GemmArgs& a, const RowSet& rs, int r) {
-  return MODE == kDense ? r : a.list[(long)rs.expert * a.list_stride + r];
+  return is_dense(MODE) ? r : a.list[(long)rs.expert * a.list_stride + r];
 }
 
 // the t-th tile of `tm` rows, the experts' rows one after the other (all lanes call it)
@@ -97,22 +112,22 @@ __device__ __forceinline__ void dense_tile(int t, int nblk, int tiles_m, int til
   tm = grp * 8 + (in_grp - tn * gm);
 }
 
-// 4 wavefronts in 2 x 2, each MB x NB blocks of 32 x 32.  kMoeUp needs NB == 2: block column 0 is
+// 4 wavefronts in 2 x 2, each MB x NB blocks of 32 x 32.  kMoeUp and kGated need NB == 2: block column 0 is
 // the gate, 1 the up projection of the same 32 outputs, so a lane holds both.
 template <typename T, typename TO, int MODE, int MB, int NB>
 __global__ void __launch_bounds__(256)
 gemm_tile_kernel(GemmArgs a, int tiles_m, int tiles_n) {
   constexpr int TM = 64 * MB, TN = 64 * NB;
-  constexpr int OUT_N = MODE == kMoeUp ? TN / 2 : TN;  // output columns of a tile
+  constexpr int OUT_N = is_up(MODE) ? TN / 2 : TN;  // output columns of a tile
   constexpr int STAGE = (TM + TN) * kBK;
   constexpr int NA = TM / 32, NW = TN / 32, PER = NA + NW;
-  static_assert(MODE != kMoeUp || NB == 2, "gate and up blocks");
+  static_assert(!is_up(MODE) || NB == 2, "gate and up blocks");
   __shared__ __attribute__((aligned(128))) int8_t smem[2 * STAGE];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int wm = wave >> 1, wn = wave & 1, l32 = lane & 31, g = lane >> 5;
   RowSet rs;
   int tn;
-  if (MODE == kDense) {
+  if (is_dense(MODE)) {
     int tm;
     dense_tile(blockIdx.x, gridDim.x, tiles_m, tiles_n, tm, tn);
     rs = RowSet{0, tm * TM, min(a.M, tm * TM + TM)};
@@ -126,7 +141,7 @@ gemm_tile_kernel(GemmArgs a, int tiles_m, int tiles_n) {
   const int nk = Kb / kBK;
   const char* A = reinterpret_cast<const char*>(a.A);
   const char* W = reinterpret_cast<const char*>(a.W);
-  if (MODE != kDense) W += (long)rs.expert * (MODE == kMoeUp ? 2 : 1) * a.N * Kb;
+  if (!is_dense(MODE)) W += (long)rs.expert * (is_up(MODE) ? 2 : 1) * a.N * Kb;
 
   uint32_t a_src[NA], w_src[NW];
 #pragma unroll
@@ -140,7 +155,7 @@ gemm_tile_kernel(GemmArgs a, int tiles_m, int tiles_n) {
     const int row = (wave + 4 * i) * 8 + (lane >> 3);
     const int c = (lane & 7) ^ key_wgt(row);
     int n;
-    if (MODE == kMoeUp) {
+    if (is_up(MODE)) {
       const int blk = row >> 5;  // wn * 2 + (gate | up)
       n = min(n0 + (blk >> 1) * 32 + (row & 31), a.N - 1) + (blk & 1) * a.N;
     } else {
@@ -165,7 +180,7 @@ gemm_tile_kernel(GemmArgs a, int tiles_m, int tiles_n) {
   };
   // float output: activations are the first operand, a store then covers whole lines; otherwise the
   // weights are, and a lane's 16 accumulators are 16 adjacent columns of one row
-  constexpr bool ROWS_IN_REGS = sizeof(TO) == 4 && MODE != kMoeUp;
+  constexpr bool ROWS_IN_REGS = sizeof(TO) == 4 && !is_up(MODE);
   int a_base[MB], w_base[NB];
 #pragma unroll
   for (int i = 0; i < MB; ++i) {
@@ -223,7 +238,7 @@ gemm_tile_kernel(GemmArgs a, int tiles_m, int tiles_n) {
 #pragma unroll
         for (int j = 0; j < NB; ++j) {
           const int n = n0 + wn * (NB * 32) + j * 32 + sigma(l32);
-          if (n < a.N) store_col<TO>(a, m, n, acc[i][j][k]);
+          if (n < a.N) store_col<TO>(a, m, n, finish<MODE>(a, n, acc[i][j][k]));
         }
       }
   } else {
@@ -233,13 +248,13 @@ gemm_tile_kernel(GemmArgs a, int tiles_m, int tiles_n) {
       if (r >= rs.last) continue;
       const long m = dst_row<MODE>(a, rs, r);
 #pragma unroll
-      for (int j = 0; j < (MODE == kMoeUp ? 1 : NB); ++j) {
-        const int n = n0 + (MODE == kMoeUp ? wn * 32 : wn * (NB * 32) + j * 32) + 16 * g;
+      for (int j = 0; j < (is_up(MODE) ? 1 : NB); ++j) {
+        const int n = n0 + (is_up(MODE) ? wn * 32 : wn * (NB * 32) + j * 32) + 16 * g;
         float v[16];
 #pragma unroll
         for (int k = 0; k < 16; ++k) {
-          if constexpr (MODE == kMoeUp) v[k] = silu_f(acc[i][0][k]) * acc[i][1][k];
-          else v[k] = acc[i][j][k];
+          if constexpr (is_up(MODE)) v[k] = gated(a, acc[i][0][k], acc[i][1][k]);
+          else v[k] = finish<MODE>(a, min(n + k, a.N - 1), acc[i][j][k]);
         }
         if (n + 16 <= min(a.N, a.n_split) && a.ldc % 8 == 0) {
           TO* p = reinterpret_cast<TO*>(a.C) + m * a.ldc + n;
@@ -269,7 +284,7 @@ template <typename T, typename TO, int MODE, int MB, int NS = 1>
 __global__ void __launch_bounds__(256)
 gemm_skinny_kernel(GemmArgs a) {
   static_assert(NS == 1 || MODE == kDense, "strips of one matrix");
-  constexpr int NB = MODE == kMoeUp ? 2 : NS;
+  constexpr int NB = is_up(MODE) ? 2 : NS;
   constexpr int V = FT<T>::kVec;
   constexpr int U = 4;  // 64-byte slices per turn: 256 bytes of every row
   __shared__ float red[4][NB][MB][16][17];
@@ -278,7 +293,7 @@ gemm_skinny_kernel(GemmArgs a) {
   const int n0 = blockIdx.x * 16 * NS;
   RowSet rs{0, 0, a.M};
   int k_lo = 0, k_hi = a.K;
-  if (MODE != kDense) {
+  if (!is_dense(MODE)) {
     rs.expert = blockIdx.y;
     rs.last = a.count[rs.expert];
     if (rs.last == 0) return;
@@ -287,11 +302,11 @@ gemm_skinny_kernel(GemmArgs a) {
     k_hi = min(a.K, k_lo + a.k_per_plane);
   }
   const T* W = reinterpret_cast<const T*>(a.W);
-  if (MODE != kDense) W += (long)rs.expert * NB * a.N * a.K;
+  if (!is_dense(MODE)) W += (long)rs.expert * NB * a.N * a.K;
   const T* wrow[NB];
 #pragma unroll
   for (int j = 0; j < NB; ++j)
-    wrow[j] = W + (MODE == kMoeUp ? (long)(min(n0 + c, a.N - 1) + j * a.N)
+    wrow[j] = W + (is_up(MODE) ? (long)(min(n0 + c, a.N - 1) + j * a.N)
                                   : (long)min(n0 + j * 16 + c, a.N - 1)) * a.K;
   const T* A = reinterpret_cast<const T*>(a.A);
   const int first_end = rs.last;
@@ -343,9 +358,9 @@ gemm_skinny_kernel(GemmArgs a) {
         s[j] = (red[0][j][i][r][tid & 15] + red[1][j][i][r][tid & 15]) +
                (red[2][j][i][r][tid & 15] + red[3][j][i][r][tid & 15]);
       const long m = dst_row<MODE>(a, rs, row);
-      if constexpr (MODE == kMoeUp) {
+      if constexpr (is_up(MODE)) {
         const int n = n0 + (tid & 15);
-        if (n < a.N) reinterpret_cast<TO*>(a.C)[m * a.ldc + n] = from_f<TO>(silu_f(s[0]) * s[NB - 1]);
+        if (n < a.N) reinterpret_cast<TO*>(a.C)[m * a.ldc + n] = from_f<TO>(gated(a, s[0], s[NB - 1]));
       } else {
 #pragma unroll
         for (int j = 0; j < NB; ++j) {
@@ -354,7 +369,7 @@ gemm_skinny_kernel(GemmArgs a) {
           if (MODE == kDense && a.planes > 1)
             reinterpret_cast<TO*>(a.C)[((long)blockIdx.y * a.M + m) * a.ldc + n] = from_f<TO>(s[j]);
           else
-            store_col<TO>(a, m, n, s[j]);
+            store_col<TO>(a, m, n, finish<MODE>(a, n, s[j]));
         }
       }
     }
@@ -367,7 +382,7 @@ gemm_skinny_kernel(GemmArgs a) {
 template <typename T, typename TO, int MODE>
 __global__ void __launch_bounds__(256)
 gemm_generic_kernel(GemmArgs a, int tiles_n) {
-  constexpr int NB = MODE == kMoeUp ? 2 : 1;
+  constexpr int NB = is_up(MODE) ? 2 : 1;
   constexpr int KS = 64 / sizeof(T);       // elements per K step
   constexpr int STR = 80 / sizeof(T);      // LDS row stride
   __shared__ __attribute__((aligned(16))) T As[64][STR], Ws[NB][64][STR];
@@ -375,12 +390,12 @@ gemm_generic_kernel(GemmArgs a, int tiles_n) {
   const int wm = wave >> 1, wn = wave & 1, c = lane & 15, q = lane >> 4;
   RowSet rs;
   const int tn = blockIdx.x % tiles_n, t = blockIdx.x / tiles_n;
-  if (MODE == kDense) rs = RowSet{0, t * 64, min(a.M, t * 64 + 64)};
+  if (is_dense(MODE)) rs = RowSet{0, t * 64, min(a.M, t * 64 + 64)};
   else if (!expert_tile(a, t, 64, rs)) return;
   const int n0 = tn * 64;
   const T* A = reinterpret_cast<const T*>(a.A);
   const T* W = reinterpret_cast<const T*>(a.W);
-  if (MODE != kDense) W += (long)rs.expert * NB * a.N * a.K;
+  if (!is_dense(MODE)) W += (long)rs.expert * NB * a.N * a.K;
   f32x4 acc[NB][2][2];
 #pragma unroll
   for (int j = 0; j < NB; ++j)
@@ -426,11 +441,11 @@ gemm_generic_kernel(GemmArgs a, int tiles_n) {
       for (int y = 0; y < 2; ++y) {
         const int n = n0 + wn * 32 + y * 16 + c;
         if (n >= a.N) continue;
-        if constexpr (MODE == kMoeUp)
+        if constexpr (is_up(MODE))
           reinterpret_cast<TO*>(a.C)[m * a.ldc + n] =
-              from_f<TO>(silu_f(acc[0][x][y][v]) * acc[NB - 1][x][y][v]);
+              from_f<TO>(gated(a, acc[0][x][y][v], acc[NB - 1][x][y][v]));
         else
-          store_col<TO>(a, m, n, acc[0][x][y][v]);
+          store_col<TO>(a, m, n, finish<MODE>(a, n, acc[0][x][y][v]));
       }
     }
 }
@@ -443,7 +458,7 @@ bool rows_aligned(const GemmArgs& a) {  // every row of A and W starts at 16 byt
 }
 template <typename T>
 bool tile_ok(const GemmArgs& a, int mode) {
-  const long wrows = (long)(mode == kMoeUp ? 2 : 1) * a.N;
+  const long wrows = (long)(is_up(mode) ? 2 : 1) * a.N;
   const long arows = mode == kMoeDown ? (long)a.M * a.top : a.M;
   return rows_aligned<T>(a) && (long)a.K * sizeof(T) % kBK == 0 &&
          wrows * a.K * (long)sizeof(T) < (1L << 32) && arows * a.lda * (long)sizeof(T) < (1L << 32) &&
@@ -452,7 +467,7 @@ bool tile_ok(const GemmArgs& a, int mode) {
 
 template <typename T, typename TO, int MODE>
 int launch_skinny(const GemmArgs& a, int rows, hipStream_t s) {
-  const dim3 grid((a.N + 15) / 16, MODE == kDense ? a.planes : a.experts);
+  const dim3 grid((a.N + 15) / 16, is_dense(MODE) ? a.planes : a.experts);
   if (grid.y > 65535) return lsh_fail(LSH_ERR_UNSUPPORTED, "float gemm: too many experts");
   if constexpr (MODE == kDense) {
     if (a.planes == 1 && rows > 16 && a.N >= 64 * cu_count()) {
@@ -463,7 +478,7 @@ int launch_skinny(const GemmArgs& a, int rows, hipStream_t s) {
     }
   }
   if (rows <= 16) gemm_skinny_kernel<T, TO, MODE, 1><<<grid, 256, 0, s>>>(a);
-  else if (rows <= 32 || MODE != kDense) gemm_skinny_kernel<T, TO, MODE, 2><<<grid, 256, 0, s>>>(a);
+  else if (rows <= 32 || !is_dense(MODE)) gemm_skinny_kernel<T, TO, MODE, 2><<<grid, 256, 0, s>>>(a);
   else gemm_skinny_kernel<T, TO, MODE, 4><<<grid, 256, 0, s>>>(a);
   return lsh_check_launch("gemm_skinny_kernel");
 }
@@ -472,24 +487,24 @@ template <typename T, typename TO, int MODE>
 int launch_any(const GemmArgs& a, hipStream_t s) {
   if (!a.A || !a.W || !a.C || a.M <= 0 || a.N <= 0 || a.K <= 0)
     return lsh_fail(LSH_ERR_INVALID, "float gemm: bad arguments");
-  const long rows = MODE == kDense ? a.M : (long)a.M * a.top;
+  const long rows = is_dense(MODE) ? a.M : (long)a.M * a.top;
   // few rows per product: the weights are what is read
-  if (rows_aligned<T>(a) && (MODE == kDense ? rows <= 64 : rows <= 24L * a.experts))
-    return launch_skinny<T, TO, MODE>(a, MODE == kDense ? a.M : (int)rows / a.experts + 1, s);
+  if (rows_aligned<T>(a) && (is_dense(MODE) ? rows <= 64 : rows <= 24L * a.experts))
+    return launch_skinny<T, TO, MODE>(a, is_dense(MODE) ? a.M : (int)rows / a.experts + 1, s);
   const auto tiles_m = [&](int tm) {  // upper bound: every expert may end in a part of a tile
-    return MODE == kDense ? (rows + tm - 1) / tm : rows / tm + std::min((long)a.experts, rows);
+    return is_dense(MODE) ? (rows + tm - 1) / tm : rows / tm + std::min((long)a.experts, rows);
   };
   if (tile_ok<T>(a, MODE)) {
-    constexpr int kBigN = MODE == kMoeUp ? 64 : 128;
+    constexpr int kBigN = is_up(MODE) ? 64 : 128;
     const long big = tiles_m(128) * ((a.N + kBigN - 1) / kBigN);
-    const bool small = MODE == kDense ? big < cu_count() : rows < 64L * a.experts;
+    const bool small = is_dense(MODE) ? big < cu_count() : rows < 64L * a.experts;
     const int tm = small ? 64 : 128;
-    const int tnn = MODE == kMoeUp ? 64 : small ? 64 : 128;
+    const int tnn = is_up(MODE) ? 64 : small ? 64 : 128;
     const long gm = tiles_m(tm), gn = (a.N + tnn - 1) / tnn;
     if (gm * gn > 0x7fffffffL) return lsh_fail(LSH_ERR_UNSUPPORTED, "float gemm: too large");
     const unsigned grid = (unsigned)(gm * gn);
     if (small)
-      gemm_tile_kernel<T, TO, MODE, 1, MODE == kMoeUp ? 2 : 1>
+      gemm_tile_kernel<T, TO, MODE, 1, is_up(MODE) ? 2 : 1>
           <<<grid, 256, 0, s>>>(a, (int)gm, (int)gn);
     else
       gemm_tile_kernel<T, TO, MODE, 2, 2><<<grid, 256, 0, s>>>(a, (int)gm, (int)gn);
@@ -505,14 +520,29 @@ int launch_any(const GemmArgs& a, hipStream_t s) {
 
 template <typename T, typename TO>
 int gemm_float(const T* A, long lda, const T* W, TO* C, long ldc, float* C2, long ld2, int n_split,
-               int M, int N, int K, hipStream_t s) {
+               int M, int N, int K, hipStream_t s, const GemmEpilogue& epilogue) {
   if (n_split < N && !C2) return lsh_fail(LSH_ERR_INVALID, "float gemm: no second output");
   GemmArgs a{};
   a.A = A; a.W = W; a.C = C; a.C2 = C2;
   a.lda = lda; a.ldc = ldc; a.ld2 = ld2; a.n_split = n_split;
   a.M = M; a.N = N; a.K = K;
   a.planes = 1; a.k_per_plane = K;
+  a.epi = epilogue;
   return launch_any<T, TO, kDense>(a, s);
+}
+
+template <typename T>
+int gemm_gated(const T* A, long lda, const T* W, T* C, long ldc, int M, int N, int K, int act,
+               hipStream_t s) {
+  if (act != kGateSilu && act != kGateRelu)
+    return lsh_fail(LSH_ERR_INVALID, "gemm_gated: unknown activation");
+  GemmArgs a{};
+  a.A = A; a.W = W; a.C = C;
+  a.lda = lda; a.ldc = ldc; a.n_split = N;
+  a.M = M; a.N = N; a.K = K;
+  a.planes = 1; a.k_per_plane = K;
+  a.act = act;
+  return launch_any<T, T, kGated>(a, s);
 }
 
 int gemm_float_preferred_planes(int M, int N, int K) {
@@ -566,13 +596,15 @@ int moe_down(const T* act, const T* w, TO* out, const int* count, const int* lis
 
 #define INST_TT(T, TO)                                                                           \
   template int gemm_float<T, TO>(const T*, long, const T*, TO*, long, float*, long, int, int,    \
-                                 int, int, hipStream_t);                                         \
+                                 int, int, hipStream_t, const GemmEpilogue&);                    \
   template int moe_down<T, TO>(const T*, const T*, TO*, const int*, const int*, int, int, int,   \
                                int, int, hipStream_t);
 INST_TT(float, float)
 INST_TT(bf16_t, bf16_t)
 INST_TT(bf16_t, float)
 #define INST_T(T)                                                                               \
+  template int gemm_gated<T>(const T*, long, const T*, T*, long, int, int, int, int,            \
+                             hipStream_t);                                                      \
   template int gemm_float_planes<T>(const T*, long, const T*, float*, int, int, int, int, int*, \
                                     hipStream_t);                                               \
   template int moe_up<T>(const T*, const T*, T*, const int*, const int*, int, int, int, int, int, \

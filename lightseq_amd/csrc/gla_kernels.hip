@@ -1,0 +1,558 @@
+// Gated linear attention:  S <- diag(a) S + k v^T;  o = S^T q  per head, with one decay per key channel,
+// a = sigmoid(A2 low + bias)^(1 / tau).  State, decays and every product of the recurrence are
+// float32; q, k, v and the output gate are read from the projection as they lie there.
+//
+//  * gla_scan_kernel   -- token by token, any size: decays, recurrence, read-out, head norm and output
+//    gate in one launch, the state in registers.  One token per sequence is its shortest case.
+//  * gla_chunk_*       -- a prompt in chunks of 64 tokens, sub-blocks of 16.  With b the running sum of
+//    log a inside a chunk and S the state before it,
+//      o_t = S^T (q_t e^(b_t)) + sum_{j <= t} [sum_d q_td k_jd e^(b_td - b_jd)] v_j,
+//      S  <- e^(b_64) S + sum_j (k_j e^(b_64 - b_j)) v_j^T.
+//    What a chunk adds to the state does not depend on the state, so one launch forms it for all
+//    chunks at once, a second adds the chunks up (element by element) and leaves the state before each,
+//    a third computes the outputs of all chunks at once.  Between sub-blocks the exponent is split at
+//    the end of the keys' block, inside one the decays are multiplied up token by token: no exponent
+//    is ever positive.
+//
+// Lane layout of the chunk kernels: wavefront w has the tokens 16 w .. 16 w + 15 of its chunk; lane
+// (c = lane % 16, qd = lane / 16) holds token c's channels 16 s + 4 qd .. + 3 for every s.  That is an
+// operand of the float32 matrix product and, for the decays, the result of one; moving along the
+// tokens is a shift within 16 lanes.
+#include <algorithm>
+
+#include "lm_launch.h"
+
+namespace lsh {
+
+namespace {
+
+constexpr int kC = 64;
+
+__device__ __forceinline__ float log_decay(float z, float inv_tau) { return -softplus_f(-z) * inv_tau; }
+
+// a lane's value from N lanes before (after) it in its row of 16, zero at the border
+template <int N>
+__device__ __forceinline__ float lanes_before(float x) {
+  if constexpr (N == 0) return x;
+  else return dpp_f<0x110 + N>(x);
+}
+template <int N>
+__device__ __forceinline__ float lanes_after(float x) {
+  return dpp_f<0x100 + N>(x);
+}
+
+template <typename T>
+__device__ __forceinline__ f32x4 load4(const T* p) {
+  float t[4];
+  ldv<4, T>(p, t);
+  return f32x4{t[0], t[1], t[2], t[3]};
+}
+__device__ __forceinline__ frag_t as_frag(f32x4 x) { return __builtin_bit_cast(frag_t, x); }
+__device__ __forceinline__ frag_t ldfrag(const float* p) { return *reinterpret_cast<const frag_t*>(p); }
+__device__ __forceinline__ f32x4 exp4(f32x4 x) {
+  return f32x4{expf(x[0]), expf(x[1]), expf(x[2]), expf(x[3])};
+}
+
+// ------------------------------------------------------------------------------------------------
+// One workgroup per (sequence, head).  LPD lanes share a row of the state (one value channel, V == 4:
+// four adjacent key channels per lane, else every LPD-th), a thread has at most RM rows.
+template <typename T, int V, int LPD, int RM, int NTH>
+__global__ void __launch_bounds__(NTH)
+gla_scan_kernel(const T* __restrict__ proj, long ld, const float* __restrict__ low, GlaWeights wt,
+                float* __restrict__ state, T* __restrict__ out, const SeqSpan* __restrict__ seqs,
+                const int* __restrict__ row_slot, const int* __restrict__ row_pos, GlaShape sh) {
+  constexpr int NVG = NTH / LPD;
+  __shared__ float as[256], qs[256], ks[256], vs[256], os[256], red[16];
+  const int D = sh.dim, VD = sh.vdim, H = sh.heads, h = blockIdx.y;
+  const int tid = threadIdx.x, l = tid % LPD, vg = tid / LPD;
+  SeqSpan sq;
+  if (seqs) sq = seqs[blockIdx.x];
+  else sq = SeqSpan{(int)blockIdx.x, 1, row_pos[blockIdx.x], row_slot[blockIdx.x]};
+  const auto channel = [&](int e) { return V == 4 ? 4 * l + e : l + LPD * e; };
+  float* sp = state + ((long)sq.slot * H + h) * VD * D;
+  float S[RM][4];
+#pragma unroll
+  for (int i = 0; i < RM; ++i) {
+    const int v = vg + NVG * i;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) S[i][e] = 0.f;
+    if (sq.pos0 > 0 && v < VD) {
+      if (V == 4) {
+        if (4 * l < D) ldv<4, float>(sp + (long)v * D + 4 * l, S[i]);
+      } else {
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          if (channel(e) < D) S[i][e] = sp[(long)v * D + channel(e)];
+      }
+    }
+  }
+  const float qscale = 1.0f / sqrtf((float)D);
+  for (int t = 0; t < sq.n; ++t) {
+    const long row = sq.row0 + t;
+    const T* pr = proj + row * ld;
+    const float gate = tid < VD ? to_f(pr[sh.g_col + h * VD + tid]) : 0.f;
+    for (int x = tid; x < 3 * D + VD; x += NTH) {
+      if (x < D) {
+        const float *a2 = wt.a2 + (long)(h * D + x) * sh.rank, *lr = low + row * sh.rank;
+        float z = wt.bias[h * D + x];
+        for (int r = 0; r < sh.rank; r += 4) {
+          const f32x4 a = load4(a2 + r), b = load4(lr + r);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) z = fmaf(a[e], b[e], z);
+        }
+        as[x] = expf(log_decay(z, sh.inv_tau));
+      } else if (x < 2 * D) {
+        qs[x - D] = to_f(pr[sh.q_col + h * D + x - D]) * qscale;
+      } else if (x < 3 * D) {
+        ks[x - 2 * D] = to_f(pr[sh.k_col + h * D + x - 2 * D]);
+      } else {
+        vs[x - 3 * D] = to_f(pr[sh.v_col + h * VD + x - 3 * D]);
+      }
+    }
+    __syncthreads();
+    float a[4], q[4], k[4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int d = channel(e);
+      const bool in = d < D;
+      a[e] = in ? as[d] : 0.f;
+      q[e] = in ? qs[d] : 0.f;
+      k[e] = in ? ks[d] : 0.f;
+    }
+#pragma unroll
+    for (int i = 0; i < RM; ++i) {
+      const int v = vg + NVG * i;
+      const float vv = v < VD ? vs[v] : 0.f;
+      float o = 0.f;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        S[i][e] = fmaf(k[e], vv, a[e] * S[i][e]);
+        o = fmaf(q[e], S[i][e], o);
+      }
+      o += dpp_f<kDppXor1>(o);
+      o += dpp_f<kDppXor2>(o);
+      o += dpp_f<kDppHalfMirror>(o);
+      o += dpp_f<kDppMirror>(o);
+      if (LPD > 16) o += __shfl_xor(o, 16);
+      if (LPD > 32) o += __shfl_xor(o, 32);
+      if (l == 0 && v < VD) os[v] = o;
+    }
+    __syncthreads();
+    const float o = tid < VD ? os[tid] : 0.f;
+    const float ss = block_sum_dpp(o * o, red);
+    if (tid < VD) {
+      const float r = 1.0f / sqrtf(ss / (float)VD + sh.eps);
+      out[(row * H + h) * VD + tid] = from_f<T>(o * r * wt.norm[tid] * silu_f(gate));
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < RM; ++i) {
+    const int v = vg + NVG * i;
+    if (v >= VD) continue;
+    if (V == 4) {
+      if (4 * l < D) stv<4, float>(sp + (long)v * D + 4 * l, S[i]);
+    } else {
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        if (channel(e) < D) sp[(long)v * D + channel(e)] = S[i][e];
+    }
+  }
+}
+
+// ------------------------------------------------------------------------------------------------
+// Workspace of one (chunk, head): what the chunk adds to the state, then the state before it, [VD][D];
+// the chunk's decay [D].  Chunk c of a sequence is number row0 / 64 + sequence index + c.
+__host__ __device__ inline long chunk_floats(const GlaShape& sh) {
+  return (long)sh.vdim * sh.dim + sh.dim;
+}
+
+// log decays of this lane's token and channels; 0 for a token that is not there
+template <int NS>
+__device__ __forceinline__ void chunk_log_decays(const float* __restrict__ low, long row, bool in,
+                                                 const GlaWeights& wt, const GlaShape& sh, int h,
+                                                 int c, int qd, f32x4 (&la)[NS]) {
+  const int ns = sh.dim / 16;
+#pragma unroll
+  for (int s = 0; s < NS; ++s) la[s] = (f32x4)0.f;
+  for (int r = 0; r < sh.rank; r += 16) {
+    const frag_t fl = ldfrag(low + row * sh.rank + r + qd * 4);
+#pragma unroll
+    for (int s = 0; s < NS; ++s)
+      if (s < ns)
+        la[s] = mma16(0.f, ldfrag(wt.a2 + (long)(h * sh.dim + s * 16 + c) * sh.rank + r + qd * 4), fl,
+                      la[s]);
+  }
+#pragma unroll
+  for (int s = 0; s < NS; ++s)
+    if (s < ns) {
+      const f32x4 b = load4(wt.bias + h * sh.dim + s * 16 + qd * 4);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) la[s][e] = in ? log_decay(la[s][e] + b[e], sh.inv_tau) : 0.f;
+    }
+}
+// sums over the tokens of the sub-block up to this one / after this one
+__device__ __forceinline__ f32x4 sum_upto(f32x4 x) {
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    x[e] += lanes_before<1>(x[e]);
+    x[e] += lanes_before<2>(x[e]);
+    x[e] += lanes_before<4>(x[e]);
+    x[e] += lanes_before<8>(x[e]);
+  }
+  return x;
+}
+__device__ __forceinline__ f32x4 sum_after(f32x4 x) {
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    x[e] = lanes_after<1>(x[e]);
+    x[e] += lanes_after<1>(x[e]);
+    x[e] += lanes_after<2>(x[e]);
+    x[e] += lanes_after<4>(x[e]);
+    x[e] += lanes_after<8>(x[e]);
+  }
+  return x;
+}
+
+// the chunk's values, transposed: Vt[v][token], zeros for tokens that are not there
+constexpr int kTS = kC + 4;
+template <typename T>
+__device__ __forceinline__ void stage_values(const T* __restrict__ proj, long ld, long row0, int n,
+                                             const GlaShape& sh, int h, float* Vt) {
+  const int t = threadIdx.x >> 2;
+  const T* src = proj + (row0 + min(t, n - 1)) * ld + sh.v_col + h * sh.vdim;
+  for (int v = (threadIdx.x & 3) * 4; v < sh.vdim; v += 16) {
+    const f32x4 x = t < n ? load4(src + v) : (f32x4)0.f;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) Vt[(v + e) * kTS + t] = x[e];
+  }
+}
+
+// what a chunk adds to the state, and its decay
+template <typename T, int NS>  // dim <= 16 * NS
+__global__ void __launch_bounds__(256)
+gla_chunk_add_kernel(const T* __restrict__ proj, long ld, const float* __restrict__ low, GlaWeights wt,
+                     float* __restrict__ ws, const SeqSpan* __restrict__ seqs, GlaShape sh) {
+  extern __shared__ __attribute__((aligned(16))) float sm[];
+  const SeqSpan sq = seqs[blockIdx.z];
+  const int c0 = blockIdx.x * kC;
+  if (c0 >= sq.n) return;
+  const int n = min(kC, sq.n - c0), h = blockIdx.y, H = sh.heads, D = sh.dim, VD = sh.vdim;
+  const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, c = lane & 15, qd = lane >> 4;
+  const int ns = D / 16, nv = VD / 16;
+  float* Kt = sm;                 // [D][kTS]
+  float* Vt = Kt + D * kTS;       // [VD][kTS]
+  float* tot = Vt + VD * kTS;     // [4][D]: log decay of every sub-block
+  const long row0 = sq.row0 + c0;
+  const int t = w * 16 + c;
+  const bool in = t < n;
+  const long row = row0 + min(t, n - 1);
+  f32x4 k[NS], la[NS];
+#pragma unroll
+  for (int s = 0; s < NS; ++s)
+    k[s] = s < ns && in ? load4(proj + row * ld + sh.k_col + h * D + s * 16 + qd * 4) : (f32x4)0.f;
+  stage_values(proj, ld, row0, n, sh, h, Vt);
+  chunk_log_decays<NS>(low, row, in, wt, sh, h, c, qd, la);
+#pragma unroll
+  for (int s = 0; s < NS; ++s)
+    if (s < ns) {
+      const f32x4 after = sum_after(la[s]);
+      if (c == 0) *reinterpret_cast<f32x4*>(&tot[w * D + s * 16 + qd * 4]) = after + la[s];
+      la[s] = after;
+    }
+  __syncthreads();
+#pragma unroll
+  for (int s = 0; s < NS; ++s)
+    if (s < ns) {
+      f32x4 left = la[s];
+      for (int m = w + 1; m < 4; ++m) left += *reinterpret_cast<const f32x4*>(&tot[m * D + s * 16 + qd * 4]);
+      const f32x4 x = k[s] * exp4(left);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) Kt[(s * 16 + qd * 4 + e) * kTS + t] = x[e];
+    }
+  float* o = ws + ((sq.row0 / kC + (long)blockIdx.z + blockIdx.x) * H + h) * chunk_floats(sh);
+  for (int d = tid; d < D; d += 256)
+    o[(long)VD * D + d] = expf((tot[d] + tot[D + d]) + (tot[2 * D + d] + tot[3 * D + d]));
+  __syncthreads();
+  for (int x = w; x < ns * nv; x += 4) {
+    const int db = x % ns, vb = x / ns;
+    f32x4 acc = (f32x4)0.f;
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      acc = mma16(0.f, ldfrag(&Kt[(db * 16 + c) * kTS + j * 16 + qd * 4]),
+                  ldfrag(&Vt[(vb * 16 + c) * kTS + j * 16 + qd * 4]), acc);
+    *reinterpret_cast<f32x4*>(&o[(long)(vb * 16 + c) * D + db * 16 + qd * 4]) = acc;
+  }
+}
+
+// adds the chunks of a sequence up; every chunk's place receives the state before it
+__global__ void __launch_bounds__(256)
+gla_chunk_state_kernel(float* __restrict__ ws, float* __restrict__ state,
+                       const SeqSpan* __restrict__ seqs, GlaShape sh) {
+  constexpr int U = 8;  // chunks requested at once
+  const SeqSpan sq = seqs[blockIdx.z];
+  const int h = blockIdx.y, H = sh.heads, D = sh.dim;
+  const int x = (blockIdx.x * 256 + threadIdx.x) * 4, size = sh.vdim * D;
+  if (x >= size) return;
+  const long stride = H * chunk_floats(sh);
+  float* base = ws + ((sq.row0 / kC + (long)blockIdx.z) * H + h) * chunk_floats(sh);
+  float* sp = state + ((long)sq.slot * H + h) * size + x;
+  const int chunks = (sq.n + kC - 1) / kC;
+  f32x4 S = (f32x4)0.f;
+  if (sq.pos0 > 0) S = load4(sp);
+  for (int ch = 0; ch < chunks; ch += U) {
+    f32x4 add[U], dec[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u)
+      if (ch + u < chunks) {
+        add[u] = load4(base + (ch + u) * stride + x);
+        dec[u] = load4(base + (ch + u) * stride + size + x % D);
+      }
+#pragma unroll
+    for (int u = 0; u < U; ++u)
+      if (ch + u < chunks) {
+        *reinterpret_cast<f32x4*>(base + (ch + u) * stride + x) = S;
+        S = dec[u] * S + add[u];
+      }
+  }
+  *reinterpret_cast<f32x4*>(sp) = S;
+}
+
+// products inside a sub-block: p[t][t - DELTA] for rising DELTA; w carries q_t times the decays of the
+// DELTA tokens up to t
+template <int NS, int DELTA>
+__device__ __forceinline__ void diagonal(const f32x4 (&k)[NS], const f32x4 (&a)[NS], f32x4 (&w)[NS],
+                                         int ns, int c, int qd, f32x4& p) {
+  if constexpr (DELTA < 16) {
+    float x = 0.f;
+#pragma unroll
+    for (int s = 0; s < NS; ++s)
+      if (s < ns) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          x = fmaf(w[s][e], lanes_before<DELTA>(k[s][e]), x);
+          w[s][e] *= lanes_before<DELTA>(a[s][e]);
+        }
+      }
+    x += __shfl_xor(x, 16);
+    x += __shfl_xor(x, 32);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) p[e] = c - DELTA == 4 * qd + e ? x : p[e];
+    diagonal<NS, DELTA + 1>(k, a, w, ns, c, qd, p);
+  }
+}
+
+// outputs of a chunk, normed and gated
+template <typename T, int NS>  // dim, vdim <= 16 * NS
+__global__ void __launch_bounds__(256)
+gla_chunk_out_kernel(const T* __restrict__ proj, long ld, const float* __restrict__ low, GlaWeights wt,
+                     const float* __restrict__ ws, T* __restrict__ out,
+                     const SeqSpan* __restrict__ seqs, GlaShape sh) {
+  extern __shared__ __attribute__((aligned(16))) float sm[];
+  const SeqSpan sq = seqs[blockIdx.z];
+  const int c0 = blockIdx.x * kC;
+  if (c0 >= sq.n) return;
+  const int n = min(kC, sq.n - c0), h = blockIdx.y, H = sh.heads, D = sh.dim, VD = sh.vdim;
+  const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, c = lane & 15, qd = lane >> 4;
+  const int ns = D / 16, nv = VD / 16, KS = D + 4;
+  float* Kh = sm;                // [48][KS]: keys decayed to the end of their sub-block
+  float* Et = Kh + 48 * KS;      // [4][D]: decay of every sub-block
+  float* Vt = Et + 4 * D;        // [VD][kTS]
+  const long row0 = sq.row0 + c0;
+  const int t = w * 16 + c;
+  const bool in = t < n;
+  const long row = row0 + min(t, n - 1);
+  const T* pr = proj + row * ld;
+  f32x4 q[NS], p = (f32x4)0.f;
+  {
+    f32x4 k[NS], la[NS], wq[NS];
+    const float qscale = 1.0f / sqrtf((float)D);
+#pragma unroll
+    for (int s = 0; s < NS; ++s) {
+      k[s] = s < ns && in ? load4(pr + sh.k_col + h * D + s * 16 + qd * 4) : (f32x4)0.f;
+      q[s] = s < ns && in ? load4(pr + sh.q_col + h * D + s * 16 + qd * 4) * qscale : (f32x4)0.f;
+      wq[s] = q[s];
+    }
+    stage_values(proj, ld, row0, n, sh, h, Vt);
+    chunk_log_decays<NS>(low, row, in, wt, sh, h, c, qd, la);
+#pragma unroll
+    for (int s = 0; s < NS; ++s)
+      if (s < ns) {
+        const f32x4 upto = exp4(sum_upto(la[s]));
+        if (c == 15) *reinterpret_cast<f32x4*>(&Et[w * D + s * 16 + qd * 4]) = upto;
+        if (w < 3)
+          *reinterpret_cast<f32x4*>(&Kh[t * KS + s * 16 + qd * 4]) = k[s] * exp4(sum_after(la[s]));
+        q[s] *= upto;
+        la[s] = exp4(la[s]);
+      }
+    diagonal<NS, 0>(k, la, wq, ns, c, qd, p);
+  }
+  __syncthreads();
+  // transposed outputs: acc[vb] has the value channels 16 vb + 4 qd .. + 3 of token c
+  f32x4 acc[NS];
+#pragma unroll
+  for (int vb = 0; vb < NS; ++vb) {
+    acc[vb] = (f32x4)0.f;
+    if (vb < nv) acc[vb] = mma16(0.f, ldfrag(&Vt[(vb * 16 + c) * kTS + w * 16 + qd * 4]), as_frag(p), acc[vb]);
+  }
+  // earlier sub-blocks; q is decayed further back with every one passed
+  for (int J = w - 1; J >= 0; --J) {
+    f32x4 pj = (f32x4)0.f;
+#pragma unroll
+    for (int s = 0; s < NS; ++s)
+      if (s < ns) pj = mma16(0.f, ldfrag(&Kh[(J * 16 + c) * KS + s * 16 + qd * 4]), as_frag(q[s]), pj);
+#pragma unroll
+    for (int vb = 0; vb < NS; ++vb)
+      if (vb < nv)
+        acc[vb] = mma16(0.f, ldfrag(&Vt[(vb * 16 + c) * kTS + J * 16 + qd * 4]), as_frag(pj), acc[vb]);
+#pragma unroll
+    for (int s = 0; s < NS; ++s)
+      if (s < ns) q[s] *= *reinterpret_cast<const f32x4*>(&Et[J * D + s * 16 + qd * 4]);
+  }
+  if (c0 > 0 || sq.pos0 > 0) {
+    const float* S = ws + ((sq.row0 / kC + (long)blockIdx.z + blockIdx.x) * H + h) * chunk_floats(sh);
+#pragma unroll
+    for (int vb = 0; vb < NS; ++vb)
+      if (vb < nv) {
+#pragma unroll
+        for (int s = 0; s < NS; ++s)
+          if (s < ns)
+            acc[vb] = mma16(0.f, ldfrag(S + (long)(vb * 16 + c) * D + s * 16 + qd * 4), as_frag(q[s]),
+                            acc[vb]);
+      }
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int vb = 0; vb < NS; ++vb)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) ss += acc[vb][e] * acc[vb][e];
+  ss += __shfl_xor(ss, 16);
+  ss += __shfl_xor(ss, 32);
+  if (!in) return;
+  const float r = 1.0f / sqrtf(ss / (float)VD + sh.eps);
+#pragma unroll
+  for (int vb = 0; vb < NS; ++vb)
+    if (vb < nv) {
+      const int v = vb * 16 + qd * 4;
+      const f32x4 g = load4(pr + sh.g_col + h * VD + v), nw = load4(wt.norm + v);
+      float o[4];
+#pragma unroll
+      for (int e = 0; e < 4; ++e) o[e] = acc[vb][e] * r * nw[e] * silu_f(g[e]);
+      stv<4, T>(out + (row * H + h) * VD + v, o);
+    }
+}
+
+int check_shape(const GlaShape& sh) {
+  if (sh.heads <= 0 || sh.heads > 65535 || sh.dim <= 0 || sh.vdim <= 0 || sh.rank <= 0 ||
+      sh.rank % 16 != 0 || sh.q_col < 0 || sh.k_col < 0 || sh.v_col < 0 || sh.g_col < 0)
+    return lsh_fail(LSH_ERR_INVALID, "gated linear attention: bad shape");
+  if (sh.dim > 256 || sh.vdim > 256)
+    return lsh_fail(LSH_ERR_UNSUPPORTED, "gated linear attention: head sizes above 256");
+  return LSH_OK;
+}
+
+template <typename T>
+int launch_scan(const T* proj, long ld, const float* low, const GlaWeights& w, float* state, T* out,
+                const SeqSpan* seqs, const int* row_slot, const int* row_pos, int n,
+                const GlaShape& sh, hipStream_t s) {
+  const dim3 grid(n, sh.heads);
+#define SCAN(V, LPD, RM, NTH)                                                                        \
+  gla_scan_kernel<T, V, LPD, RM, NTH><<<grid, NTH, 0, s>>>(proj, ld, low, w, state, out, seqs,       \
+                                                           row_slot, row_pos, sh)
+#define SCAN_V(V)                                       \
+  do {                                                  \
+    if (sh.dim <= 64) {                                 \
+      if (sh.vdim <= 64) SCAN(V, 16, 4, 256);           \
+      else SCAN(V, 16, 16, 256);                        \
+    } else if (sh.dim <= 128) {                         \
+      if (sh.vdim <= 128) SCAN(V, 32, 16, 256);         \
+      else SCAN(V, 32, 8, 1024);                        \
+    } else {                                            \
+      SCAN(V, 64, 16, 1024);                            \
+    }                                                   \
+  } while (0)
+  if (sh.dim % 4 == 0) SCAN_V(4);
+  else SCAN_V(1);
+#undef SCAN_V
+#undef SCAN
+  return lsh_check_launch("gla_scan_kernel");
+}
+
+}  // namespace
+
+template <typename T>
+int gla_step(const T* proj, long ld, const float* low, const GlaWeights& w, float* state, T* out,
+             const int* row_slot, const int* row_pos, int rows, const GlaShape& sh, hipStream_t s) {
+  if (int rc = check_shape(sh)) return rc;
+  if (!proj || !low || !w.a2 || !w.bias || !w.norm || !state || !out || !row_slot || !row_pos ||
+      rows <= 0)
+    return lsh_fail(LSH_ERR_INVALID, "gla_step: bad arguments");
+  return launch_scan<T>(proj, ld, low, w, state, out, nullptr, row_slot, row_pos, rows, sh, s);
+}
+
+template <typename T>
+int gla_scan(const T* proj, long ld, const float* low, const GlaWeights& w, float* state, T* out,
+             const SeqSpan* seqs, int n_seqs, const GlaShape& sh, hipStream_t s) {
+  if (int rc = check_shape(sh)) return rc;
+  if (!proj || !low || !w.a2 || !w.bias || !w.norm || !state || !out || !seqs || n_seqs <= 0)
+    return lsh_fail(LSH_ERR_INVALID, "gla_scan: bad arguments");
+  return launch_scan<T>(proj, ld, low, w, state, out, seqs, nullptr, nullptr, n_seqs, sh, s);
+}
+
+// columns and rows of the projection in fours, head sizes in sixteens
+bool gla_chunked_supported(const GlaShape& sh, long ld) {
+  return sh.dim % 16 == 0 && sh.vdim % 16 == 0 && sh.dim <= 256 && sh.vdim <= 256 && ld % 4 == 0 &&
+         (sh.q_col | sh.k_col | sh.v_col | sh.g_col) % 4 == 0;
+}
+
+size_t gla_chunked_workspace(int rows, int n_seqs, const GlaShape& sh) {
+  return ((size_t)rows / kC + n_seqs) * sh.heads * chunk_floats(sh);
+}
+
+template <typename T>
+int gla_chunked(const T* proj, long ld, const float* low, const GlaWeights& w, float* state, T* out,
+                float* workspace, const SeqSpan* seqs, int n_seqs, int max_n, int rows,
+                const GlaShape& sh, hipStream_t s) {
+  if (int rc = check_shape(sh)) return rc;
+  if (!proj || !low || !w.a2 || !w.bias || !w.norm || !state || !out || !workspace || !seqs ||
+      n_seqs <= 0 || n_seqs > 65535 || max_n <= 0 || max_n > rows)
+    return lsh_fail(LSH_ERR_INVALID, "gla_chunked: bad arguments");
+  if (!gla_chunked_supported(sh, ld))
+    return lsh_fail(LSH_ERR_UNSUPPORTED, "gla_chunked: head sizes must be multiples of 16");
+  const dim3 grid((max_n + kC - 1) / kC, sh.heads, n_seqs);
+  const int D = sh.dim, VD = sh.vdim;
+  const auto room = [](const void* kernel, size_t lds) {
+    return lsh_check_hip(hipFuncSetAttribute(kernel, hipFuncAttributeMaxDynamicSharedMemorySize,
+                                             (int)lds),
+                         "hipFuncSetAttribute(gla_chunk)");
+  };
+  {
+    auto kern = D <= 32 ? gla_chunk_add_kernel<T, 2> : D <= 64 ? gla_chunk_add_kernel<T, 4>
+              : D <= 128 ? gla_chunk_add_kernel<T, 8> : gla_chunk_add_kernel<T, 16>;
+    const size_t lds = sizeof(float) * ((size_t)(D + VD) * kTS + 4 * D);
+    if (int rc = room(reinterpret_cast<const void*>(kern), lds)) return rc;
+    kern<<<grid, 256, lds, s>>>(proj, ld, low, w, workspace, seqs, sh);
+    if (int rc = lsh_check_launch("gla_chunk_add_kernel")) return rc;
+  }
+  gla_chunk_state_kernel<<<dim3((VD * D / 4 + 255) / 256, sh.heads, n_seqs), 256, 0, s>>>(
+      workspace, state, seqs, sh);
+  if (int rc = lsh_check_launch("gla_chunk_state_kernel")) return rc;
+  const int wide = std::max(D, VD);
+  auto kern = wide <= 32 ? gla_chunk_out_kernel<T, 2> : wide <= 64 ? gla_chunk_out_kernel<T, 4>
+            : wide <= 128 ? gla_chunk_out_kernel<T, 8> : gla_chunk_out_kernel<T, 16>;
+  const size_t lds = sizeof(float) * (48 * (size_t)(D + 4) + 4 * D + (size_t)VD * kTS);
+  if (int rc = room(reinterpret_cast<const void*>(kern), lds)) return rc;
+  kern<<<grid, 256, lds, s>>>(proj, ld, low, w, workspace, out, seqs, sh);
+  return lsh_check_launch("gla_chunk_out_kernel");
+}
+
+#define INST(T)                                                                                     \
+  template int gla_step<T>(const T*, long, const float*, const GlaWeights&, float*, T*, const int*, \
+                           const int*, int, const GlaShape&, hipStream_t);                          \
+  template int gla_scan<T>(const T*, long, const float*, const GlaWeights&, float*, T*,             \
+                           const SeqSpan*, int, const GlaShape&, hipStream_t);                      \
+  template int gla_chunked<T>(const T*, long, const float*, const GlaWeights&, float*, T*, float*,  \
+                              const SeqSpan*, int, int, int, const GlaShape&, hipStream_t);
+INST(float)
+INST(bf16_t)
+
+}  // namespace lsh

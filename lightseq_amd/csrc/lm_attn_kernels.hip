@@ -151,8 +151,9 @@ attn_prepare4_kernel(const T* __restrict__ proj, long ld, int q_col, int k_col, 
 // computed transposed (keys x queries), so a lane owns one query: running maximum, sum and the
 // rescaling of its context need no exchange but one with the other half of the wavefront, and the
 // probabilities are the second operand of the context product as they lie in registers.  The sink
-// is the start value of the running soft-max: maximum 0, sum 1, context 0.
+// is the start value of the running soft-max: its logit as the maximum, sum 1, context 0.
 constexpr int kQT = 128, kKT = 64;
+constexpr float kLog2e = 1.44269504088896340736f;
 
 __device__ __forceinline__ float exp2_f(float x) { return __builtin_amdgcn_exp2f(x); }
 
@@ -181,6 +182,9 @@ attn_prefill_kernel(const T* __restrict__ q, const T* __restrict__ k_cache,
   const int pos = sq.pos0 + my_i;
   const int wq_lo = sq.pos0 + min(i0 + wave * 32, sq.n - 1);
   const int wq_hi = sq.pos0 + min(i0 + wave * 32 + 31, sq.n - 1);
+  // first keys that the wavefront's first, last and this lane's query see (kept ones apart)
+  const int lo_first = mask.first_seen(wq_lo), lo_last = mask.first_seen(wq_hi);
+  const int lo_mine = mask.first_seen(pos);
   const bool wave_live = i0 + wave * 32 < sq.n;
   const int kv_len = sq.pos0 + sq.n;
   const long cache0 = ((long)sq.slot * sh.kv_heads + kvh) * sh.max_step;
@@ -193,15 +197,17 @@ attn_prefill_kernel(const T* __restrict__ q, const T* __restrict__ k_cache,
 #pragma unroll
     for (int s = 0; s < NKS; ++s) qf[s] = *reinterpret_cast<const frag_t*>(qr + (2 * s + g) * V);
   }
-  const float sc2 = mask.scale * 1.44269504088896340736f;
-  float m = mask.sink ? 0.f : -INFINITY, l = mask.sink ? 1.f : 0.f;  // m in units of log2
+  const float sc2 = mask.scale * kLog2e;
+  // m in units of log2
+  float m = !mask.sink ? -INFINITY : mask.sinks ? mask.sinks[head] * kLog2e : 0.f;
+  float l = mask.sink ? 1.f : 0.f;
   f32x16v acc[NV];
 #pragma unroll
   for (int d = 0; d < NV; ++d) acc[d] = (f32x16v)0.f;
 
   const int first_pos = sq.pos0 + i0, last_pos = sq.pos0 + i_last;
   const int t_end = last_pos / kKT;  // last tile
-  const int t_win = mask.window > 0 ? max(0, first_pos - mask.window + 1) / kKT : 0;
+  const int t_win = mask.first_seen(first_pos) / kKT;
   const int t_keep = mask.keep_first > 0 ? (min(mask.keep_first, kv_len) - 1) / kKT : -1;
   // the next tile's keys (16-byte chunks; rows beyond the sequence are clamped, their scores are
   // masked) and values (4 keys x 4 columns per unit; rows beyond it are zero) wait in registers
@@ -258,11 +264,9 @@ attn_prefill_kernel(const T* __restrict__ q, const T* __restrict__ k_cache,
     if (!wave_live) continue;
     // does any query of this wavefront see any key of the tile?
     const bool causal_any = key0 <= wq_hi;
-    const bool win_any = mask.window <= 0 || wq_lo - (key0 + kKT - 1) < mask.window;
+    const bool win_any = key0 + kKT - 1 >= lo_first;
     if (!causal_any || !(win_any || key0 < mask.keep_first)) continue;
-    const bool all = key0 + kKT - 1 <= wq_lo &&
-                     (mask.window <= 0 || wq_hi - key0 < mask.window ||
-                      key0 + kKT <= mask.keep_first);
+    const bool all = key0 + kKT - 1 <= wq_lo && (key0 >= lo_last || key0 + kKT <= mask.keep_first);
     f32x16v sc[2];
 #pragma unroll
     for (int b = 0; b < 2; ++b) {
@@ -280,8 +284,7 @@ attn_prefill_kernel(const T* __restrict__ q, const T* __restrict__ k_cache,
         float v = sc[b][i] * sc2;
         if (!all) {
           const int key = key0 + b * 32 + 8 * (i >> 2) + 4 * g + (i & 3);
-          const bool see = key <= pos && (mask.window <= 0 || pos - key < mask.window ||
-                                          key < mask.keep_first);
+          const bool see = key <= pos && (key >= lo_mine || key < mask.keep_first);
           v = see ? v : -INFINITY;
         }
         sc[b][i] = v;
@@ -429,7 +432,8 @@ struct Packed {
   }
 };
 
-template <typename T, int EK, int EV, int R>  // elements per lane of a key / value row
+// EK, EV: elements per lane of a key / value row; SAME: the values are the keys, read once
+template <typename T, int EK, int EV, int R, bool SAME>
 __global__ void __launch_bounds__(kDecThreads)
 attn_decode_kernel(const T* __restrict__ q, const T* __restrict__ k_cache,
                    const T* __restrict__ v_cache, const T* __restrict__ proj, long ld, int g_col,
@@ -448,7 +452,8 @@ attn_decode_kernel(const T* __restrict__ q, const T* __restrict__ k_cache,
   const long cache0 = ((long)row_slot[row] * sh.kv_heads + kvh) * sh.max_step;
   const T* kc = k_cache + cache0 * DP + j * EK;
   const T* vc = v_cache + cache0 * VP + j * EV;
-  const int lo = mask.window > 0 ? max(0, pos - mask.window + 1) : 0;  // first key of the window
+  static_assert(!SAME || EK == EV, "values of the keys' size");
+  const int lo = mask.first_seen(pos);  // first key of the window
   const int kept = min(mask.keep_first, lo);                           // kept keys before it
   const int n_vis = kept + pos + 1 - lo;
   const int per = ((n_vis + nsplit - 1) / nsplit + 15) & ~15;
@@ -462,7 +467,7 @@ attn_decode_kernel(const T* __restrict__ q, const T* __restrict__ k_cache,
       const int v = min(c0 + u * kDecGroups + grp, v_hi - 1);
       const long key = v < kept ? v : lo + v - kept;
       ko[u].load(kc + key * DP);
-      vo[u].load(vc + key * VP);
+      if constexpr (!SAME) vo[u].load(vc + key * VP);
     }
   };
   if (v_lo < v_hi) fetch(v_lo, kb[0], vb[0]);
@@ -473,7 +478,7 @@ attn_decode_kernel(const T* __restrict__ q, const T* __restrict__ k_cache,
     Packed<T, EK> t;
     t.load(q + ((long)row * sh.heads + h0 + min(r, nh - 1)) * DP + j * EK);
 #pragma unroll
-    for (int e = 0; e < EK; ++e) qv[r][e] = t.get(e) * (mask.scale * 1.44269504088896340736f);
+    for (int e = 0; e < EK; ++e) qv[r][e] = t.get(e) * (mask.scale * kLog2e);
 #pragma unroll
     for (int e = 0; e < EV; ++e) acc[r][e] = 0.f;
     m[r] = -INFINITY;
@@ -512,7 +517,7 @@ attn_decode_kernel(const T* __restrict__ q, const T* __restrict__ k_cache,
         const float p = exp2_f(s[u][r] - ref);
         l[r] += p;
 #pragma unroll
-        for (int e = 0; e < EV; ++e) acc[r][e] = fmaf(p, vi[u].get(e), acc[r][e]);
+        for (int e = 0; e < EV; ++e) acc[r][e] = fmaf(p, SAME ? ki[u].get(e) : vi[u].get(e), acc[r][e]);
       }
     }
   };
@@ -550,10 +555,11 @@ attn_decode_kernel(const T* __restrict__ q, const T* __restrict__ k_cache,
   const bool sink = mask.sink && split == 0;
   for (int x = tid; x < nh * VP; x += kDecThreads) {
     const int r = x / VP, c = x - r * VP;
-    float mx = sink ? 0.f : -INFINITY;
+    const float sink2 = sink && mask.sinks ? mask.sinks[h0 + r] * kLog2e : 0.f;
+    float mx = sink ? sink2 : -INFINITY;
 #pragma unroll
     for (int w = 0; w < 8; ++w) mx = fmaxf(mx, pm[w][r]);
-    float a = 0.f, t = sink ? exp2_f(-mx) : 0.f;
+    float a = 0.f, t = sink ? exp2_f(sink2 - mx) : 0.f;
 #pragma unroll
     for (int w = 0; w < 8; ++w) {
       const float f = pm[w][r] == -INFINITY ? 0.f : exp2_f(pm[w][r] - mx);
@@ -618,16 +624,16 @@ int attn_prepare(const T* proj, long ld, int q_col, int k_col, int v_col, const 
                  T* k_cache, T* v_cache, const int* row_slot, const int* row_pos, int rows,
                  const AttnShape& sh, hipStream_t s) {
   if (int rc = check_shape(sh, "attn_prepare: bad shape")) return rc;
+  const bool own = k_col >= 0, values = own && v_col >= 0;
   if (!proj || !q_out || !row_slot || !row_pos || rows <= 0 || rot_pairs < 0 ||
-      2 * rot_pairs > sh.dim || (rot_pairs > 0 && !cos_sin) ||
-      (k_col >= 0 && (!k_cache || !v_cache || v_col < 0)))
+      2 * rot_pairs > sh.dim || (rot_pairs > 0 && !cos_sin) || (own && !k_cache) ||
+      (values && !v_cache))
     return lsh_fail(LSH_ERR_INVALID, "attn_prepare: bad arguments");
-  const int per_row = sh.heads + (k_col >= 0 ? 2 * sh.kv_heads : 0);
+  const int per_row = sh.heads + (own ? sh.kv_heads : 0) + (values ? sh.kv_heads : 0);
   const long units = (long)rows * per_row;
-  const bool own = k_col >= 0;
   if (sh.dim % 4 == 0 && ld % 4 == 0 && q_col % 4 == 0 && units < (1L << 24) &&
-      (!own || (sh.vdim % 4 == 0 && k_col % 4 == 0 && v_col % 4 == 0))) {
-    const int pad = own ? std::max(sh.dim_pad, sh.vdim_pad) : sh.dim_pad;
+      (!own || k_col % 4 == 0) && (!values || (sh.vdim % 4 == 0 && v_col % 4 == 0))) {
+    const int pad = values ? std::max(sh.dim_pad, sh.vdim_pad) : sh.dim_pad;
 #define PREP4(LPH)                                                                              \
   attn_prepare4_kernel<T, LPH><<<(unsigned)((units * LPH + 255) / 256), 256, 0, s>>>(           \
       proj, ld, q_col, k_col, v_col, q_norm, k_norm, eps, cos_sin, rot_pairs, q_out, k_cache,   \
@@ -662,7 +668,8 @@ int attn_prefill(const T* q, const T* k_cache, const T* v_cache, const T* proj, 
                  const AttnMask& mask, hipStream_t s) {
   if (int rc = check_shape(sh, "attn_prefill: bad shape")) return rc;
   if (!q || !k_cache || !v_cache || !out || !seqs || n_seqs <= 0 || max_n <= 0 ||
-      (g_col >= 0 && !proj) || n_seqs > 65535 || sh.heads > 65535)
+      (g_col >= 0 && !proj) || n_seqs > 65535 || sh.heads > 65535 ||
+      (v_cache == k_cache && sh.dim != sh.vdim) || mask.chunk < 0)
     return lsh_fail(LSH_ERR_INVALID, "attn_prefill: bad arguments");
   switch (sh.dim_pad / 32) {
     case 2: PICK_V(2)
@@ -676,22 +683,23 @@ size_t attn_decode_workspace(int rows, const AttnShape& sh) {
   return (size_t)rows * sh.heads * kMaxSplit * (sh.vdim_pad + 2);
 }
 
-#define DEC(EK, EV, R)                                                                           \
-  attn_decode_kernel<T, EK, EV, R><<<grid, kDecThreads, 0, s>>>(q, k_cache, v_cache, proj, ld, g_col,    \
-                                                        out, row_slot, row_pos, nsplit, groups,  \
-                                                        workspace, sh, mask)
-#define DEC_R(EK, EV)                                                                            \
+#define DEC(EK, EV, R, SAME)                                                                     \
+  attn_decode_kernel<T, EK, EV, R, SAME><<<grid, kDecThreads, 0, s>>>(                           \
+      q, k_cache, v_cache, proj, ld, g_col, out, row_slot, row_pos, nsplit, groups, workspace,   \
+      sh, mask)
+#define DEC_R(EK, EV, SAME)                                                                      \
   do {                                                                                           \
-    if (R == 1) DEC(EK, EV, 1);                                                                  \
-    else if (R == 2) DEC(EK, EV, 2);                                                             \
-    else DEC(EK, EV, 4);                                                                         \
+    if (R == 1) DEC(EK, EV, 1, SAME);                                                            \
+    else if (R == 2) DEC(EK, EV, 2, SAME);                                                       \
+    else DEC(EK, EV, 4, SAME);                                                                   \
   } while (0)
 #define DEC_V(EK)                                                                                \
-  switch (sh.vdim_pad / 16) {                                                                    \
-    case 4: DEC_R(EK, 4); break;                                                                 \
-    case 6: DEC_R(EK, 6); break;                                                                 \
-    case 8: DEC_R(EK, 8); break;                                                                 \
-    default: DEC_R(EK, 16); break;                                                               \
+  if (v_cache == k_cache) DEC_R(EK, EK, true);                                                   \
+  else switch (sh.vdim_pad / 16) {                                                               \
+    case 4: DEC_R(EK, 4, false); break;                                                          \
+    case 6: DEC_R(EK, 6, false); break;                                                          \
+    case 8: DEC_R(EK, 8, false); break;                                                          \
+    default: DEC_R(EK, 16, false); break;                                                        \
   }
 
 template <typename T>
@@ -700,7 +708,8 @@ int attn_decode(const T* q, const T* k_cache, const T* v_cache, const T* proj, l
                 float* workspace, const AttnShape& sh, const AttnMask& mask, hipStream_t s) {
   if (int rc = check_shape(sh, "attn_decode: bad shape")) return rc;
   if (!q || !k_cache || !v_cache || !out || !row_slot || !row_pos || rows <= 0 || max_len <= 0 ||
-      !workspace || (g_col >= 0 && !proj))
+      !workspace || (g_col >= 0 && !proj) || (v_cache == k_cache && sh.dim != sh.vdim) ||
+      mask.chunk < 0)
     return lsh_fail(LSH_ERR_INVALID, "attn_decode: bad arguments");
   const int rep = sh.heads / sh.kv_heads;
   // heads per workgroup: several share the loads of a key, but only as many as leave the chip filled
@@ -708,8 +717,9 @@ int attn_decode(const T* q, const T* k_cache, const T* v_cache, const T* proj, l
   const long each = (long)rows * sh.kv_heads, fill = 2L * cu_count();
   const int R = rep == 1 || each * rep <= fill ? 1 : rep == 2 || each * ((rep + 1) / 2) <= fill ? 2 : 4;
   const int groups = (rep + R - 1) / R;
-  const long most = mask.window > 0 ? std::min((long)max_len, (long)mask.window + mask.keep_first)
-                                    : (long)max_len;
+  long most = max_len;
+  if (mask.window > 0) most = std::min(most, (long)mask.window + mask.keep_first);
+  if (mask.chunk > 0) most = std::min(most, (long)mask.chunk + mask.keep_first);
   // enough workgroups to fill the chip, but parts of at least 1024 keys: a shorter part is done
   // before the launch that would join the parts has started
   const int want = (int)((2L * cu_count() + (long)rows * sh.kv_heads * groups - 1) /

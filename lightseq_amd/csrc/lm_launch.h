@@ -20,13 +20,24 @@ struct SeqSpan {
 // C[m, n] = sum_k A[m, k] W[n, k].  Columns from n_split on go to the float matrix C2 (column
 // n - n_split); n_split = N: none.  `planes` > 1 asks for that many partial sums over K, stored as
 // float planes [planes][M][N] that the caller adds (few rows only; *planes_used says how many).
+// The epilogue gives scale * sum + bias[n] (in float, before the result is rounded).
+struct GemmEpilogue {
+  float scale = 1.f;
+  const float* bias = nullptr;  // [N]
+};
 template <typename T, typename TO>
 int gemm_float(const T* A, long lda, const T* W, TO* C, long ldc, float* C2, long ld2, int n_split,
-               int M, int N, int K, hipStream_t s);
+               int M, int N, int K, hipStream_t s, const GemmEpilogue& epilogue = GemmEpilogue());
 template <typename T>
 int gemm_float_planes(const T* A, long lda, const T* W, float* C, int M, int N, int K,
                       int max_planes, int* planes_used, hipStream_t s);
 int gemm_float_preferred_planes(int M, int N, int K);
+
+// C[m, n] = act(gate_n A[m]) * (up_n A[m]), weights [2][N][K]: the gates' rows, then the others
+enum GateAct { kGateSilu = 0, kGateRelu = 1 };
+template <typename T>
+int gemm_gated(const T* A, long lda, const T* W, T* C, long ldc, int M, int N, int K, int act,
+               hipStream_t s);
 
 // Products over the rows that chose an expert.  A row is a (token, choice) pair, numbered
 // token * top + choice; expert e serves rows list[e * tokens + 0 .. count[e]).
@@ -50,26 +61,43 @@ int moe_router(const T* h, const T* w, const float* bias, float* weight, int* co
                int tokens, int width, int experts, int top, hipStream_t s);
 
 // ---- norms on the residual stream (lm_norm_kernels.hip) ---------------------------------------
-// What is added to the residual row before the norm: parts many summands, part p of row r at
+enum NormKind {
+  kLayerNorm = 0,  // (x - mean) / deviation * w + b
+  kRmsNorm = 1,    // x / root mean square * w
+};
+// A summand of the residual row: parts many pieces, piece p of row r at
 // y + p * part_stride + r * row_stride, times weight[r * parts + p] when weights are given.
-struct AddSpec {
+struct AddPart {
   const void* y = nullptr;
-  bool y_is_float = true;  // else T
   int parts = 0;
   long part_stride = 0, row_stride = 0;
   const float* weight = nullptr;
-  const float *post_w = nullptr, *post_b = nullptr;  // layer norm of the sum before it is added
+  const float *post_w = nullptr, *post_b = nullptr;  // norm of the sum of the pieces; null: none
+};
+// What is added before the norm: scale * (this summand + the second one).
+struct AddSpec : AddPart {
+  bool y_is_float = true;  // else T
+  AddPart second;          // parts == 0: none
+  float scale = 1.f;
+  NormKind post_kind = kLayerNorm;
 };
 struct NormSpec {
-  const float *w = nullptr, *b = nullptr;  // layer norm of the new residual row; null: no output
+  const float *w = nullptr, *b = nullptr;  // norm of the new residual row; w null: no output
+  NormKind kind = kLayerNorm;
 };
-// x[r] (+)= LN_post(sum of parts); h[r] = LN(x[r]).  With `ids`, x[r] = embed[ids[r]] instead.
+// Added to the row after that, ahead of the norm: its embedding again and / or a vector.
+struct InjectSpec {
+  const int* ids = nullptr;
+  const float* vec = nullptr;  // [width]
+  __host__ __device__ bool any() const { return ids || vec; }
+};
+// x[r] (+)= add; x[r] (+)= inject; h[r] = norm(x[r]).  With `ids`, x[r] = embed[ids[r]] to begin with.
 // With `rows`, output row i comes from residual row rows[i] (no addition then).
 // zero_count: n_zero ints set to zero for the routing that follows.
 template <typename T>
 int lm_norm(float* x, const AddSpec& add, const NormSpec& norm, T* h, int rows_n, int width,
             float eps, const int* ids, const T* embed, int vocab, const int* rows, int* zero_count,
-            int n_zero, hipStream_t s);
+            int n_zero, hipStream_t s, const InjectSpec& inject = InjectSpec());
 
 // ---- attention (lm_attn_kernels.hip) ----------------------------------------------------------
 struct AttnShape {
@@ -80,19 +108,32 @@ struct AttnShape {
 int attn_pad(int dim);  // 0: not supported
 // Per-head RMS norm (q and, unless shared, k), interleaved rotation with the table
 // cos_sin[position][rot_pairs] of float2 (null: none), then q -> q_out[row][heads][dim_pad] and
-// k, v -> slot caches [slot][kv_head][position][pad].  k_col < 0: the layer has no keys of its own.
+// k, v -> slot caches [slot][kv_head][position][pad].  k_col < 0: the layer has no keys of its own;
+// v_col < 0: its values are the keys.  Without norm weights there is no norm.
 template <typename T>
 int attn_prepare(const T* proj, long ld, int q_col, int k_col, int v_col, const float* q_norm,
                  const float* k_norm, float eps, const float2* cos_sin, int rot_pairs, T* q_out,
                  T* k_cache, T* v_cache, const int* row_slot, const int* row_pos, int rows,
                  const AttnShape& sh, hipStream_t s);
-// Position i sees j <= i with i - j < window or j < keep_first (window <= 0: all).  sink: one is
-// added to the soft-max denominator.  out[row][heads * vdim] = context * sigmoid(gate) (gate: T
+// Position i sees j <= i with i - j < window or j < keep_first (window <= 0: all), and with a chunk
+// size only keys of its own chunk of positions (or kept ones).  sink: exp(sinks[head]) is added to
+// the soft-max denominator, 1 without sinks.  v_cache == k_cache: the values are the keys.  out[row][heads * vdim] = context * sigmoid(gate) (gate: T
 // columns of `proj` from g_col on; g_col < 0: none).
 struct AttnMask {
   int window, keep_first;
   float scale;
   bool sink;
+  int chunk = 0;                 // 0: none
+  const float* sinks = nullptr;  // [heads]
+  // the first position that `pos` sees beside the kept ones
+  __host__ __device__ int first_seen(int pos) const {
+    int lo = window > 0 && pos >= window ? pos - window + 1 : 0;
+    if (chunk > 0) {
+      const int c = pos - pos % chunk;
+      lo = lo > c ? lo : c;
+    }
+    return lo;
+  }
 };
 template <typename T>
 int attn_prefill(const T* q, const T* k_cache, const T* v_cache, const T* proj, long ld, int g_col,
@@ -143,6 +184,35 @@ int delta_step(const T* proj, long ld, int g_col, const float* ba, const float* 
                const float* a_log, const float* dt_bias, const float* norm_w, float eps,
                T* conv_ring, float* state, T* out, const int* row_slot, const int* row_pos,
                int rows, const DeltaShape& sh, hipStream_t s);
+
+// ---- gated linear attention (gla_kernels.hip) ---------------------------------------------------
+//   S <- diag(a) S + k v^T;  o = S^T (q dim^-1/2)  per head, a = sigmoid(A2 low + bias)^(1 / tau),
+//   out = o / rms(o) * norm_w * silu(gate)
+// proj rows hold q, k [heads][dim] and v, gate [heads][vdim] from the given columns on; `low` is the
+// narrow product that the decay is made from, float [rows][rank] (rank: a multiple of 16, zero-padded);
+// a2 [heads * dim][rank].  state [slot][heads][vdim][dim] in float.
+struct GlaShape {
+  int heads, dim, vdim, rank;
+  int q_col, k_col, v_col, g_col;
+  float inv_tau, eps;
+};
+struct GlaWeights {
+  const float *a2, *bias, *norm;
+};
+// one token per sequence, row r at position row_pos[r] of slot row_slot[r]
+template <typename T>
+int gla_step(const T* proj, long ld, const float* low, const GlaWeights& w, float* state, T* out,
+             const int* row_slot, const int* row_pos, int rows, const GlaShape& sh, hipStream_t s);
+// whole spans: token by token / in chunks of 64 on the matrix cores
+template <typename T>
+int gla_scan(const T* proj, long ld, const float* low, const GlaWeights& w, float* state, T* out,
+             const SeqSpan* seqs, int n_seqs, const GlaShape& sh, hipStream_t s);
+template <typename T>
+int gla_chunked(const T* proj, long ld, const float* low, const GlaWeights& w, float* state, T* out,
+                float* workspace, const SeqSpan* seqs, int n_seqs, int max_n, int rows,
+                const GlaShape& sh, hipStream_t s);
+size_t gla_chunked_workspace(int rows, int n_seqs, const GlaShape& sh);  // floats
+bool gla_chunked_supported(const GlaShape& sh, long ld);
 
 // ---- sampling from float logits (lm_sample_kernels.hip) ---------------------------------------
 // Chooses a token per row (greedy: topk == 1; topk > 1; or topp in (0, 1] with topk == 0), writes

@@ -1,7 +1,8 @@
-// The residual stream of a floating-point decoder and its layer norms, in float32: one workgroup
+// The residual stream of a floating-point decoder and its norms, in float32: one workgroup
 // per row, the row in registers.  One launch adds a sublayer's output to the residual (after that
-// sublayer's own norm, from partial sums or weighted expert outputs as they lie in memory) and
-// applies the norm ahead of the next sublayer; another starts the stream from the embedding table.
+// sublayer's own norm, from partial sums or weighted expert outputs as they lie in memory; or that of
+// two sublayers side by side) and applies the norm ahead of the next sublayer; another starts the
+// stream from the embedding table.
 #include "lm_launch.h"
 
 namespace lsh {
@@ -21,24 +22,25 @@ struct NormArgs {
   const int* rows;
   int* zero_count;
   int n_zero;
+  InjectSpec inject;
 };
 
 // V elements per access, NI accesses per thread: width <= 256 * V * NI
 template <typename T, typename TY, int V, int NI>
 __global__ void __launch_bounds__(256)
 lm_norm_kernel(NormArgs a) {
-  __shared__ float red[4][16];
+  __shared__ float red[6][16];
   const int tid = threadIdx.x, W = a.width;
   const long r = blockIdx.x;
   if (r == 0 && a.n_zero > 0)
     for (int i = tid; i < a.n_zero; i += 256) a.zero_count[i] = 0;
   float* xr = a.x + (a.rows ? (long)a.rows[r] : r) * W;
   float x[NI][V];
-  const T* er = nullptr;
-  if (a.ids) {
-    const int id = a.ids[r];
-    er = reinterpret_cast<const T*>(a.embed) + (long)min(max(id, 0), a.vocab - 1) * W;
-  }
+  const auto embed_row = [&](const int* ids) {
+    return ids ? reinterpret_cast<const T*>(a.embed) + (long)min(max(ids[r], 0), a.vocab - 1) * W
+               : nullptr;
+  };
+  const T* er = embed_row(a.ids);
 #pragma unroll
   for (int i = 0; i < NI; ++i) {
     const int c = (i * 256 + tid) * V;
@@ -50,9 +52,19 @@ lm_norm_kernel(NormArgs a) {
     }
   }
   const float inv_w = 1.f / (float)W;
-  // mean and reciprocal deviation of a row held as v
-  auto stats = [&](const float (&v)[NI][V], float& mean, float& rstd, int which) {
+  // mean and reciprocal deviation of a row held as v (zeros beyond the width); 0 and the reciprocal
+  // root mean square
+  auto stats = [&](const float (&v)[NI][V], NormKind kind, float& mean, float& rstd, int which) {
     float s = 0.f;
+    if (kind == kRmsNorm) {
+#pragma unroll
+      for (int i = 0; i < NI; ++i)
+#pragma unroll
+        for (int k = 0; k < V; ++k) s += v[i][k] * v[i][k];
+      mean = 0.f;
+      rstd = 1.0f / sqrtf(block_sum_dpp(s, red[which]) * inv_w + a.eps);
+      return;
+    }
 #pragma unroll
     for (int i = 0; i < NI; ++i)
 #pragma unroll
@@ -70,46 +82,70 @@ lm_norm_kernel(NormArgs a) {
       }
     rstd = 1.0f / sqrtf(block_sum_dpp(s, red[which + 1]) * inv_w + a.eps);
   };
-  if (a.add.parts > 0) {
+  auto add = [&](const AddPart& p0, int which) {
     float y[NI][V];
 #pragma unroll
     for (int i = 0; i < NI; ++i)
 #pragma unroll
       for (int k = 0; k < V; ++k) y[i][k] = 0.f;
-    const TY* yr = reinterpret_cast<const TY*>(a.add.y) + r * a.add.row_stride;
-    for (int p = 0; p < a.add.parts; ++p) {
-      const float wt = a.add.weight ? a.add.weight[r * a.add.parts + p] : 1.f;
+    const TY* yr = reinterpret_cast<const TY*>(p0.y) + r * p0.row_stride;
+    for (int p = 0; p < p0.parts; ++p) {
+      const float wt = p0.weight ? p0.weight[r * p0.parts + p] : 1.f;
 #pragma unroll
       for (int i = 0; i < NI; ++i) {
         const int c = (i * 256 + tid) * V;
         if (c < W) {
           float t[V];
-          ldv<V, TY>(yr + p * a.add.part_stride + c, t);
+          ldv<V, TY>(yr + p * p0.part_stride + c, t);
 #pragma unroll
           for (int k = 0; k < V; ++k) y[i][k] += wt * t[k];
         }
       }
     }
     float mean = 0.f, rstd = 1.f;
-    if (a.add.post_w) stats(y, mean, rstd, 0);
+    if (p0.post_w) stats(y, a.add.post_kind, mean, rstd, which);
 #pragma unroll
     for (int i = 0; i < NI; ++i) {
       const int c = (i * 256 + tid) * V;
       if (c < W) {
-        if (a.add.post_w) {
+        if (p0.post_w) {
           float w[V], b[V];
-          ldv<V, float>(a.add.post_w + c, w);
-          ldv<V, float>(a.add.post_b + c, b);
+          ldv<V, float>(p0.post_w + c, w);
 #pragma unroll
-          for (int k = 0; k < V; ++k) x[i][k] += (y[i][k] - mean) * rstd * w[k] + b[k];
+          for (int k = 0; k < V; ++k) b[k] = 0.f;
+          if (p0.post_b) ldv<V, float>(p0.post_b + c, b);
+#pragma unroll
+          for (int k = 0; k < V; ++k) x[i][k] += a.add.scale * ((y[i][k] - mean) * rstd * w[k] + b[k]);
         } else {
 #pragma unroll
-          for (int k = 0; k < V; ++k) x[i][k] += y[i][k];
+          for (int k = 0; k < V; ++k) x[i][k] += a.add.scale * y[i][k];
+        }
+      }
+    }
+  };
+  if (a.add.parts > 0) add(a.add, 0);
+  if (a.add.second.parts > 0) add(a.add.second, 2);
+  if (a.inject.any()) {
+    const T* ir = embed_row(a.inject.ids);
+#pragma unroll
+    for (int i = 0; i < NI; ++i) {
+      const int c = (i * 256 + tid) * V;
+      if (c < W) {
+        float t[V];
+        if (ir) {
+          ldv<V, T>(ir + c, t);
+#pragma unroll
+          for (int k = 0; k < V; ++k) x[i][k] += t[k];
+        }
+        if (a.inject.vec) {
+          ldv<V, float>(a.inject.vec + c, t);
+#pragma unroll
+          for (int k = 0; k < V; ++k) x[i][k] += t[k];
         }
       }
     }
   }
-  if (a.add.parts > 0 || a.ids) {
+  if (a.add.parts > 0 || a.ids || a.inject.any()) {
 #pragma unroll
     for (int i = 0; i < NI; ++i) {
       const int c = (i * 256 + tid) * V;
@@ -118,7 +154,7 @@ lm_norm_kernel(NormArgs a) {
   }
   if (!a.norm.w) return;
   float mean, rstd;
-  stats(x, mean, rstd, 2);
+  stats(x, a.norm.kind, mean, rstd, 4);
   T* hr = reinterpret_cast<T*>(a.h) + r * W;
 #pragma unroll
   for (int i = 0; i < NI; ++i) {
@@ -126,7 +162,9 @@ lm_norm_kernel(NormArgs a) {
     if (c < W) {
       float w[V], b[V], o[V];
       ldv<V, float>(a.norm.w + c, w);
-      ldv<V, float>(a.norm.b + c, b);
+#pragma unroll
+      for (int k = 0; k < V; ++k) b[k] = 0.f;
+      if (a.norm.b) ldv<V, float>(a.norm.b + c, b);
 #pragma unroll
       for (int k = 0; k < V; ++k) o[k] = (x[i][k] - mean) * rstd * w[k] + b[k];
       stv<V, T>(hr + c, o);
@@ -136,7 +174,8 @@ lm_norm_kernel(NormArgs a) {
 
 template <typename T, typename TY>
 int launch_norm(const NormArgs& a, int rows, hipStream_t s) {
-  const bool vec = a.width % 4 == 0 && a.add.part_stride % 4 == 0 && a.add.row_stride % 4 == 0;
+  const bool vec = a.width % 4 == 0 && a.add.part_stride % 4 == 0 && a.add.row_stride % 4 == 0 &&
+                   a.add.second.part_stride % 4 == 0 && a.add.second.row_stride % 4 == 0;
   const int per = 256 * (vec ? 4 : 1);
   const int ni = (a.width + per - 1) / per;
   if (vec) {
@@ -158,17 +197,24 @@ int launch_norm(const NormArgs& a, int rows, hipStream_t s) {
 template <typename T>
 int lm_norm(float* x, const AddSpec& add, const NormSpec& norm, T* h, int rows_n, int width,
             float eps, const int* ids, const T* embed, int vocab, const int* rows, int* zero_count,
-            int n_zero, hipStream_t s) {
-  if (!x || rows_n <= 0 || width <= 0 || (ids && !embed) || (add.parts > 0 && !add.y) ||
-      (norm.w && (!norm.b || !h)) || (add.post_w && !add.post_b) || (rows && (add.parts > 0 || ids)))
+            int n_zero, hipStream_t s, const InjectSpec& inject) {
+  const bool adds = add.parts > 0 || add.second.parts > 0 || inject.any();
+  if (!x || rows_n <= 0 || width <= 0 || ((ids || inject.ids) && (!embed || vocab <= 0)) ||
+      (add.parts > 0 && !add.y) || (add.second.parts > 0 && (add.parts <= 0 || !add.second.y)) ||
+      (norm.w && !h) || (rows && (adds || ids)) ||
+      (norm.w && norm.kind == kLayerNorm && !norm.b) ||
+      (add.post_w && add.post_kind == kLayerNorm && !add.post_b) ||
+      (add.second.post_w && add.post_kind == kLayerNorm && !add.second.post_b))
     return lsh_fail(LSH_ERR_INVALID, "lm_norm: bad arguments");
   const NormArgs a{x, add, norm, h, width, eps, ids, embed, vocab, rows, zero_count,
-                   zero_count ? n_zero : 0};
+                   zero_count ? n_zero : 0, inject};
   return add.y_is_float ? launch_norm<T, float>(a, rows_n, s) : launch_norm<T, T>(a, rows_n, s);
 }
 template int lm_norm<float>(float*, const AddSpec&, const NormSpec&, float*, int, int, float,
-                            const int*, const float*, int, const int*, int*, int, hipStream_t);
+                            const int*, const float*, int, const int*, int*, int, hipStream_t,
+                            const InjectSpec&);
 template int lm_norm<bf16_t>(float*, const AddSpec&, const NormSpec&, bf16_t*, int, int, float,
-                             const int*, const bf16_t*, int, const int*, int*, int, hipStream_t);
+                             const int*, const bf16_t*, int, const int*, int*, int, hipStream_t,
+                             const InjectSpec&);
 
 }  // namespace lsh

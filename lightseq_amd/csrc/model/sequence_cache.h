@@ -54,9 +54,10 @@ class SequenceSlots {
 // Storage of one layer; T is the type of the activations.
 template <typename T>
 struct LayerCache {
-  DeviceBuffer<T> k, v;         // attention layers with keys of their own
+  DeviceBuffer<T> k, v;         // attention with keys of its own (no v: the values are the keys)
   DeviceBuffer<T> conv;         // delta layers: ring of the convolutions' inputs
-  DeviceBuffer<float> state;    // delta layers: [slot][heads][dim][vdim]
+  DeviceBuffer<float> state;    // recurrent layers: delta [slot][heads][dim][vdim], gated linear
+                                // attention [slot][heads][vdim][dim]
 };
 
 }  // namespace hip
