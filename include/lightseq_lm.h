@@ -29,17 +29,44 @@ typedef struct lsh_attn_shape_t {
 typedef struct lsh_attn_mask_t {
   int window, keep_first; /* position i sees j <= i with i - j < window (<= 0: any) or j < keep_first */
   float scale;
-  int sink;               /* one is added to the soft-max denominator */
+  int sink;               /* exp(sinks[head]) is added to the soft-max denominator, 1 without sinks */
+  int chunk;              /* > 0: only keys of the query's own chunk of so many positions (or kept ones) */
+  const float* sinks;     /* device, [heads], or null */
 } lsh_attn_mask_t;
 typedef struct lsh_delta_shape_t {
   int heads, kv_heads, dim, vdim, taps;
 } lsh_delta_shape_t;
+
+/* a summand of the residual row; post_w null: no norm of its own */
+typedef struct lsh_residual_part_t {
+  const void* y; /* null: none */
+  int parts;
+  int64_t part_stride, row_stride;
+  const float *weight, *post_w, *post_b;
+} lsh_residual_part_t;
+/* x <- x + scale * (part 0 + part 1) + embed[inject_ids] + inject_vec;  h = norm(x) */
+typedef struct lsh_residual_t {
+  lsh_residual_part_t part[2];
+  int y_is_float;          /* else the parts have the activations' type */
+  int post_rms, norm_rms;  /* root-mean-square norms (no mean, no bias) instead of layer norms */
+  float scale;
+  const float *norm_w, *norm_b; /* norm_w null: no output */
+  const int* inject_ids;        /* null: none */
+  const float* inject_vec;      /* null: none */
+} lsh_residual_t;
+typedef struct lsh_gla_shape_t {
+  int heads, dim, vdim, rank;      /* rank: a multiple of 16 */
+  int q_col, k_col, v_col, g_col;  /* columns of the projection */
+  float tau, eps;
+} lsh_gla_shape_t;
 
 /* row length of the key and value caches [slot][kv_head][max_step][pad]; 0: not supported */
 int lsh_lm_attn_pad(int dim);
 int64_t lsh_lm_attn_decode_workspace(int rows, const lsh_attn_shape_t* shape);           /* floats */
 int64_t lsh_lm_delta_chunked_workspace(int rows, int n_seqs, const lsh_delta_shape_t* shape);
 int lsh_lm_delta_chunked_supported(const lsh_delta_shape_t* shape);
+int64_t lsh_lm_gla_chunked_workspace(int rows, int n_seqs, const lsh_gla_shape_t* shape); /* floats */
+int lsh_lm_gla_chunked_supported(const lsh_gla_shape_t* shape, int64_t ld);
 
 int lsh_lm_moe_route(const float* logits, const float* bias, float* weight, int* count, int* list,
                      int tokens, int experts, int top, lsh_stream_t stream);
@@ -137,6 +164,39 @@ int lsh_lm_delta_step_bf16(const void* proj, int64_t ld, int g_col, const float*
     float* conv_w, const float* a_log, const float* dt_bias, const float* norm_w, float eps, void*
     conv_ring, float* state, void* out, const int* row_slot, const int* row_pos, int rows, const
     lsh_delta_shape_t* sh, lsh_stream_t stream);
+
+int lsh_lm_gemm_epilogue_f32(const void* A, int64_t lda, const void* W, void* C, int64_t ldc,
+    float* C2, int64_t ld2, int n_split, int M, int N, int K, float scale, const float* bias,
+    lsh_stream_t stream);
+int lsh_lm_gemm_gated_f32(const void* A, int64_t lda, const void* W, void* C, int64_t ldc, int M,
+    int N, int K, int act, lsh_stream_t stream); /* act 0: silu, 1: relu */
+int lsh_lm_residual_f32(float* x, const lsh_residual_t* what, void* h, int rows, int width, float eps,
+    const int* ids, const void* embed, int vocab, lsh_stream_t stream);
+int lsh_lm_gla_step_f32(const void* proj, int64_t ld, const float* low, const float* a2, const float*
+    bias, const float* norm, float* state, void* out, const int* row_slot, const int* row_pos, int
+    rows, const lsh_gla_shape_t* sh, lsh_stream_t stream);
+int lsh_lm_gla_scan_f32(const void* proj, int64_t ld, const float* low, const float* a2, const float*
+    bias, const float* norm, float* state, void* out, const lsh_seq_span_t* seqs, int n_seqs, const
+    lsh_gla_shape_t* sh, lsh_stream_t stream);
+int lsh_lm_gla_chunked_f32(const void* proj, int64_t ld, const float* low, const float* a2, const
+    float* bias, const float* norm, float* state, void* out, float* workspace, const lsh_seq_span_t*
+    seqs, int n_seqs, int max_n, int rows, const lsh_gla_shape_t* sh, lsh_stream_t stream);
+int lsh_lm_gemm_epilogue_bf16(const void* A, int64_t lda, const void* W, void* C, int64_t ldc,
+    float* C2, int64_t ld2, int n_split, int M, int N, int K, float scale, const float* bias,
+    lsh_stream_t stream);
+int lsh_lm_gemm_gated_bf16(const void* A, int64_t lda, const void* W, void* C, int64_t ldc, int M,
+    int N, int K, int act, lsh_stream_t stream); /* act 0: silu, 1: relu */
+int lsh_lm_residual_bf16(float* x, const lsh_residual_t* what, void* h, int rows, int width, float eps,
+    const int* ids, const void* embed, int vocab, lsh_stream_t stream);
+int lsh_lm_gla_step_bf16(const void* proj, int64_t ld, const float* low, const float* a2, const float*
+    bias, const float* norm, float* state, void* out, const int* row_slot, const int* row_pos, int
+    rows, const lsh_gla_shape_t* sh, lsh_stream_t stream);
+int lsh_lm_gla_scan_bf16(const void* proj, int64_t ld, const float* low, const float* a2, const float*
+    bias, const float* norm, float* state, void* out, const lsh_seq_span_t* seqs, int n_seqs, const
+    lsh_gla_shape_t* sh, lsh_stream_t stream);
+int lsh_lm_gla_chunked_bf16(const void* proj, int64_t ld, const float* low, const float* a2, const
+    float* bias, const float* norm, float* state, void* out, float* workspace, const lsh_seq_span_t*
+    seqs, int n_seqs, int max_n, int rows, const lsh_gla_shape_t* sh, lsh_stream_t stream);
 
 #ifdef __cplusplus
 }

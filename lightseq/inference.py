@@ -8,9 +8,9 @@
 run unchanged.  The float models of that module (Transformer, Gpt, Bert, Moe, Vit, T5 ...)
 are not part of this build and raise on access with a message that says so.
 """
-from lightseq_amd.inference import DecoderModel, QuantBert, QuantGpt, QuantTransformer, Sudevik  # noqa: F401
+from lightseq_amd.inference import DecoderModel, QuantBert, QuantGpt, QuantTransformer, Sudevik, Gebuzen  # noqa: F401
 
-__all__ = ["DecoderModel", "QuantBert", "QuantGpt", "QuantTransformer", "Sudevik"]
+__all__ = ["DecoderModel", "QuantBert", "QuantGpt", "QuantTransformer", "Sudevik", "Gebuzen"]
 
 _NOT_BUILT = ("Transformer", "Gpt", "Bert", "Moe", "Vit", "T5", "MT5", "XGLM", "QuantVit")
 

@@ -12,7 +12,17 @@ namespace {
 AttnShape shape_of(const lsh_attn_shape_t& a) {
   return AttnShape{a.heads, a.kv_heads, a.dim, a.vdim, attn_pad(a.dim), attn_pad(a.vdim), a.max_step};
 }
-AttnMask mask_of(const lsh_attn_mask_t& m) { return AttnMask{m.window, m.keep_first, m.scale, m.sink != 0}; }
+AttnMask mask_of(const lsh_attn_mask_t& m) {
+  return AttnMask{m.window, m.keep_first, m.scale, m.sink != 0, m.chunk, m.sinks};
+}
+GlaShape shape_of(const lsh_gla_shape_t& g) {
+  return GlaShape{g.heads, g.dim, g.vdim, g.rank, g.q_col, g.k_col, g.v_col, g.g_col,
+                  1.f / g.tau, g.eps};
+}
+void part_of(const lsh_residual_part_t& p, AddPart& out) {
+  if (!p.y) return;
+  out = AddPart{p.y, p.parts, (long)p.part_stride, (long)p.row_stride, p.weight, p.post_w, p.post_b};
+}
 DeltaShape shape_of(const lsh_delta_shape_t& d) {
   return DeltaShape{d.heads, d.kv_heads, d.dim, d.vdim, d.taps};
 }
@@ -35,6 +45,13 @@ int64_t lsh_lm_delta_chunked_workspace(int rows, int n_seqs, const lsh_delta_sha
 }
 int lsh_lm_delta_chunked_supported(const lsh_delta_shape_t* sh) {
   return sh && delta_chunked_supported(shape_of(*sh)) ? 1 : 0;
+}
+
+int64_t lsh_lm_gla_chunked_workspace(int rows, int n_seqs, const lsh_gla_shape_t* sh) {
+  return sh ? (int64_t)gla_chunked_workspace(rows, n_seqs, shape_of(*sh)) : 0;
+}
+int lsh_lm_gla_chunked_supported(const lsh_gla_shape_t* sh, int64_t ld) {
+  return sh && gla_chunked_supported(shape_of(*sh), ld) ? 1 : 0;
 }
 
 int lsh_lm_moe_route(const float* logits, const float* bias, float* weight, int* count, int* list,
@@ -175,6 +192,58 @@ int lsh_lm_sample(const float* logits, int rows, int vocab, int topk, float topp
     return delta_step<T>((const T*)proj, ld, g_col, ba, conv_w, a_log, dt_bias, norm_w, eps,       \
                          (T*)conv_ring, state, (T*)out, row_slot, row_pos, rows, shape_of(*sh),    \
                          HS(s));                                                                   \
+  } \
+  int lsh_lm_gemm_epilogue_##SUF(const void* A, int64_t lda, const void* W, void* C, int64_t ldc,  \
+                                 float* C2, int64_t ld2, int n_split, int M, int N, int K,         \
+                                 float scale, const float* bias, lsh_stream_t s) {                 \
+    GemmEpilogue e;                                                                                \
+    e.scale = scale;                                                                               \
+    e.bias = bias;                                                                                 \
+    return gemm_float<T, T>((const T*)A, lda, (const T*)W, (T*)C, ldc, C2, ld2, n_split, M, N, K,  \
+                            HS(s), e);                                                             \
+  }                                                                                                \
+  int lsh_lm_gemm_gated_##SUF(const void* A, int64_t lda, const void* W, void* C, int64_t ldc,     \
+                              int M, int N, int K, int act, lsh_stream_t s) {                      \
+    return gemm_gated<T>((const T*)A, lda, (const T*)W, (T*)C, ldc, M, N, K, act, HS(s));          \
+  }                                                                                                \
+  int lsh_lm_residual_##SUF(float* x, const lsh_residual_t* what, void* h, int rows, int width,    \
+                            float eps, const int* ids, const void* embed, int vocab,               \
+                            lsh_stream_t s) {                                                      \
+    NEED(what);                                                                                    \
+    AddSpec add;                                                                                   \
+    part_of(what->part[0], add);                                                                   \
+    part_of(what->part[1], add.second);                                                            \
+    add.y_is_float = what->y_is_float != 0;                                                        \
+    add.scale = what->scale;                                                                       \
+    add.post_kind = what->post_rms ? kRmsNorm : kLayerNorm;                                        \
+    const NormSpec norm{what->norm_w, what->norm_b, what->norm_rms ? kRmsNorm : kLayerNorm};       \
+    const InjectSpec inject{what->inject_ids, what->inject_vec};                                   \
+    return lm_norm<T>(x, add, norm, (T*)h, rows, width, eps, ids, (const T*)embed, vocab, nullptr, \
+                      nullptr, 0, HS(s), inject);                                                  \
+  }                                                                                                \
+  int lsh_lm_gla_step_##SUF(const void* proj, int64_t ld, const float* low, const float* a2,       \
+                            const float* bias, const float* norm, float* state, void* out,         \
+                            const int* row_slot, const int* row_pos, int rows,                     \
+                            const lsh_gla_shape_t* sh, lsh_stream_t s) {                           \
+    NEED(sh);                                                                                      \
+    return gla_step<T>((const T*)proj, ld, low, GlaWeights{a2, bias, norm}, state, (T*)out,        \
+                       row_slot, row_pos, rows, shape_of(*sh), HS(s));                             \
+  }                                                                                                \
+  int lsh_lm_gla_scan_##SUF(const void* proj, int64_t ld, const float* low, const float* a2,       \
+                            const float* bias, const float* norm, float* state, void* out,         \
+                            const lsh_seq_span_t* seqs, int n_seqs, const lsh_gla_shape_t* sh,     \
+                            lsh_stream_t s) {                                                      \
+    NEED(sh);                                                                                      \
+    return gla_scan<T>((const T*)proj, ld, low, GlaWeights{a2, bias, norm}, state, (T*)out,        \
+                       spans(seqs), n_seqs, shape_of(*sh), HS(s));                                 \
+  }                                                                                                \
+  int lsh_lm_gla_chunked_##SUF(const void* proj, int64_t ld, const float* low, const float* a2,    \
+                               const float* bias, const float* norm, float* state, void* out,      \
+                               float* workspace, const lsh_seq_span_t* seqs, int n_seqs, int max_n,\
+                               int rows, const lsh_gla_shape_t* sh, lsh_stream_t s) {              \
+    NEED(sh);                                                                                      \
+    return gla_chunked<T>((const T*)proj, ld, low, GlaWeights{a2, bias, norm}, state, (T*)out,     \
+                          workspace, spans(seqs), n_seqs, max_n, rows, shape_of(*sh), HS(s));      \
   }
 
 LM_TYPED(f32, float)

@@ -414,3 +414,7 @@ class DecoderModel(LSModel):
 
 class Sudevik(DecoderModel):
     """Gated-delta and sliding-window-attention layers with mixtures of experts."""
+
+
+class Gebuzen(DecoderModel):
+    """Chunked attention and gated linear attention side by side, dense feed-forwards, looped layers."""

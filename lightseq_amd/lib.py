@@ -171,6 +171,8 @@ _LM_SIGNATURES = {
     "lsh_lm_attn_decode_workspace": (False, "ip"),
     "lsh_lm_delta_chunked_workspace": (False, "iip"),
     "lsh_lm_delta_chunked_supported": (False, "p"),
+    "lsh_lm_gla_chunked_workspace": (False, "iip"),
+    "lsh_lm_gla_chunked_supported": (False, "pl"),
     "lsh_lm_moe_route": (False, "ppppp" + "iii" + "s"),
     "lsh_lm_sample": (False, "p" + "iii" + "f" + "i" + "pp" + "i" + "pppp" + "s"),
     "lsh_lm_gemm": (True, "plpplpliiiis"),
@@ -188,8 +190,15 @@ _LM_SIGNATURES = {
     "lsh_lm_delta_chunked": (True, "pppppppppiiips"),
     "lsh_lm_delta_gated_norm": (True, "pplipfpips"),
     "lsh_lm_delta_step": (True, "plipppppfpppppips"),
+    "lsh_lm_gemm_epilogue": (True, "plpplpliiiifps"),
+    "lsh_lm_gemm_gated": (True, "plppliiiis"),
+    "lsh_lm_residual": (True, "pppiifppis"),
+    "lsh_lm_gla_step": (True, "plppppppppips"),
+    "lsh_lm_gla_scan": (True, "plpppppppips"),
+    "lsh_lm_gla_chunked": (True, "plppppppppiiips"),
 }
-_LM_RETURNS_COUNT = ("lsh_lm_attn_decode_workspace", "lsh_lm_delta_chunked_workspace")
+_LM_RETURNS_COUNT = ("lsh_lm_attn_decode_workspace", "lsh_lm_delta_chunked_workspace",
+                        "lsh_lm_gla_chunked_workspace")
 
 _lib = None
 

@@ -22,7 +22,8 @@ class AttnShape(ctypes.Structure):
 
 
 class AttnMask(ctypes.Structure):
-    _fields_ = [("window", I), ("keep_first", I), ("scale", ctypes.c_float), ("sink", I)]
+    _fields_ = [("window", I), ("keep_first", I), ("scale", ctypes.c_float), ("sink", I), ("chunk", I),
+                ("sinks", ctypes.c_void_p)]
 
 
 class DeltaShape(ctypes.Structure):
@@ -97,6 +98,40 @@ def test_gemm(dt, m, n, k, split):
     call("lsh_lm_gemm_planes_" + dt, dev(a, dt), k, dev(w, dt), p, m, n, k, 8, ctypes.addressof(planes))
     assert 1 <= planes.value <= 8 and (m > 64) <= (planes.value == 1)
     close(host(p.reshape(-1)[:planes.value * m * n].reshape(planes.value, m, n)).sum(0), want, "f32")
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("m,n,k,split", [(1, 40, 64, 40), (5, 33, 48, 20), (40, 64, 1024, 64), (130, 200, 128, 176),
+                                         (300, 50, 27, 44), (50, 16500, 64, 16487), (2100, 2080, 128, 2064)])
+def test_gemm_scale_and_bias(dt, m, n, k, split):
+    r = rng(m * n + k)
+    a, w = rounded(r.normal(size=(m, k)), dt), rounded(r.normal(size=(n, k)), dt)
+    bias = np.float32(r.normal(size=n) * 10).astype(np.float64)
+    ldc = (split + 7) // 8 * 8
+    for scale, b in ((0.3, bias), (1.0, bias), (2.5, None)):
+        want = scale * (a @ w.T) + (0 if b is None else b)
+        c = torch.zeros(m, ldc, dtype=TORCH[dt], device="cuda")
+        c2 = torch.zeros(m, max(n - split, 1), device="cuda")
+        call("lsh_lm_gemm_epilogue_" + dt, dev(a, dt), k, dev(w, dt), c, ldc, c2, n - split, split, m, n, k, scale,
+             None if b is None else dev(b))
+        close(host(c)[:, :split], want[:, :split], dt)
+        if split < n:
+            close(host(c2), want[:, split:], "f32", scale=np.abs(want).max())
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("m,n,k", [(1, 40, 64), (20, 33, 48), (33, 64, 1024), (64, 100, 72), (65, 128, 64), (130, 200, 128),
+                                   (300, 50, 27), (2100, 1040, 128), (2048, 2048, 64)])
+def test_gated_product(dt, m, n, k):
+    r = rng(m + n + k)
+    h, w = rounded(r.normal(size=(m, k)), dt), rounded(r.normal(size=(2, n, k)) / np.sqrt(k), dt)
+    g, u = h @ w[0].T, h @ w[1].T
+    ldc = n + 8
+    for act, f in ((0, O.silu), (1, lambda z: np.maximum(z, 0))):
+        c = torch.full((m, ldc), 7.0, dtype=TORCH[dt], device="cuda")
+        call("lsh_lm_gemm_gated_" + dt, dev(h, dt), k, dev(w, dt), c, ldc, m, n, k, act)
+        close(host(c)[:, :n], f(g) * u, dt)
+        assert (host(c)[:, n:] == 7).all()
 
 
 # -- routing and experts --------------------------------------------------------------------------
@@ -220,6 +255,56 @@ def test_norm(dt, width):
     close(host(h)[:3], O.layer_norm(table[ids][pick], w[1], b[1], eps), dt)
 
 
+class Part(ctypes.Structure):
+    _fields_ = [("y", ctypes.c_void_p), ("parts", I), ("part_stride", ctypes.c_int64), ("row_stride", ctypes.c_int64),
+                ("weight", ctypes.c_void_p), ("post_w", ctypes.c_void_p), ("post_b", ctypes.c_void_p)]
+
+
+class Residual(ctypes.Structure):
+    _fields_ = [("part", Part * 2), ("y_is_float", I), ("post_rms", I), ("norm_rms", I), ("scale", ctypes.c_float),
+                ("norm_w", ctypes.c_void_p), ("norm_b", ctypes.c_void_p), ("inject_ids", ctypes.c_void_p),
+                ("inject_vec", ctypes.c_void_p)]
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("width", [64, 75, 1024, 1030, 3000, 8192])
+def test_residual_with_two_summands(dt, width):
+    r = rng(width)
+    rows, eps, scale = 7, 1e-3, 0.35
+    f = lambda a: np.asarray(a, np.float32).astype(np.float64)  # noqa: E731
+    x = f(r.normal(size=(rows, width)) + 3)
+    w = [f(1 + 0.3 * r.normal(size=width)) for _ in range(3)]
+    table, ids = rounded(r.normal(size=(11, width)), dt), r.integers(0, 11, rows)
+    vec = f(r.normal(size=width))
+    if width % 4 and width > 4096:
+        return
+    dw, dtab, dids, dvec = [dev(v) for v in w], dev(table, dt), ints(ids), dev(vec)
+    h = torch.zeros(rows, width, dtype=TORCH[dt], device="cuda")
+    # planes of both, each normed by itself; then the embedding again, a vector, and the norm
+    y = [f(r.normal(size=(n, rows, width)) * s) for n, s in ((3, 1.0), (2, 30.0))]
+    dy, dx = [dev(v) for v in y], dev(x)
+    d = Residual(y_is_float=1, post_rms=1, norm_rms=1, scale=scale, norm_w=dw[2].data_ptr(),
+                 inject_ids=dids.data_ptr(), inject_vec=dvec.data_ptr())
+    for i in range(2):
+        d.part[i] = Part(dy[i].data_ptr(), len(y[i]), rows * width, width, None, dw[i].data_ptr(), None)
+    call("lsh_lm_residual_" + dt, dx, d, h, rows, width, eps, None, dtab, 11)
+    want = x + scale * sum(O.rms_norm(y[i].sum(0), w[i], eps) for i in range(2)) + table[ids] + vec
+    close(host(dx), want, "f32")
+    close(host(h), O.rms_norm(want, w[2], eps), dt)
+    # one summand in the activations' type, no norm of its own, no output
+    y1 = rounded(r.normal(size=(rows, width)), dt)
+    dy1, dx = dev(y1, dt), dev(x)
+    d = Residual(scale=scale)
+    d.part[0] = Part(dy1.data_ptr(), 1, 0, width, None, None, None)
+    call("lsh_lm_residual_" + dt, dx, d, None, rows, width, eps, None, None, 0)
+    close(host(dx), x + scale * y1, "f32")
+    # from the embedding, with the vector
+    d = Residual(norm_rms=1, scale=1.0, norm_w=dw[0].data_ptr(), inject_vec=dvec.data_ptr())
+    call("lsh_lm_residual_" + dt, dx, d, h, rows, width, eps, dids, dtab, 11)
+    close(host(dx), table[ids] + vec, "f32")
+    close(host(h), O.rms_norm(table[ids] + vec, w[0], eps), dt)
+
+
 # -- attention ------------------------------------------------------------------------------------
 def cos_sin(rot, n):
     f, m = O.rope_frequencies(rot)
@@ -268,17 +353,19 @@ def test_attn_prepare(dt, H, G, D, VD, rot):
     assert (host(kcache).transpose(0, 2, 1, 3)[~written] == 7).all()
 
 
-def attend_one(q, k, v, i, scale, window, keep, sink):
-    js = [j for j in range(i + 1) if window <= 0 or i - j < window or j < keep]
+def attend_one(q, k, v, i, scale, window, keep, sink, chunk=0, logit=0.0):
+    js = [j for j in range(i + 1) if j < keep or
+          ((window <= 0 or i - j < window) and (chunk <= 0 or i // chunk == j // chunk))]
     s = k[js] @ q * scale
-    m = max(s.max(), 0.0)
+    m = max(s.max(), logit)
     e = np.exp(s - m)
-    return (e / (e.sum() + (np.exp(-m) if sink else 0))) @ v[js]
+    return (e / (e.sum() + (np.exp(logit - m) if sink else 0))) @ v[js]
 
 
-def attention_case(dt, H, G, D, VD, spans, S, window, keep, sink=1, gate=True, seed=0, scale=None):
+def attention_case(dt, H, G, D, VD, spans, S, window, keep, sink=1, gate=True, seed=0, scale=None, chunk=0,
+                   sinks=None, same=False):
     """spans: (pos0, n) per sequence.  One key per query position is made to stand out: the oldest
-    kept one, the one just inside and the one just outside the window in turn."""
+    kept one, the one just inside and the one just outside the window (the chunk) in turn."""
     from lightseq_amd import lib
     r = rng(seed + D + window)
     scale = scale or 1.5 / np.sqrt(D)
@@ -301,17 +388,22 @@ def attention_case(dt, H, G, D, VD, spans, S, window, keep, sink=1, gate=True, s
         k, v = np.zeros((G, T, dp)), np.zeros((G, T, vp))
         k[..., :D] = r.normal(size=(G, T, D))
         v[..., :VD] = r.normal(size=(G, T, VD))
+        if same:
+            v = k
         for t in range(n):
             i = p0 + t
             for g in range(G):
                 far = [keep - 1, keep, i - window + 1, i - window, 0, i][(t + g) % 6]
+                if chunk:
+                    far = [i - i % chunk, i - i % chunk - 1, 0, i][(t // 3 + g) % 4]
                 if 0 <= far <= i and far < T and t % 3 == 0:
                     q[row + t, g * (H // G), :D] = rounded(3.0 * k[g, far, :D] / np.linalg.norm(k[g, far, :D])
                                                           / scale / 2, dt)
         k, v = rounded(k, dt), rounded(v, dt)
         keys.append((k, v))
         kc[sl, :, :T] = dev(k, dt)
-        vc[sl, :, :T] = dev(v, dt)
+        if not same:
+            vc[sl, :, :T] = dev(v, dt)
         meta.append((row, n, p0, sl))
         qpos += [(sl, p0 + t) for t in range(n)]
         row += n
@@ -319,12 +411,16 @@ def attention_case(dt, H, G, D, VD, spans, S, window, keep, sink=1, gate=True, s
         for t in range(n):
             for h in range(H):
                 g = h // (H // G)
-                want[r0 + t, h] = attend_one(q[r0 + t, h], k[g], v[g][:, :VD], p0 + t, scale, window, keep, sink)
+                want[r0 + t, h] = attend_one(q[r0 + t, h], k[g], v[g][:, :VD], p0 + t, scale, window, keep, sink, chunk,
+                                             sinks[h] if sinks is not None else 0.0)
     if gate:
         want *= O.sigmoid(proj[:, gc:gc + H * VD].reshape(rows, H, VD))
-    sh, mask = AttnShape(H, G, D, VD, S), AttnMask(window, keep, scale, sink)
+    sh, mask = AttnShape(H, G, D, VD, S), AttnMask(window, keep, scale, sink, chunk)
+    if sinks is not None:
+        mask.device_sinks = dev(sinks)  # lives as long as the mask
+        mask.sinks = mask.device_sinks.data_ptr()
     out = torch.zeros(rows, H * VD, dtype=TORCH[dt], device="cuda")
-    head = (dev(q, dt), kc, vc, dev(proj, dt), ld, gc if gate else -1, out)
+    head = (dev(q, dt), kc, kc if same else vc, dev(proj, dt), ld, gc if gate else -1, out)
     return head, sh, mask, meta, qpos, want.reshape(rows, -1), out
 
 
@@ -375,6 +471,84 @@ def test_attn_decode(dt, case):
             call("lsh_lm_attn_decode_" + dt, *head, ints([s for s, _ in qpos]), ints([p for _, p in qpos]), rows,
                  max_len, ws, sh, mask)
             close(host(out), want, dt)
+
+
+# chunks, a logit per sink, values that are the keys
+CHUNKED = [
+    # H, G, D, VD, spans, window, keep, chunk, same
+    (4, 2, 64, 64, [(0, 200)], 0, 0, 48, True), (2, 1, 96, 96, [(0, 1), (0, 130), (0, 64)], 0, 0, 64, True),
+    (3, 1, 20, 27, [(0, 70), (0, 3)], 0, 2, 7, False), (2, 2, 128, 128, [(37, 90), (100, 2), (0, 129)], 0, 0, 33, True),
+    (1, 1, 200, 256, [(5, 60)], 20, 0, 50, False), (2, 1, 33, 33, [(298, 5), (0, 300)], 0, 0, 1, True),
+    (6, 2, 64, 64, [(250, 64), (63, 65), (127, 2)], 0, 0, 128, True), (1, 1, 250, 250, [(0, 150)], 0, 3, 1000, True),
+    (2, 2, 96, 40, [(128, 128)], 65, 5, 100, False),
+]
+
+
+def sink_logits(H, case):
+    """Among them one that takes nearly everything and one that takes nearly nothing."""
+    z = rng(case).normal(size=H).astype(np.float32)
+    z[0] = [6.0, -40.0, 3.0][case % 3]
+    return z
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("case", range(len(CHUNKED)))
+def test_attn_prefill_chunked(dt, case):
+    H, G, D, VD, spans, window, keep, chunk, same = CHUNKED[case]
+    for sinks in (sink_logits(H, case), None):
+        head, sh, mask, meta, _, want, out = attention_case(dt, H, G, D, VD, spans, 320, window, keep, gate=case % 2 == 0,
+                                                            chunk=chunk, sinks=sinks, same=same)
+        call("lsh_lm_attn_prefill_" + dt, *head, ints(meta), len(meta), max(m[1] for m in meta), sh, mask)
+        close(host(out), want, dt)
+
+
+CHUNKED_DECODE = [
+    # H, G, D, VD, positions, window, keep, chunk, same
+    (4, 2, 64, 64, [0, 1, 39, 40, 41, 79, 80, 300], 0, 0, 40, True), (6, 1, 96, 96, [5, 299], 0, 0, 300, True),
+    (3, 1, 20, 27, [6, 7, 8, 13, 14, 200], 0, 2, 7, False), (9, 1, 128, 128, [318, 17], 0, 0, 100, True),
+    (2, 2, 256, 256, [0, 255, 256, 257], 0, 1, 256, True), (2, 1, 33, 33, [50], 0, 0, 1, True),
+    (16, 2, 128, 128, [2047, 100, 2048, 4095], 0, 0, 2048, True), (2, 1, 64, 96, [5000, 1100, 2303], 0, 0, 4000, False),
+    (1, 1, 96, 96, [3000, 2, 2999], 0, 7, 3000, True),
+]
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("case", range(len(CHUNKED_DECODE)))
+def test_attn_decode_chunked(dt, case):
+    from lightseq_amd import lib
+    H, G, D, VD, positions, window, keep, chunk, same = CHUNKED_DECODE[case]
+    S = max(positions) + 5
+    head, sh, mask, meta, qpos, want, out = attention_case(
+        dt, H, G, D, VD, [(p, 1) for p in positions], S, window, keep, gate=False, chunk=chunk,
+        sinks=sink_logits(H, case), same=same)
+    rows = len(positions)
+    ws = torch.empty(lib.load().lsh_lm_attn_decode_workspace(rows, ctypes.addressof(sh)), device="cuda")
+    call("lsh_lm_attn_decode_" + dt, *head, ints([s for s, _ in qpos]), ints([p for _, p in qpos]), rows, S, ws, sh,
+         mask)
+    close(host(out), want, dt)
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("H,G,D", [(4, 2, 64), (3, 1, 20), (2, 2, 129), (1, 1, 256)])
+def test_attn_prepare_without_norm_rotation_and_values(dt, H, G, D):
+    from lightseq_amd import lib
+    r = rng(D)
+    rows, S, slots = 9, 50, 3
+    qc, kc = 8, 8 + H * D
+    proj = rounded(r.normal(size=(rows, kc + G * D + 4)), dt)
+    slot, pos = r.integers(0, slots, rows), r.permutation(S)[:rows]
+    dp = lib.load().lsh_lm_attn_pad(D)
+    kcache = torch.full((slots, G, S, dp), 7.0, dtype=TORCH[dt], device="cuda")
+    q = torch.full((rows, H, dp), 7.0, dtype=TORCH[dt], device="cuda")
+    call("lsh_lm_attn_prepare_" + dt, dev(proj, dt), proj.shape[1], qc, kc, -1, None, None, 0.0, None, 0, q, kcache,
+         None, ints(slot), ints(pos), rows, AttnShape(H, G, D, D, S))
+    assert np.array_equal(host(q)[..., :D], proj[:, qc:qc + H * D].reshape(rows, H, D)) and not host(q)[..., D:].any()
+    got, written = host(kcache), np.zeros((slots, S), bool)
+    for i in range(rows):
+        assert np.array_equal(got[slot[i], :, pos[i], :D], proj[i, kc:kc + G * D].reshape(G, D))
+        assert not got[slot[i], :, pos[i], D:].any()
+    written[slot, pos] = True
+    assert (got.transpose(0, 2, 1, 3)[~written] == 7).all()
 
 
 # -- gated delta rule -----------------------------------------------------------------------------
