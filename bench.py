@@ -46,7 +46,8 @@ oracle on a few steps of the same width.  The default line carries both under ``
 ``--workload sudevik`` times the bfloat16 Sudevik decoder (``lightseq_amd.synthetic`` sizes) beside
 ``QuantGpt`` of the same width, depth, heads, vocabulary and active feed-forward size: prompt tokens/s
 and decode-step time of each, from HIP events on the model's stream around the prompt pass and the step
-loop of whole ``Infer()`` calls.
+loop of whole ``Infer()`` calls.  ``--workload gebuzen`` times the Gebuzen decoder beside Sudevik in the
+same way.
 """
 import argparse
 import json
@@ -758,8 +759,8 @@ def bench_generation(workload, steps, warmup, graphs=False, with_cpu=True):
     return out
 
 
-# (batch, prompt, generated tokens) of the Sudevik comparison: a long prompt batch, a decoding batch
-SUDEVIK_SHAPES = [(8, 1024, 32), (32, 256, 64)]
+# (batch, prompt, generated tokens) of the decoder comparisons: a long prompt batch, a decoding batch
+DECODER_SHAPES = [(8, 1024, 32), (32, 256, 64)]
 
 
 def _sudevik_work(cfg, batch, prompt, new):
@@ -813,63 +814,98 @@ def _time_decoder(model, batch, prompt, new, upload, steps, warmup):
             "launches_per_step": launches}
 
 
-def bench_sudevik(args):
+def _gebuzen_work(cfg, batch, prompt, new):
+    """The same for the Gebuzen decoder; the layers of its loop count once per pass."""
+    W, V = cfg["width"], cfg["vocab"]
+    loop = cfg["loop"]
+    times = [loop["times"] if loop["start"] <= i < loop["stop"] else 1 for i in range(len(cfg["layers"]))]
+    macs = nbytes = 0.0
+    for l, n in zip(cfg["layers"], times):
+        a, r, ff = l["mixer"]["left"], l["mixer"]["right"], l["mlp"]["ff"]
+        H, G, D, chunk = a["heads"], a["kv_heads"], a["dim"], a["mask"]["size"]
+        C, VC, rank = r["heads"] * r["dim"], r["heads"] * r["vdim"], 16
+        weights = W * (2 * H * D + G * D + 2 * C + 3 * VC + rank + 3 * ff) + rank * C
+        seen = sum(i % chunk + 1 for i in range(prompt)) / prompt
+        at = [(prompt + i) % chunk + 1 for i in range(new)]
+        macs += n * (weights + 2 * H * D * seen + 2 * C * r["vdim"])
+        nbytes += n * (2 * weights + 2 * batch * G * D * sum(at) / new + 8 * batch * C * r["vdim"])
+    return 2 * macs * batch * prompt, nbytes + 2 * W * V + 4 * batch * V
+
+
+def _bench_folder(folder, work, cfg, ids, new, args):
+    """Times the decoder model in a folder; fractions of the matrix and of the memory peak."""
+    from lightseq_amd import inference
+    batch, prompt = ids.shape
+    m = inference.DecoderModel(folder, max_batch_size=batch, max_step=prompt + new, extra_decode_length=new)
+
+    def upload():
+        m.benchmark_mode(True)
+        m.infer(ids)
+    r = _time_decoder(m, batch, prompt, new, upload, args.steps, args.warmup)
+    m.close()
+    flop, nbytes = work(cfg, batch, prompt, new)
+    r["prompt_tflops"] = flop / (r["prompt_ms"] * 1e-3) / 1e12
+    r["prompt_frac_of_2500_tflops"] = r["prompt_tflops"] / 2500
+    r["decode_gbs"] = nbytes / (r["ms_per_decode_step"] * 1e-3) / 1e9
+    r["decode_frac_of_hbm"] = r["decode_gbs"] / HBM_PEAK_GBS
+    return r
+
+
+def _bench_gpt(folder, cfg, ids, new, args):
+    """The int8 GPT with the width, depth, heads, vocabulary and active feed-forward weights of a Sudevik."""
+    from lightseq_amd import inference, synthetic
+    batch, prompt = ids.shape
+    L, W, V = len(cfg["layers"]), cfg["width"], cfg["vocab"]
+    mlp = cfg["layers"][0]["mlp"]
+    inner = 3 * mlp["router"]["top"] * mlp["expert"]["ff"] // 2
+    g = dict(n_layer=L, hidden=W, inner=inner, head_num=cfg["layers"][0]["mixer"]["heads"], max_step=prompt + new,
+             vocab=V, padding_id=V - 1, eos_id=V - 1, topk=1, extra_decode_length=new, sampling_method="topk")
+    path = os.path.join(folder, "gpt.pb")
+    synthetic.write_quant_gpt(path, g, seed=0)
+    m = inference.QuantGpt(path, batch)
+    os.remove(path)
+    r = _time_decoder(m, batch, prompt, new, lambda: m._upload(ids), args.steps, args.warmup)
+    m.close()
+    per_tok = L * (4 * W * W + 2 * W * inner + 2 * W * (prompt + 1) / 2)
+    r["prompt_tops"] = 2 * per_tok * batch * prompt / (r["prompt_ms"] * 1e-3) / 1e12
+    r["prompt_frac_of_5000_tops"] = r["prompt_tops"] / INT8_MFMA_PEAK_TOPS
+    nbytes = L * (4 * W * W + 2 * W * inner) + V * W + L * batch * 2 * W * (prompt + new / 2) + 2 * batch * V
+    r["decode_gbs"] = nbytes / (r["ms_per_decode_step"] * 1e-3) / 1e9
+    r["decode_frac_of_hbm"] = r["decode_gbs"] / HBM_PEAK_GBS
+    return r
+
+
+def bench_decoder(args):
+    """A decoder model in a folder beside the closest other model of equal size: Sudevik beside QuantGpt,
+    Gebuzen beside Sudevik."""
     import shutil
     import numpy as np
-    from lightseq_amd import inference, synthetic
-    out = {"metric": "decoder throughput beside QuantGpt", "dtype": "bf16 (QuantGpt: int8)", "data": "synthetic",
+    from lightseq_amd import synthetic
+    names = {"sudevik": ("sudevik", "gpt"), "gebuzen": ("gebuzen", "sudevik")}[args.workload]
+    configs = {"sudevik": (synthetic.sudevik_config, _sudevik_work), "gebuzen": (synthetic.gebuzen_config, _gebuzen_work)}
+    out = {"metric": "decoder throughput, %s beside %s" % names, "dtype": "bf16 (gpt: int8)", "data": "synthetic",
            "n_gpus": 1, "steps": args.steps, "warmup": args.warmup, "results": []}
     rng = np.random.default_rng(0)
     for size in args.sizes.split(","):
-        cfg = synthetic.sudevik_config(size)
-        L, W, V = len(cfg["layers"]), cfg["width"], cfg["vocab"]
-        H = cfg["layers"][0]["mixer"]["heads"]
-        mlp = cfg["layers"][0]["mlp"]
-        inner = 3 * mlp["router"]["top"] * mlp["expert"]["ff"] // 2  # the same active weights
-        folder = tempfile.mkdtemp(prefix="ls_bench_")
-        try:
-            if args.only != "gpt":
-                synthetic.write_sudevik(folder, cfg)
-            for batch, prompt, new in SUDEVIK_SHAPES:
-                res = {"size": size, "layers": L, "width": W, "heads": H, "vocab": V, "active_ffn": inner,
-                       "batch": batch, "prompt": prompt, "new": new}
-                ids = rng.integers(0, V - 1, size=(batch, prompt), dtype=np.int32)
-                if args.only != "gpt":
-                    m = inference.DecoderModel(folder, max_batch_size=batch, max_step=prompt + new,
-                                               extra_decode_length=new)
-
-                    def upload():
-                        m.benchmark_mode(True)
-                        m.infer(ids)
-                    r = _time_decoder(m, batch, prompt, new, upload, args.steps, args.warmup)
-                    m.close()
-                    flop, nbytes = _sudevik_work(cfg, batch, prompt, new)
-                    r["prompt_tflops"] = flop / (r["prompt_ms"] * 1e-3) / 1e12
-                    r["prompt_frac_of_2500_tflops"] = r["prompt_tflops"] / 2500
-                    r["decode_gbs"] = nbytes / (r["ms_per_decode_step"] * 1e-3) / 1e9
-                    r["decode_frac_of_hbm"] = r["decode_gbs"] / HBM_PEAK_GBS
-                    res["sudevik"] = r
-                if args.only != "sudevik":
-                    g = dict(n_layer=L, hidden=W, inner=inner, head_num=H, max_step=prompt + new, vocab=V,
-                             padding_id=V - 1, eos_id=V - 1, topk=1, extra_decode_length=new, sampling_method="topk")
-                    path = os.path.join(folder, "gpt.pb")
-                    synthetic.write_quant_gpt(path, g, seed=0)
-                    m = inference.QuantGpt(path, batch)
-                    os.remove(path)
-                    r = _time_decoder(m, batch, prompt, new, lambda: m._upload(ids), args.steps, args.warmup)
-                    m.close()
-                    per_tok = L * (4 * W * W + 2 * W * inner + 2 * W * (prompt + 1) / 2)
-                    r["prompt_tops"] = 2 * per_tok * batch * prompt / (r["prompt_ms"] * 1e-3) / 1e12
-                    r["prompt_frac_of_5000_tops"] = r["prompt_tops"] / INT8_MFMA_PEAK_TOPS
-                    nbytes = L * (4 * W * W + 2 * W * inner) + V * W + L * batch * 2 * W * (prompt + new / 2) \
-                        + 2 * batch * V
-                    r["decode_gbs"] = nbytes / (r["ms_per_decode_step"] * 1e-3) / 1e9
-                    r["decode_frac_of_hbm"] = r["decode_gbs"] / HBM_PEAK_GBS
-                    res["quant_gpt"] = r
-                out["results"].append(res)
-                print(json.dumps(res), file=sys.stderr, flush=True)
-        finally:
-            shutil.rmtree(folder, ignore_errors=True)
+        results = [{"size": size, "batch": b, "prompt": p, "new": n} for b, p, n in DECODER_SHAPES]
+        for name in names:
+            if args.only not in ("", name):
+                continue
+            folder = tempfile.mkdtemp(prefix="ls_bench_")
+            try:
+                cfg = configs[name if name in configs else "sudevik"][0](size)
+                if name in configs:
+                    synthetic.write_decoder(folder, cfg)
+                for res in results:
+                    ids = rng.integers(0, cfg["vocab"] - 1, size=(res["batch"], res["prompt"]), dtype=np.int32)
+                    if name in configs:
+                        res[name] = _bench_folder(folder, configs[name][1], cfg, ids, res["new"], args)
+                    else:
+                        res[name] = _bench_gpt(folder, cfg, ids, res["new"], args)
+                    print(json.dumps(res), file=sys.stderr, flush=True)
+            finally:
+                shutil.rmtree(folder, ignore_errors=True)
+        out["results"] += results
     return out
 
 
@@ -890,7 +926,7 @@ def main():
     ap.add_argument("--steps", type=int, default=None)
     ap.add_argument("--warmup", type=int, default=None)
     ap.add_argument("--workload", default="bert_base",
-                    choices=["bert_base", "transformer_big", "gpt2_medium", "sudevik"])
+                    choices=["bert_base", "transformer_big", "gpt2_medium", "sudevik", "gebuzen"])
     ap.add_argument("--no-cpu-baseline", action="store_true")
     ap.add_argument("--no-fused", action="store_true",
                     help="skip the stand-alone timing of the fused kernels")
@@ -898,8 +934,8 @@ def main():
                     help="default workload: skip the two generation workloads of the `generation` block")
     ap.add_argument("--ffn-segment", action="store_true",
                     help="A/B and phase stamps of the one-launch feed-forward segment (not the headline line)")
-    ap.add_argument("--only", default="", help="sudevik workload: one of sudevik, gpt (for a profiler run)")
-    ap.add_argument("--sizes", default="base,large", help="sudevik workload: configurations to time")
+    ap.add_argument("--only", default="", help="decoder workloads: one of the two models (for a profiler run)")
+    ap.add_argument("--sizes", default="base,large", help="decoder workloads: configurations to time")
     ap.add_argument("--graphs", action="store_true",
                     help="generation workloads: replay the steps as HIP graphs (ls_model_set_graph_mode)")
     ap.add_argument("--copy-calibration", action="store_true",
@@ -930,8 +966,8 @@ def main():
         print(json.dumps(bench_ffn_segment(args)))
         _leave()
         return
-    if args.workload == "sudevik":
-        print(json.dumps(bench_sudevik(args)))
+    if args.workload in ("sudevik", "gebuzen"):
+        print(json.dumps(bench_decoder(args)))
         _leave()
         return
     out = bench_bert(args) if bert else bench_generation(args.workload, args.steps, args.warmup,

@@ -394,14 +394,64 @@ def sudevik_shapes(cfg):
     return t
 
 
-def write_sudevik(folder, cfg, seed=0):
+def gebuzen_config(name):
+    """Shapes of the named synthetic Gebuzen decoders; as many layer runs, heads and active feed-forward
+    weights as the Sudevik decoder of that name has."""
+    def layer(heads, kv_heads, dim, chunk, ff):
+        return {"type": "parallel", "mlp": {"kind": "dense", "ff": ff}, "mixer": {
+            "left": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5,
+                     "mask": {"size": chunk}},
+            "right": {"heads": heads, "dim": dim, "vdim": dim, "tau": 16.0}}}
+    cfgs = {
+        "base": dict(vocab=32000, width=1024, layers=[layer(16, 4, 64, 512, 2048)] * 8,
+                     loop={"start": 2, "stop": 6, "times": 2}),
+        "large": dict(vocab=32000, width=2048, layers=[layer(16, 4, 128, 1024, 4096)] * 4,
+                      loop={"start": 1, "stop": 3, "times": 2}),
+    }
+    return dict(cfgs[name], architecture="Gebuzen", norm={"eps": 1e-6}, residual_mult=0.7, logit_scale=0.5)
+
+
+def gebuzen_shapes(cfg, rank=16):
+    """name -> shape of every tensor of a Gebuzen model."""
+    W, V, t = cfg["width"], cfg["vocab"], {}
+    t["embed"] = t["head"] = (V, W)
+    t["final.norm"] = (W,)
+    if cfg.get("loop"):
+        t["loop.step"] = (cfg["loop"]["times"], W)
+    for i, l in enumerate(cfg["layers"]):
+        p, a, b = "l%d." % i, l["mixer"]["left"], l["mixer"]["right"]
+        t[p + "norm1"] = (W,)
+        m = p + "mix.left."
+        for n, rows in (("q", a["heads"] * a["dim"]), ("k", a["kv_heads"] * a["dim"])):
+            t[m + n], t[m + n + ".b"] = (rows, W), (rows,)
+        t[m + "sink"], t[m + "o"], t[m + "out"] = (a["heads"],), (W, a["heads"] * a["dim"]), (W,)
+        m = p + "mix.right."
+        C, VC = b["heads"] * b["dim"], b["heads"] * b["vdim"]
+        for n, rows in (("q", C), ("k", C), ("v", VC), ("g", VC), ("a1", rank)):
+            t[m + n] = (rows, W)
+        t[m + "a2"], t[m + "a2.b"] = (C, rank), (C,)
+        t[m + "norm"], t[m + "o"], t[m + "out"] = (b["vdim"],), (W, VC), (W,)
+        if l.get("mlp"):
+            ff = l["mlp"]["ff"]
+            t[p + "norm2"] = (W,)
+            t[p + "mlp.gate"] = t[p + "mlp.up"] = (ff, W)
+            t[p + "mlp.down"] = (W, ff)
+    return t
+
+
+def write_decoder(folder, cfg, seed=0):
+    """A folder with random weights for a configuration of this module, by its architecture."""
+    shapes = {"Sudevik": sudevik_shapes, "Gebuzen": gebuzen_shapes}[cfg["architecture"]](cfg)
+    return _write_folder(folder, cfg, shapes, seed)
+
+
+def _write_folder(folder, cfg, shapes, seed):
     """Random weights ~N(0, 1 / inputs) (norm weights 1, biases 0), bfloat16.  Large matrices are cut
     from one pool of random numbers, scaled by powers of two in their exponents."""
     import json
     import os
     rng = np.random.default_rng(seed)
     pool = (rng.standard_normal(1 << 22, dtype=np.float32).view(np.uint32) >> 16).astype(np.uint16)
-    shapes = sudevik_shapes(cfg)
     os.makedirs(folder, exist_ok=True)
     with open(os.path.join(folder, "config.json"), "w") as f:
         json.dump(cfg, f)
@@ -417,7 +467,7 @@ def write_sudevik(folder, cfg, seed=0):
         for name, s in shapes.items():
             n = int(np.prod(s))
             if len(s) == 1:
-                one = name.endswith("norm") or name[:-1].endswith("norm1") or ".norm" in name
+                one = name.endswith(("norm", ".out")) or name[:-1].endswith("norm1") or ".norm" in name
                 v = 0x3f80 if one and not name.endswith(".b") else 0
                 if name.endswith("A_log"):
                     v = 0xbf80
