@@ -254,7 +254,21 @@ gemm_tile_kernel(GemmArgs a, int tiles_m, int tiles_n) {
 #pragma unroll
         for (int k = 0; k < 16; ++k) {
           if constexpr (is_up(MODE)) v[k] = gated(a, acc[i][0][k], acc[i][1][k]);
-          else v[k] = finish<MODE>(a, min(n + k, a.N - 1), acc[i][j][k]);
+          else v[k] = acc[i][j][k] * (MODE == kDense ? a.epi.scale : 1.f);
+        }
+        if (MODE == kDense && a.epi.bias) {
+          if (n + 16 <= a.N) {
+#pragma unroll
+            for (int k = 0; k < 16; k += 4) {
+              const f32x4 b = *reinterpret_cast<const f32x4*>(a.epi.bias + n + k);
+#pragma unroll
+              for (int e = 0; e < 4; ++e) v[k + e] += b[e];
+            }
+          } else {
+#pragma unroll
+            for (int k = 0; k < 16; ++k)
+              if (n + k < a.N) v[k] += a.epi.bias[n + k];
+          }
         }
         if (n + 16 <= min(a.N, a.n_split) && a.ldc % 8 == 0) {
           TO* p = reinterpret_cast<TO*>(a.C) + m * a.ldc + n;
@@ -462,7 +476,7 @@ bool tile_ok(const GemmArgs& a, int mode) {
   const long arows = mode == kMoeDown ? (long)a.M * a.top : a.M;
   return rows_aligned<T>(a) && (long)a.K * sizeof(T) % kBK == 0 &&
          wrows * a.K * (long)sizeof(T) < (1L << 32) && arows * a.lda * (long)sizeof(T) < (1L << 32) &&
-         (reinterpret_cast<uintptr_t>(a.C) & 15u) == 0;
+         ((reinterpret_cast<uintptr_t>(a.C) | reinterpret_cast<uintptr_t>(a.epi.bias)) & 15u) == 0;
 }
 
 template <typename T, typename TO, int MODE>

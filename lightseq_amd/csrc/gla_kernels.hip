@@ -28,17 +28,31 @@ namespace {
 
 constexpr int kC = 64;
 
-__device__ __forceinline__ float log_decay(float z, float inv_tau) { return -softplus_f(-z) * inv_tau; }
+__device__ __forceinline__ float exp2_f(float x) { return __builtin_amdgcn_exp2f(x); }
+// log2 of sigmoid(z)^(1 / tau) = -(max(-z, 0) log2(e) + log2(1 + u)) / tau with u = e^-|z|.  The sum 1 + u
+// loses the low bits of a small u; scaling its logarithm by u / ((1 + u) - 1) puts them back.
+__device__ __forceinline__ float log2_decay(float z, float inv_tau) {
+  constexpr float kLog2e = 1.44269504088896340736f;
+  const float u = exp2_f(-fabsf(z) * kLog2e), w = 1.f + u, d = w - 1.f;
+  const float l = d == 0.f ? u * kLog2e : __builtin_amdgcn_logf(w) * (u * __builtin_amdgcn_rcpf(d));
+  return -(fmaxf(-z, 0.f) * kLog2e + l) * inv_tau;
+}
 
-// a lane's value from N lanes before (after) it in its row of 16, zero at the border
+// a lane's value from N lanes before (after) it in its row of 16, zero at the border (a form that the
+// compiler folds into the operation that uses it)
+template <int CTRL>
+__device__ __forceinline__ float row_shift(float x) {
+  return __builtin_bit_cast(
+      float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, x), CTRL, 0xf, 0xf, true));
+}
 template <int N>
 __device__ __forceinline__ float lanes_before(float x) {
   if constexpr (N == 0) return x;
-  else return dpp_f<0x110 + N>(x);
+  else return row_shift<0x110 + N>(x);
 }
 template <int N>
 __device__ __forceinline__ float lanes_after(float x) {
-  return dpp_f<0x100 + N>(x);
+  return row_shift<0x100 + N>(x);
 }
 
 template <typename T>
@@ -49,8 +63,8 @@ __device__ __forceinline__ f32x4 load4(const T* p) {
 }
 __device__ __forceinline__ frag_t as_frag(f32x4 x) { return __builtin_bit_cast(frag_t, x); }
 __device__ __forceinline__ frag_t ldfrag(const float* p) { return *reinterpret_cast<const frag_t*>(p); }
-__device__ __forceinline__ f32x4 exp4(f32x4 x) {
-  return f32x4{expf(x[0]), expf(x[1]), expf(x[2]), expf(x[3])};
+__device__ __forceinline__ f32x4 exp4(f32x4 x) {  // 2^x
+  return f32x4{exp2_f(x[0]), exp2_f(x[1]), exp2_f(x[2]), exp2_f(x[3])};
 }
 
 // ------------------------------------------------------------------------------------------------
@@ -100,7 +114,7 @@ gla_scan_kernel(const T* __restrict__ proj, long ld, const float* __restrict__ l
 #pragma unroll
           for (int e = 0; e < 4; ++e) z = fmaf(a[e], b[e], z);
         }
-        as[x] = expf(log_decay(z, sh.inv_tau));
+        as[x] = exp2_f(log2_decay(z, sh.inv_tau));
       } else if (x < 2 * D) {
         qs[x - D] = to_f(pr[sh.q_col + h * D + x - D]) * qscale;
       } else if (x < 3 * D) {
@@ -166,12 +180,12 @@ __host__ __device__ inline long chunk_floats(const GlaShape& sh) {
   return (long)sh.vdim * sh.dim + sh.dim;
 }
 
-// log decays of this lane's token and channels; 0 for a token that is not there
+// log2 decays of this lane's token and channels from slice s0 on; 0 for a token that is not there
 template <int NS>
 __device__ __forceinline__ void chunk_log_decays(const float* __restrict__ low, long row, bool in,
-                                                 const GlaWeights& wt, const GlaShape& sh, int h,
+                                                 const GlaWeights& wt, const GlaShape& sh, int h, int s0,
                                                  int c, int qd, f32x4 (&la)[NS]) {
-  const int ns = sh.dim / 16;
+  const int ns = sh.dim / 16 - s0;
 #pragma unroll
   for (int s = 0; s < NS; ++s) la[s] = (f32x4)0.f;
   for (int r = 0; r < sh.rank; r += 16) {
@@ -179,15 +193,15 @@ __device__ __forceinline__ void chunk_log_decays(const float* __restrict__ low, 
 #pragma unroll
     for (int s = 0; s < NS; ++s)
       if (s < ns)
-        la[s] = mma16(0.f, ldfrag(wt.a2 + (long)(h * sh.dim + s * 16 + c) * sh.rank + r + qd * 4), fl,
+        la[s] = mma16(0.f, ldfrag(wt.a2 + (long)(h * sh.dim + (s0 + s) * 16 + c) * sh.rank + r + qd * 4), fl,
                       la[s]);
   }
 #pragma unroll
   for (int s = 0; s < NS; ++s)
     if (s < ns) {
-      const f32x4 b = load4(wt.bias + h * sh.dim + s * 16 + qd * 4);
+      const f32x4 b = load4(wt.bias + h * sh.dim + (s0 + s) * 16 + qd * 4);
 #pragma unroll
-      for (int e = 0; e < 4; ++e) la[s][e] = in ? log_decay(la[s][e] + b[e], sh.inv_tau) : 0.f;
+      for (int e = 0; e < 4; ++e) la[s][e] = in ? log2_decay(la[s][e] + b[e], sh.inv_tau) : 0.f;
     }
 }
 // sums over the tokens of the sub-block up to this one / after this one
@@ -251,7 +265,7 @@ gla_chunk_add_kernel(const T* __restrict__ proj, long ld, const float* __restric
   for (int s = 0; s < NS; ++s)
     k[s] = s < ns && in ? load4(proj + row * ld + sh.k_col + h * D + s * 16 + qd * 4) : (f32x4)0.f;
   stage_values(proj, ld, row0, n, sh, h, Vt);
-  chunk_log_decays<NS>(low, row, in, wt, sh, h, c, qd, la);
+  chunk_log_decays<NS>(low, row, in, wt, sh, h, 0, c, qd, la);
 #pragma unroll
   for (int s = 0; s < NS; ++s)
     if (s < ns) {
@@ -271,7 +285,7 @@ gla_chunk_add_kernel(const T* __restrict__ proj, long ld, const float* __restric
     }
   float* o = ws + ((sq.row0 / kC + (long)blockIdx.z + blockIdx.x) * H + h) * chunk_floats(sh);
   for (int d = tid; d < D; d += 256)
-    o[(long)VD * D + d] = expf((tot[d] + tot[D + d]) + (tot[2 * D + d] + tot[3 * D + d]));
+    o[(long)VD * D + d] = exp2_f((tot[d] + tot[D + d]) + (tot[2 * D + d] + tot[3 * D + d]));
   __syncthreads();
   for (int x = w; x < ns * nv; x += 4) {
     const int db = x % ns, vb = x / ns;
@@ -317,36 +331,32 @@ gla_chunk_state_kernel(float* __restrict__ ws, float* __restrict__ state,
   *reinterpret_cast<f32x4*>(sp) = S;
 }
 
-// products inside a sub-block: p[t][t - DELTA] for rising DELTA; w carries q_t times the decays of the
-// DELTA tokens up to t
-template <int NS, int DELTA>
-__device__ __forceinline__ void diagonal(const f32x4 (&k)[NS], const f32x4 (&a)[NS], f32x4 (&w)[NS],
-                                         int ns, int c, int qd, f32x4& p) {
+// products inside a sub-block, x[DELTA] of p[t][t - DELTA] for rising DELTA; w carries q_t times the
+// decays of the DELTA tokens up to t
+template <int N, int DELTA>
+__device__ __forceinline__ void diagonal(const f32x4 (&k)[N], const f32x4 (&a)[N], f32x4 (&w)[N],
+                                         float (&x)[16]) {
   if constexpr (DELTA < 16) {
-    float x = 0.f;
 #pragma unroll
-    for (int s = 0; s < NS; ++s)
-      if (s < ns) {
+    for (int s = 0; s < N; ++s)
 #pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          x = fmaf(w[s][e], lanes_before<DELTA>(k[s][e]), x);
-          w[s][e] *= lanes_before<DELTA>(a[s][e]);
-        }
+      for (int e = 0; e < 4; ++e) {
+        x[DELTA] = fmaf(w[s][e], lanes_before<DELTA>(k[s][e]), x[DELTA]);
+        if (DELTA < 15) w[s][e] *= lanes_before<DELTA>(a[s][e]);
       }
-    x += __shfl_xor(x, 16);
-    x += __shfl_xor(x, 32);
-#pragma unroll
-    for (int e = 0; e < 4; ++e) p[e] = c - DELTA == 4 * qd + e ? x : p[e];
-    diagonal<NS, DELTA + 1>(k, a, w, ns, c, qd, p);
+    diagonal<N, DELTA + 1>(k, a, w, x);
   }
 }
 
-// outputs of a chunk, normed and gated
+// Outputs of a chunk, normed and gated.  First every wavefront forms the weights of its 16 tokens, then
+// it takes value blocks w, w + 4, .. of all 64, so that state and values are read once.
 template <typename T, int NS>  // dim, vdim <= 16 * NS
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(256, NS <= 4 ? 3 : NS <= 8 ? 2 : 1)
 gla_chunk_out_kernel(const T* __restrict__ proj, long ld, const float* __restrict__ low, GlaWeights wt,
                      const float* __restrict__ ws, T* __restrict__ out,
                      const SeqSpan* __restrict__ seqs, GlaShape sh) {
+  constexpr int GS = NS < 4 ? NS : 4;  // slices whose keys and decays are in registers at a time
+  constexpr int NVB = (NS + 3) / 4;    // value blocks of a wavefront
   extern __shared__ __attribute__((aligned(16))) float sm[];
   const SeqSpan sq = seqs[blockIdx.z];
   const int c0 = blockIdx.x * kC;
@@ -354,91 +364,140 @@ gla_chunk_out_kernel(const T* __restrict__ proj, long ld, const float* __restric
   const int n = min(kC, sq.n - c0), h = blockIdx.y, H = sh.heads, D = sh.dim, VD = sh.vdim;
   const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, c = lane & 15, qd = lane >> 4;
   const int ns = D / 16, nv = VD / 16, KS = D + 4;
-  float* Kh = sm;                // [48][KS]: keys decayed to the end of their sub-block
-  float* Et = Kh + 48 * KS;      // [4][D]: decay of every sub-block
-  float* Vt = Et + 4 * D;        // [VD][kTS]
+  float* Q = sm;                 // [64][KS]: queries with their decays back to a block's end
+  float* Kh = Q + kC * KS;       // [48][KS]: keys decayed to the end of their sub-block
+  float* P = Kh + 48 * KS;       // [64][kTS]: weights of the chunk's tokens (lower blocks)
+  float* Et = P + kC * kTS;      // [4][D]: decay of every sub-block
+  float* sq_sum = Et + 4 * D;    // [4][64]
   const long row0 = sq.row0 + c0;
   const int t = w * 16 + c;
   const bool in = t < n;
   const long row = row0 + min(t, n - 1);
   const T* pr = proj + row * ld;
-  f32x4 q[NS], p = (f32x4)0.f;
+  const bool has_state = c0 > 0 || sq.pos0 > 0;
   {
-    f32x4 k[NS], la[NS], wq[NS];
     const float qscale = 1.0f / sqrtf((float)D);
+    float x[16];
 #pragma unroll
-    for (int s = 0; s < NS; ++s) {
-      k[s] = s < ns && in ? load4(pr + sh.k_col + h * D + s * 16 + qd * 4) : (f32x4)0.f;
-      q[s] = s < ns && in ? load4(pr + sh.q_col + h * D + s * 16 + qd * 4) * qscale : (f32x4)0.f;
-      wq[s] = q[s];
-    }
-    stage_values(proj, ld, row0, n, sh, h, Vt);
-    chunk_log_decays<NS>(low, row, in, wt, sh, h, c, qd, la);
+    for (int i = 0; i < 16; ++i) x[i] = 0.f;
+#pragma unroll 1
+    for (int s0 = 0; s0 < ns; s0 += GS) {
+      f32x4 k[GS], la[GS], wq[GS];
 #pragma unroll
-    for (int s = 0; s < NS; ++s)
-      if (s < ns) {
-        const f32x4 upto = exp4(sum_upto(la[s]));
-        if (c == 15) *reinterpret_cast<f32x4*>(&Et[w * D + s * 16 + qd * 4]) = upto;
-        if (w < 3)
-          *reinterpret_cast<f32x4*>(&Kh[t * KS + s * 16 + qd * 4]) = k[s] * exp4(sum_after(la[s]));
-        q[s] *= upto;
-        la[s] = exp4(la[s]);
+      for (int s = 0; s < GS; ++s) {
+        const int d = h * D + (s0 + s) * 16 + qd * 4;
+        const bool there = s0 + s < ns && in;
+        k[s] = there ? load4(pr + sh.k_col + d) : (f32x4)0.f;
+        wq[s] = there ? load4(pr + sh.q_col + d) * qscale : (f32x4)0.f;
       }
-    diagonal<NS, 0>(k, la, wq, ns, c, qd, p);
+      chunk_log_decays<GS>(low, row, in, wt, sh, h, s0, c, qd, la);
+#pragma unroll
+      for (int s = 0; s < GS; ++s)
+        if (s0 + s < ns) {
+          const int d = (s0 + s) * 16 + qd * 4;
+          const f32x4 upto = exp4(sum_upto(la[s]));
+          if (c == 15) *reinterpret_cast<f32x4*>(&Et[w * D + d]) = upto;
+          if (w < 3) *reinterpret_cast<f32x4*>(&Kh[t * KS + d]) = k[s] * exp4(sum_after(la[s]));
+          *reinterpret_cast<f32x4*>(&Q[t * KS + d]) = wq[s] * upto;
+          la[s] = exp4(la[s]);
+        }
+      diagonal<GS, 0>(k, la, wq, x);
+    }
+    f32x4 p = (f32x4)0.f;
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      x[i] += __shfl_xor(x[i], 16);
+      x[i] += __shfl_xor(x[i], 32);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) p[e] = c - i == 4 * qd + e ? x[i] : p[e];
+    }
+    *reinterpret_cast<f32x4*>(&P[t * kTS + w * 16 + qd * 4]) = p;
   }
   __syncthreads();
-  // transposed outputs: acc[vb] has the value channels 16 vb + 4 qd .. + 3 of token c
-  f32x4 acc[NS];
-#pragma unroll
-  for (int vb = 0; vb < NS; ++vb) {
-    acc[vb] = (f32x4)0.f;
-    if (vb < nv) acc[vb] = mma16(0.f, ldfrag(&Vt[(vb * 16 + c) * kTS + w * 16 + qd * 4]), as_frag(p), acc[vb]);
-  }
-  // earlier sub-blocks; q is decayed further back with every one passed
+  // earlier sub-blocks; q (this wavefront's rows only) is decayed further back with every one passed
   for (int J = w - 1; J >= 0; --J) {
     f32x4 pj = (f32x4)0.f;
-#pragma unroll
-    for (int s = 0; s < NS; ++s)
-      if (s < ns) pj = mma16(0.f, ldfrag(&Kh[(J * 16 + c) * KS + s * 16 + qd * 4]), as_frag(q[s]), pj);
-#pragma unroll
-    for (int vb = 0; vb < NS; ++vb)
-      if (vb < nv)
-        acc[vb] = mma16(0.f, ldfrag(&Vt[(vb * 16 + c) * kTS + J * 16 + qd * 4]), as_frag(pj), acc[vb]);
-#pragma unroll
-    for (int s = 0; s < NS; ++s)
-      if (s < ns) q[s] *= *reinterpret_cast<const f32x4*>(&Et[J * D + s * 16 + qd * 4]);
+#pragma unroll 4
+    for (int s = 0; s < ns; ++s) {
+      const int d = s * 16 + qd * 4;
+      f32x4* qp = reinterpret_cast<f32x4*>(&Q[t * KS + d]);
+      const f32x4 q = *qp;
+      pj = mma16(0.f, ldfrag(&Kh[(J * 16 + c) * KS + d]), as_frag(q), pj);
+      *qp = q * *reinterpret_cast<const f32x4*>(&Et[J * D + d]);
+    }
+    *reinterpret_cast<f32x4*>(&P[t * kTS + J * 16 + qd * 4]) = pj;
   }
-  if (c0 > 0 || sq.pos0 > 0) {
-    const float* S = ws + ((sq.row0 / kC + (long)blockIdx.z + blockIdx.x) * H + h) * chunk_floats(sh);
+  // values as they lie (a clamped token's weights are zero)
+  T v[NVB][4][4];
 #pragma unroll
-    for (int vb = 0; vb < NS; ++vb)
-      if (vb < nv) {
+  for (int b = 0; b < NVB; ++b)
+    if (w + 4 * b < nv) {
+      const T* src = proj + row0 * ld + sh.v_col + h * VD + (w + 4 * b) * 16 + c;
 #pragma unroll
-        for (int s = 0; s < NS; ++s)
-          if (s < ns)
-            acc[vb] = mma16(0.f, ldfrag(S + (long)(vb * 16 + c) * D + s * 16 + qd * 4), as_frag(q[s]),
-                            acc[vb]);
+      for (int J = 0; J < 4; ++J)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) v[b][J][j] = src[min(J * 16 + qd * 4 + j, n - 1) * ld];
+    }
+  const float* S = ws + ((sq.row0 / kC + (long)blockIdx.z + blockIdx.x) * H + h) * chunk_floats(sh);
+  __syncthreads();
+  // transposed outputs: acc[b][I] has the value channels 16 (w + 4 b) + 4 qd .. + 3 of token 16 I + c
+  f32x4 acc[NVB][4];
+  float ss[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int b = 0; b < NVB; ++b) {
+#pragma unroll
+    for (int I = 0; I < 4; ++I) acc[b][I] = (f32x4)0.f;
+    const int vb = w + 4 * b;
+    if (vb >= nv) continue;
+    if (has_state) {
+      frag_t fs[NS];
+#pragma unroll
+      for (int s = 0; s < NS; ++s)
+        if (s < ns) fs[s] = ldfrag(S + (long)(vb * 16 + c) * D + s * 16 + qd * 4);
+#pragma unroll
+      for (int s = 0; s < NS; ++s)
+        if (s < ns) {
+#pragma unroll
+          for (int I = 0; I < 4; ++I)
+            acc[b][I] = mma16(0.f, fs[s], ldfrag(&Q[(I * 16 + c) * KS + s * 16 + qd * 4]), acc[b][I]);
+        }
+    }
+#pragma unroll
+    for (int J = 0; J < 4; ++J) {
+      const f32x4 fv = {to_f(v[b][J][0]), to_f(v[b][J][1]), to_f(v[b][J][2]), to_f(v[b][J][3])};
+#pragma unroll
+      for (int I = J; I < 4; ++I)
+        acc[b][I] = mma16(0.f, as_frag(fv), ldfrag(&P[(I * 16 + c) * kTS + J * 16 + qd * 4]), acc[b][I]);
+    }
+#pragma unroll
+    for (int I = 0; I < 4; ++I)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) ss[I] += acc[b][I][e] * acc[b][I][e];
+  }
+#pragma unroll
+  for (int I = 0; I < 4; ++I) {
+    ss[I] += __shfl_xor(ss[I], 16);
+    ss[I] += __shfl_xor(ss[I], 32);
+    if (qd == 0) sq_sum[w * kC + I * 16 + c] = ss[I];
+  }
+  __syncthreads();
+#pragma unroll
+  for (int I = 0; I < 4; ++I) {
+    const int ti = I * 16 + c;
+    if (ti >= n) continue;
+    const float sum = (sq_sum[ti] + sq_sum[kC + ti]) + (sq_sum[2 * kC + ti] + sq_sum[3 * kC + ti]);
+    const float r = 1.0f / sqrtf(sum / (float)VD + sh.eps);
+#pragma unroll
+    for (int b = 0; b < NVB; ++b)
+      if (w + 4 * b < nv) {
+        const int vc = (w + 4 * b) * 16 + qd * 4;
+        const f32x4 g = load4(proj + (row0 + ti) * ld + sh.g_col + h * VD + vc), nw = load4(wt.norm + vc);
+        float o[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) o[e] = acc[b][I][e] * r * nw[e] * silu_f(g[e]);
+        stv<4, T>(out + ((row0 + ti) * H + h) * VD + vc, o);
       }
   }
-  float ss = 0.f;
-#pragma unroll
-  for (int vb = 0; vb < NS; ++vb)
-#pragma unroll
-    for (int e = 0; e < 4; ++e) ss += acc[vb][e] * acc[vb][e];
-  ss += __shfl_xor(ss, 16);
-  ss += __shfl_xor(ss, 32);
-  if (!in) return;
-  const float r = 1.0f / sqrtf(ss / (float)VD + sh.eps);
-#pragma unroll
-  for (int vb = 0; vb < NS; ++vb)
-    if (vb < nv) {
-      const int v = vb * 16 + qd * 4;
-      const f32x4 g = load4(pr + sh.g_col + h * VD + v), nw = load4(wt.norm + v);
-      float o[4];
-#pragma unroll
-      for (int e = 0; e < 4; ++e) o[e] = acc[vb][e] * r * nw[e] * silu_f(g[e]);
-      stv<4, T>(out + (row * H + h) * VD + v, o);
-    }
 }
 
 int check_shape(const GlaShape& sh) {
@@ -539,7 +598,7 @@ int gla_chunked(const T* proj, long ld, const float* low, const GlaWeights& w, f
   const int wide = std::max(D, VD);
   auto kern = wide <= 32 ? gla_chunk_out_kernel<T, 2> : wide <= 64 ? gla_chunk_out_kernel<T, 4>
             : wide <= 128 ? gla_chunk_out_kernel<T, 8> : gla_chunk_out_kernel<T, 16>;
-  const size_t lds = sizeof(float) * (48 * (size_t)(D + 4) + 4 * D + (size_t)VD * kTS);
+  const size_t lds = sizeof(float) * ((size_t)(kC + 48) * (D + 4) + kC * kTS + 4 * D + 4 * kC);
   if (int rc = room(reinterpret_cast<const void*>(kern), lds)) return rc;
   kern<<<grid, 256, lds, s>>>(proj, ld, low, w, workspace, out, seqs, sh);
   return lsh_check_launch("gla_chunk_out_kernel");
