@@ -172,6 +172,12 @@ int lsh_lm_gemm_gated_f32(const void* A, int64_t lda, const void* W, void* C, in
     int N, int K, int act, lsh_stream_t stream); /* act 0: silu, 1: relu */
 int lsh_lm_residual_f32(float* x, const lsh_residual_t* what, void* h, int rows, int width, float eps,
     const int* ids, const void* embed, int vocab, lsh_stream_t stream);
+int lsh_lm_attn_decode_append_f32(const void* proj, int64_t ld, int q_col, int k_col, void* k_cache,
+    void* out, const int* row_slot, const int* row_pos, int rows, int max_len, float* workspace, const
+    lsh_attn_shape_t* sh, const lsh_attn_mask_t* mask, lsh_stream_t stream);
+int lsh_lm_gemm_planes2_f32(const void* A0, int64_t lda0, const void* W0, float* C0, int K0, const
+    void* A1, int64_t lda1, const void* W1, float* C1, int K1, int M, int N, int max_planes, int*
+    planes0, int* planes1, lsh_stream_t stream);
 int lsh_lm_gla_step_f32(const void* proj, int64_t ld, const float* low, const float* a2, const float*
     bias, const float* norm, float* state, void* out, const int* row_slot, const int* row_pos, int
     rows, const lsh_gla_shape_t* sh, lsh_stream_t stream);
@@ -188,6 +194,12 @@ int lsh_lm_gemm_gated_bf16(const void* A, int64_t lda, const void* W, void* C, i
     int N, int K, int act, lsh_stream_t stream); /* act 0: silu, 1: relu */
 int lsh_lm_residual_bf16(float* x, const lsh_residual_t* what, void* h, int rows, int width, float eps,
     const int* ids, const void* embed, int vocab, lsh_stream_t stream);
+int lsh_lm_attn_decode_append_bf16(const void* proj, int64_t ld, int q_col, int k_col, void* k_cache,
+    void* out, const int* row_slot, const int* row_pos, int rows, int max_len, float* workspace, const
+    lsh_attn_shape_t* sh, const lsh_attn_mask_t* mask, lsh_stream_t stream);
+int lsh_lm_gemm_planes2_bf16(const void* A0, int64_t lda0, const void* W0, float* C0, int K0, const
+    void* A1, int64_t lda1, const void* W1, float* C1, int K1, int M, int N, int max_planes, int*
+    planes0, int* planes1, lsh_stream_t stream);
 int lsh_lm_gla_step_bf16(const void* proj, int64_t ld, const float* low, const float* a2, const float*
     bias, const float* norm, float* state, void* out, const int* row_slot, const int* row_pos, int
     rows, const lsh_gla_shape_t* sh, lsh_stream_t stream);

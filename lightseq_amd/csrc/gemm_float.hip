@@ -36,6 +36,13 @@ struct GemmArgs {
   int planes, k_per_plane;  // gemm_skinny_kernel, kDense
   GemmEpilogue epi;         // kDense
   int act;                  // kMoeUp, kGated
+  // gemm_skinny_kernel, kDense: a second product of the same M, N and ldc (blockIdx.z == 1)
+  struct {
+    const void *A, *W;
+    void* C;
+    long lda;
+    int K, planes, k_per_plane;
+  } other;
 };
 
 // rows of one tile: where they are read and written
@@ -292,19 +299,31 @@ gemm_tile_kernel(GemmArgs a, int tiles_m, int tiles_n) {
 
 // ------------------------------------------------------------------------------------------------
 // 16 * NS columns per workgroup (kDense; several strips share the activations), groups of 16 * MB
-// rows.  The weight fragment is the first operand: lane
+// rows; NW wavefronts split K.  HALVES (kGated): 8 columns, a fragment holds their gate rows and their
+// up rows.  The weight fragment is the first operand: lane
 // (c = lane % 16, q = lane / 16) holds column n0 + c's 16-byte chunk q of a 64-byte K slice.
-template <typename T, typename TO, int MODE, int MB, int NS = 1>
-__global__ void __launch_bounds__(256)
+template <typename T, typename TO, int MODE, int MB, int NS = 1, int NW = 4, bool HALVES = false>
+__global__ void __launch_bounds__(64 * NW)
 gemm_skinny_kernel(GemmArgs a) {
   static_assert(NS == 1 || MODE == kDense, "strips of one matrix");
-  constexpr int NB = is_up(MODE) ? 2 : NS;
+  static_assert(!HALVES || MODE == kGated, "gate and up rows");
+  constexpr int NB = is_up(MODE) && !HALVES ? 2 : NS;
   constexpr int V = FT<T>::kVec;
   constexpr int U = 4;  // 64-byte slices per turn: 256 bytes of every row
-  __shared__ float red[4][NB][MB][16][17];
+  __shared__ float red[NW][NB][MB][16][17];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int c = lane & 15, q = lane >> 4;
-  const int n0 = blockIdx.x * 16 * NS;
+  const int n0 = blockIdx.x * (HALVES ? 8 : 16 * NS);
+  if (MODE == kDense && blockIdx.z == 1) {
+    a.A = a.other.A;
+    a.W = a.other.W;
+    a.C = a.other.C;
+    a.lda = a.other.lda;
+    a.K = a.other.K;
+    a.planes = a.other.planes;
+    a.k_per_plane = a.other.k_per_plane;
+  }
+  if (MODE == kDense && (int)blockIdx.y >= a.planes) return;
   RowSet rs{0, 0, a.M};
   int k_lo = 0, k_hi = a.K;
   if (!is_dense(MODE)) {
@@ -320,7 +339,8 @@ gemm_skinny_kernel(GemmArgs a) {
   const T* wrow[NB];
 #pragma unroll
   for (int j = 0; j < NB; ++j)
-    wrow[j] = W + (is_up(MODE) ? (long)(min(n0 + c, a.N - 1) + j * a.N)
+    wrow[j] = HALVES ? W + (long)(min(n0 + (c & 7), a.N - 1) + (c >> 3) * a.N) * a.K
+                     : W + (is_up(MODE) ? (long)(min(n0 + c, a.N - 1) + j * a.N)
                                   : (long)min(n0 + j * 16 + c, a.N - 1)) * a.K;
   const T* A = reinterpret_cast<const T*>(a.A);
   const int first_end = rs.last;
@@ -334,7 +354,7 @@ gemm_skinny_kernel(GemmArgs a) {
     for (int j = 0; j < NB; ++j)
 #pragma unroll
       for (int i = 0; i < MB; ++i) acc[j][i] = (f32x4)0.f;
-    for (int k = k_lo + wave * (U * 4 * V); k < k_hi; k += 4 * U * 4 * V) {
+    for (int k = k_lo + wave * (U * 4 * V); k < k_hi; k += NW * U * 4 * V) {
       frag_t fw[U][NB], fa[U][MB];
 #pragma unroll
       for (int u = 0; u < U; ++u) {
@@ -361,18 +381,27 @@ gemm_skinny_kernel(GemmArgs a) {
 #pragma unroll
         for (int v = 0; v < 4; ++v) red[wave][j][i][c][4 * q + v] = acc[j][i][v];
     __syncthreads();
-    const int r = tid >> 4;
+    const int r = (tid >> 4) & 15;
 #pragma unroll
-    for (int i = 0; i < MB; ++i) {
+    for (int i = tid >> 8; i < MB; i += NW / 4) {
       const int row = first + i * 16 + r;
       if (row >= rs.last) continue;
       float s[NB];
 #pragma unroll
-      for (int j = 0; j < NB; ++j)
-        s[j] = (red[0][j][i][r][tid & 15] + red[1][j][i][r][tid & 15]) +
-               (red[2][j][i][r][tid & 15] + red[3][j][i][r][tid & 15]);
+      for (int j = 0; j < NB; ++j) {
+        s[j] = 0.f;
+#pragma unroll
+        for (int x = 0; x < NW; x += 4)
+          s[j] += (red[x][j][i][r][tid & 15] + red[x + 1][j][i][r][tid & 15]) +
+                  (red[x + 2][j][i][r][tid & 15] + red[x + 3][j][i][r][tid & 15]);
+      }
       const long m = dst_row<MODE>(a, rs, row);
-      if constexpr (is_up(MODE)) {
+      if constexpr (HALVES) {
+        const int n = n0 + (tid & 7);
+        const float up = __shfl_xor(s[0], 8);  // a row's 16 lanes are all here
+        if ((tid & 15) < 8 && n < a.N)
+          reinterpret_cast<TO*>(a.C)[m * a.ldc + n] = from_f<TO>(gated(a, s[0], up));
+      } else if constexpr (is_up(MODE)) {
         const int n = n0 + (tid & 15);
         if (n < a.N) reinterpret_cast<TO*>(a.C)[m * a.ldc + n] = from_f<TO>(gated(a, s[0], s[NB - 1]));
       } else {
@@ -481,19 +510,48 @@ bool tile_ok(const GemmArgs& a, int mode) {
 
 template <typename T, typename TO, int MODE>
 int launch_skinny(const GemmArgs& a, int rows, hipStream_t s) {
-  const dim3 grid((a.N + 15) / 16, is_dense(MODE) ? a.planes : a.experts);
-  if (grid.y > 65535) return lsh_fail(LSH_ERR_UNSUPPORTED, "float gemm: too many experts");
-  if constexpr (MODE == kDense) {
-    if (a.planes == 1 && rows > 16 && a.N >= 64 * cu_count()) {
-      const dim3 half((a.N + 31) / 32, 1);
-      if (rows <= 32) gemm_skinny_kernel<T, TO, MODE, 2, 2><<<half, 256, 0, s>>>(a);
-      else gemm_skinny_kernel<T, TO, MODE, 4, 2><<<half, 256, 0, s>>>(a);
-      return lsh_check_launch("gemm_skinny_kernel");
+  const int strips = (a.N + 15) / 16;
+  if constexpr (is_dense(MODE)) {
+    const dim3 grid(strips, std::max(a.planes, a.other.planes), a.other.A ? 2 : 1);
+    // a long K is split over eight wavefronts where there is at most a workgroup per compute unit
+    const bool deep = a.planes == 1 && a.K * (int)sizeof(T) >= 2048;
+    const bool wide = deep && strips <= cu_count();
+    if constexpr (MODE == kDense) {
+      if (a.planes == 1 && !a.other.A && rows > 16 && a.N >= 64 * cu_count()) {
+        const dim3 half((a.N + 31) / 32, 1);
+        if (rows <= 32) gemm_skinny_kernel<T, TO, MODE, 2, 2><<<half, 256, 0, s>>>(a);
+        else gemm_skinny_kernel<T, TO, MODE, 4, 2><<<half, 256, 0, s>>>(a);
+      } else if (rows <= 16) {
+        if (wide) gemm_skinny_kernel<T, TO, MODE, 1, 1, 8><<<grid, 512, 0, s>>>(a);
+        else gemm_skinny_kernel<T, TO, MODE, 1><<<grid, 256, 0, s>>>(a);
+      } else if (rows <= 32) {
+        if (wide) gemm_skinny_kernel<T, TO, MODE, 2, 1, 8><<<grid, 512, 0, s>>>(a);
+        else gemm_skinny_kernel<T, TO, MODE, 2><<<grid, 256, 0, s>>>(a);
+      } else {
+        gemm_skinny_kernel<T, TO, MODE, 4><<<grid, 256, 0, s>>>(a);
+      }
+    } else {
+      // strips of 8 columns fill the chip better, but read the activations twice as often
+      const dim3 eights((a.N + 7) / 8);
+      const bool halves = strips < (rows <= 16 ? 2 : 1) * cu_count();
+#define GATED(MB)                                                                             \
+  do {                                                                                        \
+    if (halves && deep) gemm_skinny_kernel<T, TO, MODE, MB, 1, 8, true><<<eights, 512, 0, s>>>(a); \
+    else if (halves) gemm_skinny_kernel<T, TO, MODE, MB, 1, 4, true><<<eights, 256, 0, s>>>(a);    \
+    else if (wide) gemm_skinny_kernel<T, TO, MODE, MB, 1, 8><<<grid, 512, 0, s>>>(a);         \
+    else gemm_skinny_kernel<T, TO, MODE, MB><<<grid, 256, 0, s>>>(a);                         \
+  } while (0)
+      if (rows <= 16) GATED(1);
+      else if (rows <= 32) GATED(2);
+      else gemm_skinny_kernel<T, TO, MODE, 4><<<grid, 256, 0, s>>>(a);
+#undef GATED
     }
+  } else {
+    if (a.experts > 65535) return lsh_fail(LSH_ERR_UNSUPPORTED, "float gemm: too many experts");
+    const dim3 grid(strips, a.experts);
+    if (rows <= 16) gemm_skinny_kernel<T, TO, MODE, 1><<<grid, 256, 0, s>>>(a);
+    else gemm_skinny_kernel<T, TO, MODE, 2><<<grid, 256, 0, s>>>(a);
   }
-  if (rows <= 16) gemm_skinny_kernel<T, TO, MODE, 1><<<grid, 256, 0, s>>>(a);
-  else if (rows <= 32 || !is_dense(MODE)) gemm_skinny_kernel<T, TO, MODE, 2><<<grid, 256, 0, s>>>(a);
-  else gemm_skinny_kernel<T, TO, MODE, 4><<<grid, 256, 0, s>>>(a);
   return lsh_check_launch("gemm_skinny_kernel");
 }
 
@@ -567,22 +625,46 @@ int gemm_float_preferred_planes(int M, int N, int K) {
   return p;
 }
 
+namespace {
+
+template <typename T>
+GemmArgs planes_args(const FloatProduct<T>& p, int M, int N, int max_planes) {
+  GemmArgs a{};
+  a.A = p.A; a.W = p.W; a.C = p.C;
+  a.lda = p.lda; a.ldc = N; a.n_split = N;
+  a.M = M; a.N = N; a.K = p.K;
+  a.planes = 1; a.k_per_plane = p.K;
+  if (M <= 64 && max_planes > 1 && rows_aligned<T>(a)) {
+    constexpr int step = 256 / sizeof(T);
+    const int n = std::min(gemm_float_preferred_planes(M, N, p.K), max_planes);
+    a.k_per_plane = ((p.K + n - 1) / n + step - 1) / step * step;
+    a.planes = (p.K + a.k_per_plane - 1) / a.k_per_plane;
+  }
+  return a;
+}
+
+}  // namespace
+
 template <typename T>
 int gemm_float_planes(const T* A, long lda, const T* W, float* C, int M, int N, int K,
                       int max_planes, int* planes_used, hipStream_t s) {
-  GemmArgs a{};
-  a.A = A; a.W = W; a.C = C;
-  a.lda = lda; a.ldc = N; a.n_split = N;
-  a.M = M; a.N = N; a.K = K;
-  a.planes = 1; a.k_per_plane = K;
-  if (M <= 64 && max_planes > 1 && rows_aligned<T>(a)) {
-    constexpr int step = 256 / sizeof(T);
-    int p = gemm_float_preferred_planes(M, N, K);
-    if (p > max_planes) p = max_planes;
-    a.k_per_plane = ((K + p - 1) / p + step - 1) / step * step;
-    a.planes = (K + a.k_per_plane - 1) / a.k_per_plane;
-  }
+  const GemmArgs a = planes_args(FloatProduct<T>{A, lda, W, C, K}, M, N, max_planes);
   *planes_used = a.planes;
+  return launch_any<T, float, kDense>(a, s);
+}
+
+template <typename T>
+int gemm_float_planes2(const FloatProduct<T>& p0, const FloatProduct<T>& p1, int M, int N,
+                       int max_planes, int* planes0, int* planes1, hipStream_t s) {
+  GemmArgs a = planes_args(p0, M, N, max_planes);
+  const GemmArgs b = planes_args(p1, M, N, max_planes);
+  *planes0 = a.planes;
+  *planes1 = b.planes;
+  if (!b.A || !b.W || !b.C || b.K <= 0 || M > 64 || !rows_aligned<T>(a) || !rows_aligned<T>(b)) {
+    if (int rc = launch_any<T, float, kDense>(a, s)) return rc;
+    return launch_any<T, float, kDense>(b, s);
+  }
+  a.other = {b.A, b.W, b.C, b.lda, b.K, b.planes, b.k_per_plane};
   return launch_any<T, float, kDense>(a, s);
 }
 
@@ -617,6 +699,8 @@ INST_TT(float, float)
 INST_TT(bf16_t, bf16_t)
 INST_TT(bf16_t, float)
 #define INST_T(T)                                                                               \
+  template int gemm_float_planes2<T>(const FloatProduct<T>&, const FloatProduct<T>&, int, int,  \
+                                     int, int*, int*, hipStream_t);                             \
   template int gemm_gated<T>(const T*, long, const T*, T*, long, int, int, int, int,            \
                              hipStream_t);                                                      \
   template int gemm_float_planes<T>(const T*, long, const T*, float*, int, int, int, int, int*, \

@@ -426,16 +426,30 @@ struct Packed {
       for (int i = 0; i < W; ++i) w[i] = reinterpret_cast<const uint32_t*>(p)[i];
     }
   }
+  __device__ __forceinline__ void store(T* p) const {
+#pragma unroll
+    for (int i = 0; i < W; ++i) reinterpret_cast<uint32_t*>(p)[i] = w[i];
+  }
   __device__ __forceinline__ float get(int e) const {
     if constexpr (sizeof(T) == 4) return __builtin_bit_cast(float, w[e]);
     else return __builtin_bit_cast(float, e & 1 ? w[e >> 1] & 0xffff0000u : w[e >> 1] << 16);
   }
 };
 
+// Where the queries lie, and (new_k; only where the values are the keys) the position's own key when
+// the cache does not hold it yet: every workgroup takes it from there, one of them appends it.
+template <typename T>
+struct DecodeSource {
+  const T* q;
+  long q_ld, q_head;  // elements from row to row, from head to head
+  const T* new_k;
+  long k_ld;
+};
+
 // EK, EV: elements per lane of a key / value row; SAME: the values are the keys, read once
 template <typename T, int EK, int EV, int R, bool SAME>
 __global__ void __launch_bounds__(kDecThreads)
-attn_decode_kernel(const T* __restrict__ q, const T* __restrict__ k_cache,
+attn_decode_kernel(DecodeSource<T> src, const T* __restrict__ k_cache,
                    const T* __restrict__ v_cache, const T* __restrict__ proj, long ld, int g_col,
                    T* __restrict__ out, const int* __restrict__ row_slot,
                    const int* __restrict__ row_pos, int nsplit, int head_groups,
@@ -452,6 +466,7 @@ attn_decode_kernel(const T* __restrict__ q, const T* __restrict__ k_cache,
   const long cache0 = ((long)row_slot[row] * sh.kv_heads + kvh) * sh.max_step;
   const T* kc = k_cache + cache0 * DP + j * EK;
   const T* vc = v_cache + cache0 * VP + j * EV;
+  const T* nk = SAME && src.new_k ? src.new_k + row * src.k_ld + kvh * DP + j * EK : nullptr;
   static_assert(!SAME || EK == EV, "values of the keys' size");
   const int lo = mask.first_seen(pos);  // first key of the window
   const int kept = min(mask.keep_first, lo);                           // kept keys before it
@@ -466,7 +481,8 @@ attn_decode_kernel(const T* __restrict__ q, const T* __restrict__ k_cache,
     for (int u = 0; u < U; ++u) {
       const int v = min(c0 + u * kDecGroups + grp, v_hi - 1);
       const long key = v < kept ? v : lo + v - kept;
-      ko[u].load(kc + key * DP);
+      if constexpr (SAME) ko[u].load(nk && key == pos ? nk : kc + key * DP);
+      else ko[u].load(kc + key * DP);
       if constexpr (!SAME) vo[u].load(vc + key * VP);
     }
   };
@@ -476,7 +492,7 @@ attn_decode_kernel(const T* __restrict__ q, const T* __restrict__ k_cache,
 #pragma unroll
   for (int r = 0; r < R; ++r) {
     Packed<T, EK> t;
-    t.load(q + ((long)row * sh.heads + h0 + min(r, nh - 1)) * DP + j * EK);
+    t.load(src.q + row * src.q_ld + (h0 + min(r, nh - 1)) * src.q_head + j * EK);
 #pragma unroll
     for (int e = 0; e < EK; ++e) qv[r][e] = t.get(e) * (mask.scale * kLog2e);
 #pragma unroll
@@ -528,6 +544,13 @@ attn_decode_kernel(const T* __restrict__ q, const T* __restrict__ k_cache,
     if (c0 + STEP < v_hi) {
       if (c0 + 2 * STEP < v_hi) fetch(c0 + 2 * STEP, kb[0], vb[0]);
       turn(c0 + STEP, kb[1], vb[1]);
+    }
+  }
+  if constexpr (SAME) {
+    if (nk && hg == 0 && split == 0 && grp == 0) {  // read from the cache by later launches only
+      Packed<T, EK> t;
+      t.load(nk);
+      t.store(const_cast<T*>(kc) + (long)pos * DP);
     }
   }
   // merge the groups: the wavefront's four by lane exchange, the wavefronts over LDS
@@ -685,7 +708,7 @@ size_t attn_decode_workspace(int rows, const AttnShape& sh) {
 
 #define DEC(EK, EV, R, SAME)                                                                     \
   attn_decode_kernel<T, EK, EV, R, SAME><<<grid, kDecThreads, 0, s>>>(                           \
-      q, k_cache, v_cache, proj, ld, g_col, out, row_slot, row_pos, nsplit, groups, workspace,   \
+      src, k_cache, v_cache, proj, ld, g_col, out, row_slot, row_pos, nsplit, groups, workspace,   \
       sh, mask)
 #define DEC_R(EK, EV, SAME)                                                                      \
   do {                                                                                           \
@@ -702,12 +725,14 @@ size_t attn_decode_workspace(int rows, const AttnShape& sh) {
     default: DEC_R(EK, 16, false); break;                                                        \
   }
 
+namespace {
+
 template <typename T>
-int attn_decode(const T* q, const T* k_cache, const T* v_cache, const T* proj, long ld, int g_col,
-                T* out, const int* row_slot, const int* row_pos, int rows, int max_len,
-                float* workspace, const AttnShape& sh, const AttnMask& mask, hipStream_t s) {
+int launch_decode(const DecodeSource<T>& src, const T* k_cache, const T* v_cache, const T* proj, long ld,
+                  int g_col, T* out, const int* row_slot, const int* row_pos, int rows, int max_len,
+                  float* workspace, const AttnShape& sh, const AttnMask& mask, hipStream_t s) {
   if (int rc = check_shape(sh, "attn_decode: bad shape")) return rc;
-  if (!q || !k_cache || !v_cache || !out || !row_slot || !row_pos || rows <= 0 || max_len <= 0 ||
+  if (!src.q || !k_cache || !v_cache || !out || !row_slot || !row_pos || rows <= 0 || max_len <= 0 ||
       !workspace || (g_col >= 0 && !proj) || (v_cache == k_cache && sh.dim != sh.vdim) ||
       mask.chunk < 0)
     return lsh_fail(LSH_ERR_INVALID, "attn_decode: bad arguments");
@@ -742,6 +767,34 @@ int attn_decode(const T* q, const T* k_cache, const T* v_cache, const T* proj, l
   return LSH_OK;
 }
 
+}  // namespace
+
+template <typename T>
+int attn_decode(const T* q, const T* k_cache, const T* v_cache, const T* proj, long ld, int g_col,
+                T* out, const int* row_slot, const int* row_pos, int rows, int max_len,
+                float* workspace, const AttnShape& sh, const AttnMask& mask, hipStream_t s) {
+  return launch_decode<T>(DecodeSource<T>{q, (long)sh.heads * sh.dim_pad, sh.dim_pad, nullptr, 0},
+                          k_cache, v_cache, proj, ld, g_col, out, row_slot, row_pos, rows, max_len,
+                          workspace, sh, mask, s);
+}
+
+bool attn_decode_append_supported(const AttnShape& sh, int q_col, int k_col, long ld) {
+  return sh.dim == sh.vdim && sh.dim == sh.dim_pad && (q_col | k_col) % 8 == 0 && ld % 8 == 0;
+}
+
+template <typename T>
+int attn_decode_append(const T* proj, long ld, int q_col, int k_col, T* k_cache, T* out,
+                       const int* row_slot, const int* row_pos, int rows, int max_len,
+                       float* workspace, const AttnShape& sh, const AttnMask& mask, hipStream_t s) {
+  if (!proj || q_col < 0 || k_col < 0 || (reinterpret_cast<uintptr_t>(proj) & 15u) != 0)
+    return lsh_fail(LSH_ERR_INVALID, "attn_decode_append: bad arguments");
+  if (!attn_decode_append_supported(sh, q_col, k_col, ld))
+    return lsh_fail(LSH_ERR_UNSUPPORTED, "attn_decode_append: head sizes or columns need padding");
+  return launch_decode<T>(DecodeSource<T>{proj + q_col, ld, sh.dim, proj + k_col, ld}, k_cache,
+                          k_cache, nullptr, 0, -1, out, row_slot, row_pos, rows, max_len, workspace,
+                          sh, mask, s);
+}
+
 #define INST(T)                                                                                   \
   template int attn_prepare<T>(const T*, long, int, int, int, const float*, const float*, float,  \
                                const float2*, int, T*, T*, T*, const int*, const int*, int,       \
@@ -751,7 +804,10 @@ int attn_decode(const T* q, const T* k_cache, const T* v_cache, const T* proj, l
                                hipStream_t);                                                      \
   template int attn_decode<T>(const T*, const T*, const T*, const T*, long, int, T*, const int*,  \
                               const int*, int, int, float*, const AttnShape&, const AttnMask&,    \
-                              hipStream_t);
+                              hipStream_t);                                                       \
+  template int attn_decode_append<T>(const T*, long, int, int, T*, T*, const int*, const int*,    \
+                                     int, int, float*, const AttnShape&, const AttnMask&,         \
+                                     hipStream_t);
 INST(float)
 INST(bf16_t)
 

@@ -221,6 +221,25 @@ int lsh_lm_sample(const float* logits, int rows, int vocab, int topk, float topp
     return lm_norm<T>(x, add, norm, (T*)h, rows, width, eps, ids, (const T*)embed, vocab, nullptr, \
                       nullptr, 0, HS(s), inject);                                                  \
   }                                                                                                \
+  int lsh_lm_attn_decode_append_##SUF(const void* proj, int64_t ld, int q_col, int k_col,          \
+                                      void* k_cache, void* out, const int* row_slot,               \
+                                      const int* row_pos, int rows, int max_len, float* workspace, \
+                                      const lsh_attn_shape_t* sh, const lsh_attn_mask_t* mask,     \
+                                      lsh_stream_t s) {                                            \
+    NEED(sh && mask);                                                                              \
+    return attn_decode_append<T>((const T*)proj, ld, q_col, k_col, (T*)k_cache, (T*)out, row_slot, \
+                                 row_pos, rows, max_len, workspace, shape_of(*sh), mask_of(*mask), \
+                                 HS(s));                                                           \
+  }                                                                                                \
+  int lsh_lm_gemm_planes2_##SUF(const void* A0, int64_t lda0, const void* W0, float* C0, int K0,   \
+                                const void* A1, int64_t lda1, const void* W1, float* C1, int K1,   \
+                                int M, int N, int max_planes, int* planes0, int* planes1,          \
+                                lsh_stream_t s) {                                                  \
+    NEED(planes0 && planes1);                                                                      \
+    return gemm_float_planes2<T>(FloatProduct<T>{(const T*)A0, lda0, (const T*)W0, C0, K0},        \
+                                 FloatProduct<T>{(const T*)A1, lda1, (const T*)W1, C1, K1}, M, N,  \
+                                 max_planes, planes0, planes1, HS(s));                             \
+  }                                                                                                \
   int lsh_lm_gla_step_##SUF(const void* proj, int64_t ld, const float* low, const float* a2,       \
                             const float* bias, const float* norm, float* state, void* out,         \
                             const int* row_slot, const int* row_pos, int rows,                     \

@@ -32,6 +32,18 @@ template <typename T>
 int gemm_float_planes(const T* A, long lda, const T* W, float* C, int M, int N, int K,
                       int max_planes, int* planes_used, hipStream_t s);
 int gemm_float_preferred_planes(int M, int N, int K);
+// two such products of different inputs and weights, in one launch for few rows
+template <typename T>
+struct FloatProduct {
+  const T* A;
+  long lda;
+  const T* W;
+  float* C;
+  int K;
+};
+template <typename T>
+int gemm_float_planes2(const FloatProduct<T>& p0, const FloatProduct<T>& p1, int M, int N,
+                       int max_planes, int* planes0, int* planes1, hipStream_t s);
 
 // C[m, n] = act(gate_n A[m]) * (up_n A[m]), weights [2][N][K]: the gates' rows, then the others
 enum GateAct { kGateSilu = 0, kGateRelu = 1 };
@@ -145,6 +157,13 @@ template <typename T>
 int attn_decode(const T* q, const T* k_cache, const T* v_cache, const T* proj, long ld, int g_col,
                 T* out, const int* row_slot, const int* row_pos, int rows, int max_len,
                 float* workspace, const AttnShape& sh, const AttnMask& mask, hipStream_t s);
+// The same with queries and the position's key straight from the projection, where the values are the
+// keys: the key is appended to the cache on the way.
+template <typename T>
+int attn_decode_append(const T* proj, long ld, int q_col, int k_col, T* k_cache, T* out,
+                       const int* row_slot, const int* row_pos, int rows, int max_len,
+                       float* workspace, const AttnShape& sh, const AttnMask& mask, hipStream_t s);
+bool attn_decode_append_supported(const AttnShape& sh, int q_col, int k_col, long ld);
 size_t attn_decode_workspace(int rows, const AttnShape& sh);
 
 // ---- gated delta rule (delta_kernels.hip) -----------------------------------------------------

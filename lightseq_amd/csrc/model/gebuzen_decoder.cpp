@@ -98,8 +98,7 @@ class Stack : public DecoderStack {
       }
       mixer(i, b);
       AddSpec add = spec(few, 0.5f * (float)_c.residual_mult);
-      product(_left, l.heads * l.dim, w.left_o, R, few, 0, add);
-      product(_right, l.gla_heads * l.gla_vdim, w.right_o, R, few, 1, add.second);
+      products_out(l, w, R, few, add);
       add.post_w = w.left_norm.get();
       add.second.post_w = w.right_norm.get();
       if (l.ff) {
@@ -108,7 +107,7 @@ class Stack : public DecoderStack {
         LSH_CALL(gemm_gated<T>(_h.get(), W, w.up.get(), _act.get(), l.ff, R, l.ff, W, kGateRelu,
                                _stream));
         add = spec(few, (float)_c.residual_mult);
-        product(_act, l.ff, w.down, R, few, 0, add);
+        product_down(l, w, R, few, add);
       }
       InjectSpec inject = i + 1 < n ? ahead_of(i + 1, b) : InjectSpec{};
       if (inject.any() && taps.wants(i, tap_step, "res_out")) {
@@ -180,24 +179,32 @@ class Stack : public DecoderStack {
     LSH_CALL((gemm_float<T, T>(_h.get(), _c.width, w.in.get(), _proj.get(), ld, _low.get(), w.rank,
                                w.t_cols, R, w.in_cols, _c.width, _stream, biased)));
     const AttnShape sh = attn_shape(l);
-    LSH_CALL(attn_prepare<T>(_proj.get(), ld, w.q_col, w.k_col, -1, nullptr, nullptr, 0.f, nullptr, 0,
-                             _q.get(), c.k.get(), nullptr, b.row_slot, b.row_pos, R, sh, _stream));
     AttnMask mask{0, 0, (float)l.scale, true};
     mask.chunk = l.chunk;
     mask.sinks = w.sink.get();
     const GlaShape gs = gla_shape(layer);
     const GlaWeights gw{w.a2.get(), w.a2_bias.get(), w.head_norm.get()};
-    if (b.max_n == 1) {
-      LSH_CALL(attn_decode<T>(_q.get(), c.k.get(), c.k.get(), nullptr, 0, -1, _left.get(),
-                              b.row_slot, b.row_pos, R, b.max_len, _attn_ws.get(), sh, mask,
-                              _stream));
+    const bool one = b.max_n == 1;
+    if (one && attn_decode_append_supported(sh, w.q_col, w.k_col, ld)) {
+      LSH_CALL(attn_decode_append<T>(_proj.get(), ld, w.q_col, w.k_col, c.k.get(), _left.get(),
+                                     b.row_slot, b.row_pos, R, b.max_len, _attn_ws.get(), sh, mask,
+                                     _stream));
+    } else {
+      LSH_CALL(attn_prepare<T>(_proj.get(), ld, w.q_col, w.k_col, -1, nullptr, nullptr, 0.f, nullptr,
+                               0, _q.get(), c.k.get(), nullptr, b.row_slot, b.row_pos, R, sh,
+                               _stream));
+      if (one)
+        LSH_CALL(attn_decode<T>(_q.get(), c.k.get(), c.k.get(), nullptr, 0, -1, _left.get(),
+                                b.row_slot, b.row_pos, R, b.max_len, _attn_ws.get(), sh, mask,
+                                _stream));
+      else
+        LSH_CALL(attn_prefill<T>(_q.get(), c.k.get(), c.k.get(), nullptr, 0, -1, _left.get(), b.spans,
+                                 b.n_seqs, b.max_n, sh, mask, _stream));
+    }
+    if (one)
       LSH_CALL(gla_step<T>(_proj.get(), ld, _low.get(), gw, c.state.get(), _right.get(), b.row_slot,
                            b.row_pos, R, gs, _stream));
-      return;
-    }
-    LSH_CALL(attn_prefill<T>(_q.get(), c.k.get(), c.k.get(), nullptr, 0, -1, _left.get(), b.spans,
-                             b.n_seqs, b.max_n, sh, mask, _stream));
-    if (b.max_n > kScanRows && gla_chunked_supported(gs, ld))
+    else if (b.max_n > kScanRows && gla_chunked_supported(gs, ld))
       LSH_CALL(gla_chunked<T>(_proj.get(), ld, _low.get(), gw, c.state.get(), _right.get(),
                               _chunk.get(), b.spans, b.n_seqs, b.max_n, R, gs, _stream));
     else
@@ -205,22 +212,44 @@ class Stack : public DecoderStack {
                            b.n_seqs, gs, _stream));
   }
 
-  // a [R][k] times the weights [width][k]: what is left to add to the stream
-  void product(const DeviceBuffer<T>& a, int k, const DeviceBuffer<T>& w, int R, bool few, int which,
-               AddPart& part) {
-    const int W = _c.width;
-    part.row_stride = W;
-    part.parts = 1;
+  // both mixers' output projections: what is left to add to the stream
+  void products_out(const GebuzenLayerConfig& l, const GebuzenLayerWeight<T>& w, int R, bool few,
+                    AddSpec& add) {
+    const int k0 = l.heads * l.dim, k1 = l.gla_heads * l.gla_vdim;
     if (few) {
-      LSH_CALL(gemm_float_planes<T>(a.get(), k, w.get(), _yf[which].get(), R, W, k, kMaxPlanes,
-                                    &part.parts, _stream));
-      part.y = _yf[which].get();
-      part.part_stride = (long)R * W;
+      add.part_stride = add.second.part_stride = (long)R * _c.width;
+      LSH_CALL(gemm_float_planes2<T>(FloatProduct<T>{_left.get(), k0, w.left_o.get(), _yf[0].get(), k0},
+                                     FloatProduct<T>{_right.get(), k1, w.right_o.get(), _yf[1].get(), k1},
+                                     R, _c.width, kMaxPlanes, &add.parts, &add.second.parts, _stream));
     } else {
-      LSH_CALL((gemm_float<T, T>(a.get(), k, w.get(), _y[which].get(), W, nullptr, 0, W, R, W, k,
-                                 _stream)));
-      part.y = _y[which].get();
+      add.parts = add.second.parts = 1;
+      many_rows(_left, k0, w.left_o, R, 0);
+      many_rows(_right, k1, w.right_o, R, 1);
     }
+    locate(few, 0, add);
+    locate(few, 1, add.second);
+  }
+  // the feed-forward's
+  void product_down(const GebuzenLayerConfig& l, const GebuzenLayerWeight<T>& w, int R, bool few,
+                    AddSpec& add) {
+    add.parts = 1;
+    if (few) {
+      add.part_stride = (long)R * _c.width;
+      LSH_CALL(gemm_float_planes<T>(_act.get(), l.ff, w.down.get(), _yf[0].get(), R, _c.width, l.ff,
+                                    kMaxPlanes, &add.parts, _stream));
+    } else {
+      many_rows(_act, l.ff, w.down, R, 0);
+    }
+    locate(few, 0, add);
+  }
+  void many_rows(const DeviceBuffer<T>& a, int k, const DeviceBuffer<T>& w, int R, int which) {
+    const int W = _c.width;
+    LSH_CALL((gemm_float<T, T>(a.get(), k, w.get(), _y[which].get(), W, nullptr, 0, W, R, W, k,
+                               _stream)));
+  }
+  void locate(bool few, int which, AddPart& part) {
+    part.row_stride = _c.width;
+    part.y = few ? (const void*)_yf[which].get() : (const void*)_y[which].get();
   }
 
   const GebuzenConfig _c;

@@ -193,6 +193,8 @@ _LM_SIGNATURES = {
     "lsh_lm_gemm_epilogue": (True, "plpplpliiiifps"),
     "lsh_lm_gemm_gated": (True, "plppliiiis"),
     "lsh_lm_residual": (True, "pppiifppis"),
+    "lsh_lm_attn_decode_append": (True, "pliipp" + "pp" + "ii" + "ppps"),
+    "lsh_lm_gemm_planes2": (True, "plppiplppi" + "iiipps"),
     "lsh_lm_gla_step": (True, "plppppppppips"),
     "lsh_lm_gla_scan": (True, "plpppppppips"),
     "lsh_lm_gla_chunked": (True, "plppppppppiiips"),

@@ -76,7 +76,7 @@ def rng(seed=0):
 @pytest.mark.parametrize("m,n,k,split", [
     (1, 40, 64, 40), (5, 33, 48, 20), (16, 256, 512, 250), (40, 64, 1024, 64), (64, 100, 72, 64),
     (65, 128, 64, 128), (130, 200, 128, 190), (257, 96, 192, 96), (300, 50, 27, 44), (3, 70, 75, 70),
-    (20, 16400, 72, 16400), (50, 16500, 64, 16487), (2048, 2048, 256, 2048), (2100, 2080, 128, 2072),
+    (20, 16400, 72, 16400), (50, 16500, 64, 16487), (32, 700, 2056, 690), (7, 50, 1024, 50), (2048, 2048, 256, 2048), (2100, 2080, 128, 2072),
 ])
 def test_gemm(dt, m, n, k, split):
     r = rng(m * n + k)
@@ -120,7 +120,7 @@ def test_gemm_scale_and_bias(dt, m, n, k, split):
 
 
 @pytest.mark.parametrize("dt", DTYPES)
-@pytest.mark.parametrize("m,n,k", [(1, 40, 64), (20, 33, 48), (33, 64, 1024), (64, 100, 72), (65, 128, 64), (130, 200, 128),
+@pytest.mark.parametrize("m,n,k", [(1, 40, 64), (20, 33, 48), (33, 64, 1024), (9, 50, 1032), (32, 200, 2048), (16, 8200, 64), (30, 8200, 72), (64, 100, 72), (65, 128, 64), (130, 200, 128),
                                    (300, 50, 27), (2100, 1040, 128), (2048, 2048, 64)])
 def test_gated_product(dt, m, n, k):
     r = rng(m + n + k)
@@ -526,6 +526,53 @@ def test_attn_decode_chunked(dt, case):
     call("lsh_lm_attn_decode_" + dt, *head, ints([s for s, _ in qpos]), ints([p for _, p in qpos]), rows, S, ws, sh,
          mask)
     close(host(out), want, dt)
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("case", range(len(CHUNKED_DECODE)))
+def test_attn_decode_append(dt, case):
+    """The position's own key comes with the projection and is in the cache afterwards."""
+    from lightseq_amd import lib
+    from lightseq_amd.lib import LSHError
+    H, G, D, VD, positions, window, keep, chunk, same = CHUNKED_DECODE[case]
+    S, rows = max(positions) + 5, len(positions)
+    (q, kc, *_, out), sh, mask, meta, qpos, want, out = attention_case(
+        dt, H, G, D, D, [(p, 1) for p in positions], S, window, keep, gate=False, chunk=chunk,
+        sinks=sink_logits(H, case), same=True)
+    slots, pos = [s for s, _ in qpos], [p for _, p in qpos]
+    ld, qc, kcol = 16 + (H + G) * D + (-(H + G) * D) % 8, 16 + G * D, 8
+    proj = np.zeros((rows, ld))
+    proj[:, qc:qc + H * D] = host(q)[..., :D].reshape(rows, -1)
+    before = host(kc)
+    for i in range(rows):
+        proj[i, kcol:kcol + G * D] = before[slots[i], :, pos[i], :D].reshape(-1)
+        kc[slots[i], :, pos[i]] = float("nan")
+    ws = torch.empty(lib.load().lsh_lm_attn_decode_workspace(rows, ctypes.addressof(sh)), device="cuda")
+    args = ("lsh_lm_attn_decode_append_" + dt, dev(proj, dt), ld, qc, kcol, kc, out, ints(slots), ints(pos), rows, S, ws,
+            sh, mask)
+    if D not in (64, 96, 128, 256):
+        with pytest.raises(LSHError, match="need padding"):
+            call(*args)
+        return
+    call(*args)
+    close(host(out), want, dt)
+    assert np.array_equal(host(kc), before, equal_nan=True)
+
+
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("m,n,k0,k1", [(1, 40, 64, 2048), (16, 128, 1024, 96), (33, 250, 512, 512), (64, 64, 72, 4096),
+                                       (65, 48, 64, 128), (5, 30, 27, 64), (20, 16400, 64, 72)])
+def test_two_products_at_once(dt, m, n, k0, k1):
+    r = rng(m + k0)
+    a = [rounded(r.normal(size=(m, k)), dt) for k in (k0, k1)]
+    w = [rounded(r.normal(size=(n, k)), dt) for k in (k0, k1)]
+    c = [torch.full((8, m, n), float("nan"), device="cuda") for _ in range(2)]
+    planes = [ctypes.c_int(0), ctypes.c_int(0)]
+    call("lsh_lm_gemm_planes2_" + dt, dev(a[0], dt), k0, dev(w[0], dt), c[0], k0, dev(a[1], dt), k1, dev(w[1], dt), c[1],
+         k1, m, n, 8, *map(ctypes.addressof, planes))
+    for i in range(2):
+        got = host(c[i]).reshape(-1)[:planes[i].value * m * n].reshape(planes[i].value, m, n).sum(0)
+        close(got, a[i] @ w[i].T, "f32")
 
 
 @pytest.mark.parametrize("dt", DTYPES)
