@@ -227,25 +227,36 @@ __device__ __forceinline__ f32x4 sum_after(f32x4 x) {
   return x;
 }
 
-// the chunk's values, transposed: Vt[v][token], zeros for tokens that are not there
-constexpr int kTS = kC + 4;
-template <typename T>
-__device__ __forceinline__ void stage_values(const T* __restrict__ proj, long ld, long row0, int n,
-                                             const GlaShape& sh, int h, float* Vt) {
-  const int t = threadIdx.x >> 2;
-  const T* src = proj + (row0 + min(t, n - 1)) * ld + sh.v_col + h * sh.vdim;
-  for (int v = (threadIdx.x & 3) * 4; v < sh.vdim; v += 16) {
-    const f32x4 x = t < n ? load4(src + v) : (f32x4)0.f;
+constexpr int kTS = kC + 4;  // row length of a matrix with the chunk's tokens as columns
+
+// Values of a wavefront's blocks w, w + 4, .. as an operand: value channel c of its block, the tokens
+// 16 J + 4 qd .. + 3.  A token that is not there is the last one again (its weights are zero).
+template <typename T, int NVB>
+struct ChunkValues {
+  T x[NVB][4][4];
+  __device__ __forceinline__ void fetch(const T* __restrict__ proj, long ld, long row0, int n,
+                                        const GlaShape& sh, int h, int w, int c, int qd) {
 #pragma unroll
-    for (int e = 0; e < 4; ++e) Vt[(v + e) * kTS + t] = x[e];
+    for (int b = 0; b < NVB; ++b)
+      if ((w + 4 * b) * 16 < sh.vdim) {
+        const T* src = proj + row0 * ld + sh.v_col + h * sh.vdim + (w + 4 * b) * 16 + c;
+#pragma unroll
+        for (int J = 0; J < 4; ++J)
+#pragma unroll
+          for (int j = 0; j < 4; ++j) x[b][J][j] = src[min(J * 16 + qd * 4 + j, n - 1) * ld];
+      }
   }
-}
+  __device__ __forceinline__ frag_t frag(int b, int J) const {
+    return as_frag(f32x4{to_f(x[b][J][0]), to_f(x[b][J][1]), to_f(x[b][J][2]), to_f(x[b][J][3])});
+  }
+};
 
 // what a chunk adds to the state, and its decay
-template <typename T, int NS>  // dim <= 16 * NS
-__global__ void __launch_bounds__(256)
+template <typename T, int NS>  // dim, vdim <= 16 * NS
+__global__ void __launch_bounds__(256, NS <= 4 ? 4 : NS <= 8 ? 3 : 1)
 gla_chunk_add_kernel(const T* __restrict__ proj, long ld, const float* __restrict__ low, GlaWeights wt,
                      float* __restrict__ ws, const SeqSpan* __restrict__ seqs, GlaShape sh) {
+  constexpr int NVB = (NS + 3) / 4;  // value blocks of a wavefront
   extern __shared__ __attribute__((aligned(16))) float sm[];
   const SeqSpan sq = seqs[blockIdx.z];
   const int c0 = blockIdx.x * kC;
@@ -254,8 +265,7 @@ gla_chunk_add_kernel(const T* __restrict__ proj, long ld, const float* __restric
   const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, c = lane & 15, qd = lane >> 4;
   const int ns = D / 16, nv = VD / 16;
   float* Kt = sm;                 // [D][kTS]
-  float* Vt = Kt + D * kTS;       // [VD][kTS]
-  float* tot = Vt + VD * kTS;     // [4][D]: log decay of every sub-block
+  float* tot = Kt + D * kTS;      // [4][D]: log decay of every sub-block
   const long row0 = sq.row0 + c0;
   const int t = w * 16 + c;
   const bool in = t < n;
@@ -264,7 +274,8 @@ gla_chunk_add_kernel(const T* __restrict__ proj, long ld, const float* __restric
 #pragma unroll
   for (int s = 0; s < NS; ++s)
     k[s] = s < ns && in ? load4(proj + row * ld + sh.k_col + h * D + s * 16 + qd * 4) : (f32x4)0.f;
-  stage_values(proj, ld, row0, n, sh, h, Vt);
+  ChunkValues<T, NVB> values;
+  values.fetch(proj, ld, row0, n, sh, h, w, c, qd);
   chunk_log_decays<NS>(low, row, in, wt, sh, h, 0, c, qd, la);
 #pragma unroll
   for (int s = 0; s < NS; ++s)
@@ -287,14 +298,19 @@ gla_chunk_add_kernel(const T* __restrict__ proj, long ld, const float* __restric
   for (int d = tid; d < D; d += 256)
     o[(long)VD * D + d] = exp2_f((tot[d] + tot[D + d]) + (tot[2 * D + d] + tot[3 * D + d]));
   __syncthreads();
-  for (int x = w; x < ns * nv; x += 4) {
-    const int db = x % ns, vb = x / ns;
-    f32x4 acc = (f32x4)0.f;
+  for (int db = 0; db < ns; ++db) {
+    frag_t fk[4];
 #pragma unroll
-    for (int j = 0; j < 4; ++j)
-      acc = mma16(0.f, ldfrag(&Kt[(db * 16 + c) * kTS + j * 16 + qd * 4]),
-                  ldfrag(&Vt[(vb * 16 + c) * kTS + j * 16 + qd * 4]), acc);
-    *reinterpret_cast<f32x4*>(&o[(long)(vb * 16 + c) * D + db * 16 + qd * 4]) = acc;
+    for (int J = 0; J < 4; ++J) fk[J] = ldfrag(&Kt[(db * 16 + c) * kTS + J * 16 + qd * 4]);
+#pragma unroll
+    for (int b = 0; b < NVB; ++b) {
+      const int vb = w + 4 * b;
+      if (vb >= nv) continue;
+      f32x4 acc = (f32x4)0.f;
+#pragma unroll
+      for (int J = 0; J < 4; ++J) acc = mma16(0.f, fk[J], values.frag(b, J), acc);
+      *reinterpret_cast<f32x4*>(&o[(long)(vb * 16 + c) * D + db * 16 + qd * 4]) = acc;
+    }
   }
 }
 
@@ -380,17 +396,34 @@ gla_chunk_out_kernel(const T* __restrict__ proj, long ld, const float* __restric
     float x[16];
 #pragma unroll
     for (int i = 0; i < 16; ++i) x[i] = 0.f;
+    // the next group's keys, queries and decays are under way while the present one is worked on
+    typedef T T4 __attribute__((ext_vector_type(4)));
+    T4 kn[GS], qn[GS];
+    f32x4 ln[GS];
+    const auto fetch = [&](int s0) {
+#pragma unroll
+      for (int s = 0; s < GS; ++s) {
+        const int d = h * D + (s0 + s) * 16 + qd * 4;
+        const bool there = s0 + s < ns && in;
+        kn[s] = there ? *reinterpret_cast<const T4*>(pr + sh.k_col + d) : (T4)0.f;
+        qn[s] = there ? *reinterpret_cast<const T4*>(pr + sh.q_col + d) : (T4)0.f;
+      }
+      chunk_log_decays<GS>(low, row, in, wt, sh, h, s0, c, qd, ln);
+    };
+    fetch(0);
 #pragma unroll 1
     for (int s0 = 0; s0 < ns; s0 += GS) {
       f32x4 k[GS], la[GS], wq[GS];
 #pragma unroll
       for (int s = 0; s < GS; ++s) {
-        const int d = h * D + (s0 + s) * 16 + qd * 4;
-        const bool there = s0 + s < ns && in;
-        k[s] = there ? load4(pr + sh.k_col + d) : (f32x4)0.f;
-        wq[s] = there ? load4(pr + sh.q_col + d) * qscale : (f32x4)0.f;
+        la[s] = ln[s];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          k[s][e] = to_f((T)kn[s][e]);
+          wq[s][e] = to_f((T)qn[s][e]) * qscale;
+        }
       }
-      chunk_log_decays<GS>(low, row, in, wt, sh, h, s0, c, qd, la);
+      if (s0 + GS < ns) fetch(s0 + GS);
 #pragma unroll
       for (int s = 0; s < GS; ++s)
         if (s0 + s < ns) {
@@ -427,17 +460,8 @@ gla_chunk_out_kernel(const T* __restrict__ proj, long ld, const float* __restric
     }
     *reinterpret_cast<f32x4*>(&P[t * kTS + J * 16 + qd * 4]) = pj;
   }
-  // values as they lie (a clamped token's weights are zero)
-  T v[NVB][4][4];
-#pragma unroll
-  for (int b = 0; b < NVB; ++b)
-    if (w + 4 * b < nv) {
-      const T* src = proj + row0 * ld + sh.v_col + h * VD + (w + 4 * b) * 16 + c;
-#pragma unroll
-      for (int J = 0; J < 4; ++J)
-#pragma unroll
-        for (int j = 0; j < 4; ++j) v[b][J][j] = src[min(J * 16 + qd * 4 + j, n - 1) * ld];
-    }
+  ChunkValues<T, NVB> values;
+  values.fetch(proj, ld, row0, n, sh, h, w, c, qd);
   const float* S = ws + ((sq.row0 / kC + (long)blockIdx.z + blockIdx.x) * H + h) * chunk_floats(sh);
   __syncthreads();
   // transposed outputs: acc[b][I] has the value channels 16 (w + 4 b) + 4 qd .. + 3 of token 16 I + c
@@ -464,10 +488,10 @@ gla_chunk_out_kernel(const T* __restrict__ proj, long ld, const float* __restric
     }
 #pragma unroll
     for (int J = 0; J < 4; ++J) {
-      const f32x4 fv = {to_f(v[b][J][0]), to_f(v[b][J][1]), to_f(v[b][J][2]), to_f(v[b][J][3])};
+      const frag_t fv = values.frag(b, J);
 #pragma unroll
       for (int I = J; I < 4; ++I)
-        acc[b][I] = mma16(0.f, as_frag(fv), ldfrag(&P[(I * 16 + c) * kTS + J * 16 + qd * 4]), acc[b][I]);
+        acc[b][I] = mma16(0.f, fv, ldfrag(&P[(I * 16 + c) * kTS + J * 16 + qd * 4]), acc[b][I]);
     }
 #pragma unroll
     for (int I = 0; I < 4; ++I)
@@ -578,16 +602,16 @@ int gla_chunked(const T* proj, long ld, const float* low, const GlaWeights& w, f
   if (!gla_chunked_supported(sh, ld))
     return lsh_fail(LSH_ERR_UNSUPPORTED, "gla_chunked: head sizes must be multiples of 16");
   const dim3 grid((max_n + kC - 1) / kC, sh.heads, n_seqs);
-  const int D = sh.dim, VD = sh.vdim;
+  const int D = sh.dim, VD = sh.vdim, wide = std::max(D, VD);
   const auto room = [](const void* kernel, size_t lds) {
     return lsh_check_hip(hipFuncSetAttribute(kernel, hipFuncAttributeMaxDynamicSharedMemorySize,
                                              (int)lds),
                          "hipFuncSetAttribute(gla_chunk)");
   };
   {
-    auto kern = D <= 32 ? gla_chunk_add_kernel<T, 2> : D <= 64 ? gla_chunk_add_kernel<T, 4>
-              : D <= 128 ? gla_chunk_add_kernel<T, 8> : gla_chunk_add_kernel<T, 16>;
-    const size_t lds = sizeof(float) * ((size_t)(D + VD) * kTS + 4 * D);
+    auto kern = wide <= 32 ? gla_chunk_add_kernel<T, 2> : wide <= 64 ? gla_chunk_add_kernel<T, 4>
+              : wide <= 128 ? gla_chunk_add_kernel<T, 8> : gla_chunk_add_kernel<T, 16>;
+    const size_t lds = sizeof(float) * ((size_t)D * kTS + 4 * D);
     if (int rc = room(reinterpret_cast<const void*>(kern), lds)) return rc;
     kern<<<grid, 256, lds, s>>>(proj, ld, low, w, workspace, seqs, sh);
     if (int rc = lsh_check_launch("gla_chunk_add_kernel")) return rc;
@@ -595,7 +619,6 @@ int gla_chunked(const T* proj, long ld, const float* low, const GlaWeights& w, f
   gla_chunk_state_kernel<<<dim3((VD * D / 4 + 255) / 256, sh.heads, n_seqs), 256, 0, s>>>(
       workspace, state, seqs, sh);
   if (int rc = lsh_check_launch("gla_chunk_state_kernel")) return rc;
-  const int wide = std::max(D, VD);
   auto kern = wide <= 32 ? gla_chunk_out_kernel<T, 2> : wide <= 64 ? gla_chunk_out_kernel<T, 4>
             : wide <= 128 ? gla_chunk_out_kernel<T, 8> : gla_chunk_out_kernel<T, 16>;
   const size_t lds = sizeof(float) * ((size_t)(kC + 48) * (D + 4) + kC * kTS + 4 * D + 4 * kC);
