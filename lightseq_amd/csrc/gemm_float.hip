@@ -309,8 +309,18 @@ gemm_skinny_kernel(GemmArgs a) {
   static_assert(!HALVES || MODE == kGated, "gate and up rows");
   constexpr int NB = is_up(MODE) && !HALVES ? 2 : NS;
   constexpr int V = FT<T>::kVec;
-  constexpr int U = 4;  // 64-byte slices per turn: 256 bytes of every row
-  __shared__ float red[NW][NB][MB][16][17];
+  // A turn takes U 64-byte slices of every row.  A wavefront loads whole lines, LR lanes to a row (a
+  // fragment's lanes are 16 rows apart from each other in memory: loaded as such they would cost a
+  // cache access each), and turns them into fragments in a part of LDS of its own.
+  constexpr int U = (NB + MB) * NW <= 12 ? 4 : 2;
+  constexpr int LR = 4 * U, RI = 64 / LR;        // lanes per row, rows per load
+  constexpr int LW = 16 * NB / RI, LA = 16 * MB / RI;  // loads of weights, of activations
+  constexpr int STR = U * 64 + 16;               // bytes from row to row in LDS
+  constexpr int STAGE = 16 * (NB + MB) * STR;
+  typedef float Red[NB][MB][16][17];
+  constexpr int LDS = NW * STAGE > NW * (int)sizeof(Red) ? NW * STAGE : NW * (int)sizeof(Red);
+  __shared__ __attribute__((aligned(16))) char smem[LDS];
+  Red* red = reinterpret_cast<Red*>(smem);
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int c = lane & 15, q = lane >> 4;
   const int n0 = blockIdx.x * (HALVES ? 8 : 16 * NS);
@@ -336,44 +346,61 @@ gemm_skinny_kernel(GemmArgs a) {
   }
   const T* W = reinterpret_cast<const T*>(a.W);
   if (!is_dense(MODE)) W += (long)rs.expert * NB * a.N * a.K;
-  const T* wrow[NB];
+  const int lr = lane / LR, lc = lane % LR;
+  const T* wrow[LW];
 #pragma unroll
-  for (int j = 0; j < NB; ++j)
-    wrow[j] = HALVES ? W + (long)(min(n0 + (c & 7), a.N - 1) + (c >> 3) * a.N) * a.K
-                     : W + (is_up(MODE) ? (long)(min(n0 + c, a.N - 1) + j * a.N)
-                                  : (long)min(n0 + j * 16 + c, a.N - 1)) * a.K;
+  for (int i = 0; i < LW; ++i) {
+    const int j = i * RI / 16, r = i * RI % 16 + lr;
+    wrow[i] = W + lc * V +
+              (HALVES ? (long)(min(n0 + (r & 7), a.N - 1) + (r >> 3) * a.N)
+                      : is_up(MODE) ? (long)(min(n0 + r, a.N - 1) + j * a.N)
+                                    : (long)min(n0 + j * 16 + r, a.N - 1)) * a.K;
+  }
   const T* A = reinterpret_cast<const T*>(a.A);
+  char* put = smem + wave * STAGE + lr * STR + lc * 16;
+  const char* get = smem + wave * STAGE + c * STR + q * 16;
   const int first_end = rs.last;
   for (int first = 0; first < first_end; first += 16 * MB) {
-    const T* arow[MB];
+    const T* arow[LA];
 #pragma unroll
-    for (int i = 0; i < MB; ++i)
-      arow[i] = A + src_row<MODE>(a, rs, first + i * 16 + c) * a.lda;
+    for (int i = 0; i < LA; ++i) arow[i] = A + src_row<MODE>(a, rs, first + i * RI + lr) * a.lda + lc * V;
     f32x4 acc[NB][MB];
 #pragma unroll
     for (int j = 0; j < NB; ++j)
 #pragma unroll
       for (int i = 0; i < MB; ++i) acc[j][i] = (f32x4)0.f;
-    for (int k = k_lo + wave * (U * 4 * V); k < k_hi; k += NW * U * 4 * V) {
-      frag_t fw[U][NB], fa[U][MB];
+    frag_t lw[LW], la[LA];
+    auto fetch = [&](int k) {
+      const bool in = k + lc * V < k_hi;
+#pragma unroll
+      for (int i = 0; i < LW; ++i) lw[i] = in ? *reinterpret_cast<const frag_t*>(wrow[i] + k) : (frag_t)0u;
+#pragma unroll
+      for (int i = 0; i < LA; ++i) la[i] = in ? *reinterpret_cast<const frag_t*>(arow[i] + k) : (frag_t)0u;
+    };
+    constexpr int STEP = NW * U * 4 * V;
+    int k = k_lo + wave * (U * 4 * V);
+    if (k < k_hi) fetch(k);
+    for (; k < k_hi; k += STEP) {
+#pragma unroll
+      for (int i = 0; i < LW; ++i) *reinterpret_cast<frag_t*>(put + i * RI * STR) = lw[i];
+#pragma unroll
+      for (int i = 0; i < LA; ++i) *reinterpret_cast<frag_t*>(put + (16 * NB + i * RI) * STR) = la[i];
+      if (k + STEP < k_hi) fetch(k + STEP);
 #pragma unroll
       for (int u = 0; u < U; ++u) {
-        const int kk = k + (u * 4 + q) * V;
-        const bool in = kk < k_hi;
+        frag_t fw[NB], fa[MB];
 #pragma unroll
-        for (int j = 0; j < NB; ++j)
-          fw[u][j] = in ? *reinterpret_cast<const frag_t*>(wrow[j] + kk) : (frag_t)0u;
+        for (int j = 0; j < NB; ++j) fw[j] = *reinterpret_cast<const frag_t*>(get + j * 16 * STR + u * 64);
 #pragma unroll
         for (int i = 0; i < MB; ++i)
-          fa[u][i] = in ? *reinterpret_cast<const frag_t*>(arow[i] + kk) : (frag_t)0u;
-      }
-#pragma unroll
-      for (int u = 0; u < U; ++u)
+          fa[i] = *reinterpret_cast<const frag_t*>(get + (NB + i) * 16 * STR + u * 64);
 #pragma unroll
         for (int j = 0; j < NB; ++j)
 #pragma unroll
-          for (int i = 0; i < MB; ++i) acc[j][i] = mma16(T{}, fw[u][j], fa[u][i], acc[j][i]);
+          for (int i = 0; i < MB; ++i) acc[j][i] = mma16(T{}, fw[j], fa[i], acc[j][i]);
+      }
     }
+    __syncthreads();  // the sums take the place of the operands
 #pragma unroll
     for (int j = 0; j < NB; ++j)
 #pragma unroll
