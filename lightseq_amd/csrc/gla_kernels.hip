@@ -174,8 +174,10 @@ gla_scan_kernel(const T* __restrict__ proj, long ld, const float* __restrict__ l
 }
 
 // ------------------------------------------------------------------------------------------------
-// Workspace of one (chunk, head): what the chunk adds to the state, then the state before it, [VD][D];
-// the chunk's decay [D].  Chunk c of a sequence is number row0 / 64 + sequence index + c.
+// Workspace of one (chunk, head): what the chunk adds to the state, then the state before it; the
+// chunk's decay [D].  Chunk c of a sequence is number row0 / 64 + sequence index + c.  The state is cut
+// into blocks of 16 x 16 (value block vb, slice s: number vb * (D / 16) + s), each as the lanes of a
+// wavefront hold it as an operand: lane (c, qd) value channel 16 vb + c, key channels 16 s + 4 qd .. + 3.
 __host__ __device__ inline long chunk_floats(const GlaShape& sh) {
   return (long)sh.vdim * sh.dim + sh.dim;
 }
@@ -309,7 +311,7 @@ gla_chunk_add_kernel(const T* __restrict__ proj, long ld, const float* __restric
       f32x4 acc = (f32x4)0.f;
 #pragma unroll
       for (int J = 0; J < 4; ++J) acc = mma16(0.f, fk[J], values.frag(b, J), acc);
-      *reinterpret_cast<f32x4*>(&o[(long)(vb * 16 + c) * D + db * 16 + qd * 4]) = acc;
+      *reinterpret_cast<f32x4*>(&o[(vb * ns + db) * 256 + lane * 4]) = acc;
     }
   }
 }
@@ -325,7 +327,9 @@ gla_chunk_state_kernel(float* __restrict__ ws, float* __restrict__ state,
   if (x >= size) return;
   const long stride = H * chunk_floats(sh);
   float* base = ws + ((sq.row0 / kC + (long)blockIdx.z) * H + h) * chunk_floats(sh);
-  float* sp = state + ((long)sq.slot * H + h) * size + x;
+  const int lane = x / 4 % 64, block = x / 256, ns = D / 16;
+  const int v = block / ns * 16 + lane % 16, d = block % ns * 16 + lane / 16 * 4;
+  float* sp = state + ((long)sq.slot * H + h) * size + (long)v * D + d;
   const int chunks = (sq.n + kC - 1) / kC;
   f32x4 S = (f32x4)0.f;
   if (sq.pos0 > 0) S = load4(sp);
@@ -335,7 +339,7 @@ gla_chunk_state_kernel(float* __restrict__ ws, float* __restrict__ state,
     for (int u = 0; u < U; ++u)
       if (ch + u < chunks) {
         add[u] = load4(base + (ch + u) * stride + x);
-        dec[u] = load4(base + (ch + u) * stride + size + x % D);
+        dec[u] = load4(base + (ch + u) * stride + size + d);
       }
 #pragma unroll
     for (int u = 0; u < U; ++u)
@@ -477,7 +481,7 @@ gla_chunk_out_kernel(const T* __restrict__ proj, long ld, const float* __restric
       frag_t fs[NS];
 #pragma unroll
       for (int s = 0; s < NS; ++s)
-        if (s < ns) fs[s] = ldfrag(S + (long)(vb * 16 + c) * D + s * 16 + qd * 4);
+        if (s < ns) fs[s] = ldfrag(S + (vb * ns + s) * 256 + lane * 4);
 #pragma unroll
       for (int s = 0; s < NS; ++s)
         if (s < ns) {

@@ -82,38 +82,57 @@ lm_norm_kernel(NormArgs a) {
       }
     rstd = 1.0f / sqrtf(block_sum_dpp(s, red[which + 1]) * inv_w + a.eps);
   };
-  auto add = [&](const AddPart& p0, int which) {
-    float y[NI][V];
+  // the sum of a summand's pieces, PU of them requested at a time
+  constexpr int PU = NI <= 2 ? 4 : NI <= 4 ? 2 : 1;
+  auto gather = [&](const AddPart& part, float (&y)[NI][V]) {
 #pragma unroll
     for (int i = 0; i < NI; ++i)
 #pragma unroll
       for (int k = 0; k < V; ++k) y[i][k] = 0.f;
-    const TY* yr = reinterpret_cast<const TY*>(p0.y) + r * p0.row_stride;
-    for (int p = 0; p < p0.parts; ++p) {
-      const float wt = p0.weight ? p0.weight[r * p0.parts + p] : 1.f;
+    const TY* yr = reinterpret_cast<const TY*>(part.y) + r * part.row_stride;
+    if (part.parts == 1 && !part.weight) {
 #pragma unroll
       for (int i = 0; i < NI; ++i) {
         const int c = (i * 256 + tid) * V;
-        if (c < W) {
-          float t[V];
-          ldv<V, TY>(yr + p * p0.part_stride + c, t);
+        if (c < W) ldv<V, TY>(yr + c, y[i]);
+      }
+      return;
+    }
+    for (int p0 = 0; p0 < part.parts; p0 += PU) {
+      float t[PU][NI][V], wt[PU];
 #pragma unroll
-          for (int k = 0; k < V; ++k) y[i][k] += wt * t[k];
+      for (int u = 0; u < PU; ++u) {
+        const bool there = p0 + u < part.parts;
+        wt[u] = there && part.weight ? part.weight[r * part.parts + p0 + u] : 1.f;
+#pragma unroll
+        for (int i = 0; i < NI; ++i) {
+          const int c = (i * 256 + tid) * V;
+#pragma unroll
+          for (int k = 0; k < V; ++k) t[u][i][k] = 0.f;
+          if (there && c < W) ldv<V, TY>(yr + (p0 + u) * part.part_stride + c, t[u][i]);
         }
       }
+#pragma unroll
+      for (int u = 0; u < PU; ++u)
+#pragma unroll
+        for (int i = 0; i < NI; ++i)
+#pragma unroll
+          for (int k = 0; k < V; ++k) y[i][k] += wt[u] * t[u][i][k];
     }
+  };
+  auto add = [&](const AddPart& part, const float (&y)[NI][V], int which) {
     float mean = 0.f, rstd = 1.f;
-    if (p0.post_w) stats(y, a.add.post_kind, mean, rstd, which);
+    if (part.post_w) stats(y, a.add.post_kind, mean, rstd, which);
 #pragma unroll
     for (int i = 0; i < NI; ++i) {
       const int c = (i * 256 + tid) * V;
       if (c < W) {
-        if (p0.post_w) {
+        if (part.post_w) {
           float w[V], b[V];
-          ldv<V, float>(p0.post_w + c, w);
+          ldv<V, float>(part.post_w + c, w);
 #pragma unroll
           for (int k = 0; k < V; ++k) b[k] = 0.f;
-          if (p0.post_b) ldv<V, float>(p0.post_b + c, b);
+          if (part.post_b) ldv<V, float>(part.post_b + c, b);
 #pragma unroll
           for (int k = 0; k < V; ++k) x[i][k] += a.add.scale * ((y[i][k] - mean) * rstd * w[k] + b[k]);
         } else {
@@ -123,8 +142,18 @@ lm_norm_kernel(NormArgs a) {
       }
     }
   };
-  if (a.add.parts > 0) add(a.add, 0);
-  if (a.add.second.parts > 0) add(a.add.second, 2);
+  if (a.add.parts > 0) {
+    float y[NI][V];
+    gather(a.add, y);
+    if (a.add.second.parts > 0) {
+      float z[NI][V];
+      gather(a.add.second, z);
+      add(a.add, y, 0);
+      add(a.add.second, z, 2);
+    } else {
+      add(a.add, y, 0);
+    }
+  }
   if (a.inject.any()) {
     const T* ir = embed_row(a.inject.ids);
 #pragma unroll
